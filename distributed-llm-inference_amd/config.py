@@ -36,7 +36,14 @@ class MixerSpec:
     the state multiplied by a tanh-GELU branch) or ``"gated_latent_attention"`` (latent attention whose queries come from a
     normed latent of size ``q_rank``: half-split rotation with optionally stretched frequencies, sliding ``window``, a
     per-head ``sink`` in the softmax denominator, an element-wise sigmoid output gate; ``kv_from`` ≥ 0: the layer reads that
-    layer's cached latents and rotated keys and expands them with its own matrices)."""
+    layer's cached latents and rotated keys and expands them with its own matrices), ``"delta"`` (gated delta rule: unit-length
+    q / k of ``kv_heads`` heads behind ``conv_taps``-tap convolutions, a decay and a write strength per head and token, a
+    ``[D, Dv]`` state per head), ``"mlstm"`` (matrix memory with exponential input and sigmoid forget gates soft-capped at
+    ``gate_cap``, a normaliser vector beside the ``[D, Dv]`` state and a running maximum per head), ``"conv_attention"``
+    (causal grouped-query attention whose q and k pass a convolution and half-split rotation; the values are the keys before
+    rotation; a per-head sink in the denominator), ``"ssd"`` (Mamba-2: ``heads`` heads of ``vdim`` channels over ``kv_heads``
+    groups of ``dim`` state columns, gate before a norm over ``norm_groups`` parts) or ``"normed_pair"`` (the two mixers in
+    ``parts`` read the same input; half the sum of their outputs, each RMS-normed over the width)."""
     kind: str
     heads: int
     dim: int                            # per-head query / key size (latent attention: the unrotated part)
@@ -49,7 +56,8 @@ class MixerSpec:
     rot_base: float = 10000.0
     rot_dims: int = 0                   # leading entries of the rotated part that are actually rotated
     decay: tuple = ()                   # lightning: per-head state decay
-    rot_scaling: tuple = ()             # sink / gated latent attention: (factor, original length, fast turns, slow turns) or ()
+    rot_scaling: tuple = ()             # sink / gated latent attention: (factor, original length, fast turns, slow turns) or ();
+                                        # conv attention: (factor, original length, high, low)
     lora: int = 0                       # time mix: rank of the decay projection
     parts: tuple = ()                   # parallel: the mixers run side by side (MixerSpec each)
     part_scales: tuple = ()             # parallel: weight of every part's output
@@ -61,18 +69,22 @@ class MixerSpec:
     shared_ff: int = 0                  # moe: inner width of the expert every token takes (0: none)
     kv_from: int = -1                   # gated (latent) attention: index of the layer whose cached rows this layer reads (-1: its own)
     ff_act: str = "relu2"               # feed-forward activation: "relu2" | "gelu_tanh" / "silu" (gated) | "clamped" (gated experts)
+                                        # | "gelu_tanh_plain" (not gated)
     router: str = "sigmoid"             # moe: "sigmoid" (scores, not renormalised) | "softmax" (biased logits, softmax over the chosen)
                                         # | "softmax_all" (softmax over all logits, a choice bias, renormalised over the chosen)
     q_rank: int = 0                     # gated latent attention: size of the normed query latent
     sink: bool = False                  # gated latent attention: a learned per-head logit in the softmax denominator
-    conv_taps: int = 0                  # rglru: taps of the causal convolution in front of the recurrence
+    conv_taps: int = 0                  # rglru, delta, ssd, conv attention: taps of the causal convolution behind the projections
     identity_experts: int = 0           # moe ("softmax_all"): trailing router outputs whose expert returns its input
     ff_limit: float = 0.0               # moe ("clamped" experts): bound of the gate (above) and of the up projection (both sides)
     ff_bias: bool = False               # dense feed-forward: the three projections have biases
+    gate_cap: float = 0.0               # mlstm: soft bound of the gates' pre-activations
+    norm_groups: int = 1                # ssd: equal parts of the inner width that are normed on their own
 
     @property
     def stateful(self) -> bool:
-        return self.kind in ("lightning", "time_mix", "retention", "rglru") or any(p.stateful for p in self.parts)
+        return (self.kind in ("lightning", "time_mix", "retention", "rglru", "delta", "mlstm", "ssd", "conv_attention")
+                or any(p.stateful for p in self.parts))
 
     @property
     def cache_row(self) -> tuple:
@@ -80,7 +92,9 @@ class MixerSpec:
         one row (latent | rotated key) that serves as both; a recurrent one keeps none."""
         if self.kind in ("attention", "sink_attention") or (self.kind == "gated_attention" and self.kv_from < 0):
             return self.kv_heads * self.dim, self.kv_heads * self.vdim
-        if self.kind == "parallel":
+        if self.kind == "conv_attention":
+            return self.kv_heads * self.dim, self.kv_heads * self.dim
+        if self.kind in ("parallel", "normed_pair"):
             return tuple(sum(w) for w in zip(*(p.cache_row for p in self.parts)))
         if self.kind == "latent_attention" or (self.kind == "gated_latent_attention" and self.kv_from < 0):
             return self.kv_rank + self.rot_dim, 0
@@ -88,11 +102,13 @@ class MixerSpec:
 
     @property
     def state_shape(self) -> tuple:
-        if self.kind == "parallel":
+        if self.kind in ("parallel", "normed_pair"):
             return next((p.state_shape for p in self.parts if p.state_shape), ())
+        if self.kind == "mlstm":                # the state's columns, then the normaliser
+            return (self.heads, self.dim * (self.vdim + 1))
         if self.kind == "rglru":
             return (self.heads * self.dim,)
-        return (self.heads, self.dim, self.vdim) if self.kind in ("lightning", "time_mix", "retention") else ()
+        return (self.heads, self.dim, self.vdim) if self.kind in ("lightning", "time_mix", "retention", "delta", "ssd") else ()
 
 
 @dataclass
@@ -161,6 +177,8 @@ class ModelConfig:
         h, i, v, l = self.hidden_size, self.intermediate_size, self.vocab_size, self.num_layers
         if self.arch == "sevelorn":
             return 2 * v * h + h + sum(_hyper_layer_params(m, h, self.streams, self.conv_taps) for m in self.layer_specs)
+        if self.arch == "nefarax":
+            return v * h + 2 * h + 1 + sum(_nefarax_layer_params(m, h) for m in self.layer_specs)
         if self.arch == "sinilorn":
             return 2 * v * h + h + sum(_sinilorn_layer_params(m, h, self.streams) for m in self.layer_specs)
         if self.layer_specs:
@@ -231,6 +249,21 @@ def _sinilorn_layer_params(m: MixerSpec, h: int, streams: int) -> int:
         n_out = m.experts + m.identity_experts
         tot += h + hc + (m.experts * 3 * h * m.ff + n_out * (h + 1) if m.ff_kind == "moe" else 3 * h * m.ff + 2 * m.ff + h)
     return tot
+
+
+def _nefarax_layer_params(m: MixerSpec, h: int) -> int:
+    """Parameters of one Nefarax layer (its one norm, mixer, feed-forward)."""
+    tot = 2 * h + 1 + 2 * h * m.ff
+    if m.kind == "delta":
+        qk, v = m.kv_heads * m.dim, m.heads * m.vdim
+        return tot + h * (2 * qk + 3 * v + 2 * m.heads) + m.conv_taps * (2 * qk + v) + 2 * m.heads + m.vdim
+    if m.kind == "mlstm":
+        return tot + h * m.heads * (2 * m.dim + 3 * m.vdim + 2) + 2 * m.heads + m.heads * m.vdim
+    a, b = m.parts
+    ca, inner = (a.heads + a.kv_heads) * a.dim, b.heads * b.vdim
+    cb = inner + 2 * b.kv_heads * b.dim
+    return (tot + 2 * h + ca * (h + a.conv_taps) + a.heads + h * a.heads * a.dim
+            + h * (inner + cb + b.heads) + cb * (b.conv_taps + 1) + 3 * b.heads + inner + h * inner)
 
 
 def _rodelix_spec(entry: dict) -> MixerSpec:
@@ -416,7 +449,61 @@ def sinilorn_config(cfg: dict, name: str = "sinilorn", dtype: str = "bfloat16") 
                        stream_norm="layer", logit_scale=float(cfg.get("logit_scale", 1.0)))
 
 
-_CONFIG_READERS = {"Rodelix": rodelix_config, "Vibunex": vibunex_config, "Sevelorn": sevelorn_config, "Sinilorn": sinilorn_config}
+def _nefarax_spec(entry: dict, index: int) -> MixerSpec:
+    m, mlp = entry["mixer"], entry.get("mlp")
+    kind = entry["type"]
+
+    def need(ok, what):
+        if not ok:
+            raise ValueError(f"layer {index}: {what}")
+
+    ff = {}
+    if mlp:
+        need(mlp.get("kind") == "dense", f"unknown feed-forward kind {mlp.get('kind')!r}")
+        ff = dict(ff=int(mlp["ff"]), ff_kind="dense", ff_act="gelu_tanh_plain")
+    if kind == "delta":
+        spec = MixerSpec(kind="delta", heads=int(m["heads"]), kv_heads=int(m["kv_heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]),
+                         conv_taps=int(m["conv"]), **ff)
+        need(spec.heads % spec.kv_heads == 0, f"{spec.heads} heads over {spec.kv_heads} query/key heads")
+        need(spec.conv_taps >= 1, "a convolution has at least the current token's tap")
+        return spec
+    if kind == "mlstm":
+        spec = MixerSpec(kind="mlstm", heads=int(m["heads"]), kv_heads=int(m["heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]),
+                         gate_cap=float(m["gate_cap"]), **ff)
+        need(spec.gate_cap > 0.0, "the gates need a positive cap")
+        return spec
+    need(kind == "parallel", f"unknown mixer type {kind!r}")
+    a, b = m["left"], m["right"]
+    rot = a.get("rot") or {}
+    sc = rot.get("scaling")
+    left = MixerSpec(kind="conv_attention", heads=int(a["heads"]), kv_heads=int(a["kv_heads"]), dim=int(a["dim"]), vdim=int(a["dim"]),
+                     scale=float(a["scale"]), conv_taps=int(a["conv"]), sink=True, rot_base=float(rot.get("base", 10000.0)),
+                     rot_dims=int(rot.get("dims", 0)),
+                     rot_scaling=(float(sc["factor"]), float(sc["original"]), float(sc["high"]), float(sc["low"])) if sc else ())
+    right = MixerSpec(kind="ssd", heads=int(b["heads"]), kv_heads=int(b["groups"]), dim=int(b["state"]), vdim=int(b["vdim"]),
+                      conv_taps=int(b["conv"]), norm_groups=int(b["norm_groups"]))
+    need(int(a.get("vdim", left.dim)) == left.dim, f"values of {a.get('vdim')} entries cannot be the keys of {left.dim}")
+    need(left.heads % left.kv_heads == 0, f"{left.heads} query heads over {left.kv_heads} key/value heads")
+    need(left.rot_dims % 2 == 0 and left.rot_dims <= left.dim, f"{left.rot_dims} rotated entries of {left.dim}")
+    need(right.heads % right.kv_heads == 0, f"{right.heads} heads over {right.kv_heads} groups")
+    need(right.heads * right.vdim % right.norm_groups == 0, f"{right.heads * right.vdim} channels in {right.norm_groups} norm groups")
+    need(min(left.conv_taps, right.conv_taps) >= 1, "a convolution has at least the current token's tap")
+    return MixerSpec(kind="normed_pair", heads=left.heads, dim=left.dim, vdim=left.vdim, kv_heads=left.kv_heads, parts=(left, right), **ff)
+
+
+def nefarax_config(cfg: dict, name: str = "nefarax", dtype: str = "bfloat16") -> ModelConfig:
+    """``ModelConfig`` of a Nefarax checkpoint from the dict its ``config.json`` holds."""
+    specs = tuple(_nefarax_spec(e, i) for i, e in enumerate(cfg["layers"]))
+    att = next((s for s in specs if s.kind == "normed_pair"), specs[0])
+    return ModelConfig(name=name, arch="nefarax", vocab_size=int(cfg["vocab"]), hidden_size=int(cfg["width"]),
+                       intermediate_size=max([s.ff for s in specs] + [0]), num_layers=len(specs), num_heads=att.heads,
+                       num_kv_heads=max(att.kv_heads, 1), head_dim=att.dim, max_position=1 << 24, rms_eps=float(cfg["norm"]["eps"]),
+                       dtype=dtype, bos_token_id=0, eos_token_id=-1, layer_specs=specs, tie_embeddings=True,
+                       residual_mult=float(cfg.get("residual_mult", 1.0)))
+
+
+_CONFIG_READERS = {"Rodelix": rodelix_config, "Vibunex": vibunex_config, "Sevelorn": sevelorn_config, "Sinilorn": sinilorn_config,
+                   "Nefarax": nefarax_config}
 
 
 def safetensors_shapes(path: str) -> dict:
@@ -560,6 +647,18 @@ MODEL_PRESETS: dict[str, ModelConfig] = {
              "mixer": {"heads": 2, "dim": 24, "rot_dim": 8, "vdim": 16, "kv_rank": 32, "q_rank": 24, "scale": 0.25, "kv_from": 0,
                        "rot": {"base": 5000.0, "dims": 8, "scaling": {"factor": 2.0, "original": 64, "fast": 16.0, "slow": 2.0}}}}]},
         name="tiny-sinilorn", dtype="float32"),
+    # one tanh norm per layer in front of mixer and feed-forward side by side: gated delta rule, mLSTM, and attention beside a
+    # Mamba-2 recurrence; tied embeddings
+    "tiny-nefarax": nefarax_config({
+        "vocab": 304, "width": 80, "residual_mult": 0.7, "norm": {"eps": 1e-5},
+        "layers": [
+            {"type": "delta", "mlp": {"kind": "dense", "ff": 96}, "mixer": {"heads": 4, "kv_heads": 2, "dim": 16, "vdim": 24, "conv": 3}},
+            {"type": "mlstm", "mlp": {"kind": "dense", "ff": 64}, "mixer": {"heads": 3, "dim": 16, "vdim": 32, "gate_cap": 12.0}},
+            {"type": "parallel", "mlp": None,
+             "mixer": {"left": {"heads": 4, "kv_heads": 2, "dim": 16, "vdim": 16, "conv": 2, "scale": 0.3,
+                                "rot": {"base": 10000.0, "dims": 8, "scaling": {"factor": 4.0, "high": 4.0, "low": 1.0, "original": 64}}},
+                       "right": {"heads": 3, "vdim": 16, "state": 24, "groups": 1, "conv": 4, "norm_groups": 2}}}]},
+        name="tiny-nefarax", dtype="float32"),
     "tiny-opt": ModelConfig(name="tiny-opt", arch="opt", vocab_size=512, hidden_size=64,
                             intermediate_size=128, num_layers=2, num_heads=4, num_kv_heads=4,
                             head_dim=16, max_position=512, pos_offset=2, tie_embeddings=True,

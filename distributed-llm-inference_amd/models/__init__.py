@@ -17,6 +17,7 @@ from ..config import ModelConfig
 from ..parallel.state import SINGLE, ParallelContext
 from .layers import random_full_tensor
 from .llama import LlamaForCausalLM
+from .nefarax import NefaraxForCausalLM
 from .opt import OPTForCausalLM
 from .rodelix import RodelixForCausalLM
 from .sevelorn import SevelornForCausalLM
@@ -24,7 +25,8 @@ from .sinilorn import SinilornForCausalLM
 from .vibunex import VibunexForCausalLM
 
 _ARCH = {"llama": LlamaForCausalLM, "mixtral": LlamaForCausalLM, "opt": OPTForCausalLM, "rodelix": RodelixForCausalLM,
-         "vibunex": VibunexForCausalLM, "sevelorn": SevelornForCausalLM, "sinilorn": SinilornForCausalLM}
+         "vibunex": VibunexForCausalLM, "sevelorn": SevelornForCausalLM, "sinilorn": SinilornForCausalLM,
+         "nefarax": NefaraxForCausalLM}
 
 
 def torch_dtype(name: str) -> torch.dtype:
@@ -123,7 +125,9 @@ def load_safetensors(model, path: str) -> None:
     for name, w, _kind in model.named_weights():
         if fused is not None:                                # the model names its checkpoint tensors itself
             keys = fused.get(name, [name])
-            if isinstance(keys[0], (list, tuple)):                   # stacked: one slice per entry (each a concatenation)
+            if keys[0] == "@cols":                                   # matrices side by side: concatenated along their columns
+                full = torch.cat([shards.get(k) for k in keys[1:]], dim=1)
+            elif isinstance(keys[0], (list, tuple)):                   # stacked: one slice per entry (each a concatenation)
                 full = torch.stack([shards.cat(ks) for ks in keys])
             else:
                 full = shards.cat(keys)

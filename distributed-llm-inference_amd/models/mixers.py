@@ -37,6 +37,18 @@ experts chosen by softmax scores plus a correction) are the feed-forwards of ``H
 the fp32 stream: every sublayer reads a weighted sum of them through a norm (RMS with ``1 + w`` weights, or a layer norm
 without bias; the mixer optionally also through a short causal convolution over time) and writes back through a mixing matrix.
 
+* ``DeltaRule`` – gated delta rule: unit-length q / k behind short convolutions, a decay and a write strength per head and
+  token; every write first subtracts what the key already reads from the ``[D, Dv]`` fp32 state;
+* ``MatrixMemory`` – mLSTM: exponential input gate, sigmoid forget gate, a running maximum that keeps both in range and a
+  normaliser vector beside the ``[D, Dv]`` fp32 state;
+* ``ConvAttention`` – causal grouped-query attention with convolved, half-split-rotated q / k, the unrotated keys as values
+  and a per-head sink in the softmax denominator;
+* ``StateSpace`` – Mamba-2: ``[N, Dv]`` fp32 state per head, B / C shared by groups of heads, gate before a grouped norm;
+* ``NormedPair`` – the last two on the same input, their outputs RMS-normed and averaged.
+
+``SingleNormLayer`` runs one of these five and an optional tanh-GELU feed-forward on the same norm ``tanh(α x) · w + b`` of
+the stream: ``x += m · (mixer(h) + ff(h))`` — one input GEMM and, but for the pair, one output GEMM for both.
+
 ``MixerLayer`` wraps one of the first three (and an optional dense feed-forward) in the sandwich
 ``x += m · norm_b(sublayer(norm(x)))`` with token shift in front of the mixer.  The residual stream ``x`` is
 fp32; GEMM operands are the model dtype.  Tensor parallelism is not implemented for these stacks.
@@ -59,13 +71,20 @@ from .layers import Weight
 @dataclass
 class LayerCache:
     """What one layer run keeps between steps: token-major pages (``k`` / ``v``; latent attention: ``k`` only), the
-    recurrent ``state`` rows and the token-shift rows ``shift`` (previous token's normed input) — the latter two indexed
-    by state slot."""
+    recurrent ``state`` rows, the token-shift rows ``shift`` (previous token's normed input, or a convolution's last inputs) and
+    further per-sequence values ``aux`` — the latter three indexed by state slot.  Mixers side by side keep theirs in ``parts``."""
     k: Optional[torch.Tensor] = None
     v: Optional[torch.Tensor] = None
     state: Optional[torch.Tensor] = None
     shift: Optional[torch.Tensor] = None
     owns_pages: bool = True             # False: ``k`` / ``v`` are another layer's pages (a mixer without keys / values of its own)
+    aux: Optional[torch.Tensor] = None
+    parts: tuple = ()
+
+    def state_tensors(self) -> list:
+        """Every tensor indexed by state slot."""
+        own = [t for t in (self.state, self.shift, self.aux) if t is not None]
+        return own + [t for p in self.parts for t in p.state_tensors()]
 
 
 def _param(shape, ctx, device) -> Weight:
@@ -505,9 +524,211 @@ class GatedLatentAttention(nn.Module):
         return ops.linear(seqmix.gate_heads(out, both[:, nq + nkv:nq + nkv + ng]), self.o.data)
 
 
+class DeltaRule(nn.Module):
+    """Per head: ``S ← g S``, ``u = β (v - Sᵀ k)``, ``S ← S + k uᵀ``, ``o = Sᵀ q`` (``g``, ``β`` per token); each head's ``o`` divided by its
+    root mean square, times a weight shared by the heads, times ``silu(W_g h)``.
+
+    The mixers of ``SingleNormLayer`` read their columns ``proj`` of the layer's one input GEMM (``in_sources``: the checkpoint
+    tensors of its rows, in order) and write the ``out_cols`` activations in front of their output projection into ``out``."""
+
+    def __init__(self, spec: MixerSpec, width: int, eps: float, ctx: ParallelContext, dtype, device):
+        super().__init__()
+        self.s, self.eps = spec, eps
+        H, G, D, Dv, taps = spec.heads, spec.kv_heads, spec.dim, spec.vdim, spec.conv_taps
+        self.conv_cols = 2 * G * D + H * Dv
+        self.in_cols, self.out_cols = self.conv_cols + H * Dv + 2 * H, H * Dv               # q | k | v | output gate | β | decay
+        self.conv = _param((self.conv_cols, taps), ctx, device)
+        self.A_log, self.dt_bias, self.norm = _param((H,), ctx, device), _param((H,), ctx, device), _param((Dv,), ctx, device)
+        self._taps = self._rate = None                                                      # derived at first use (after loading)
+
+    def in_sources(self, p):
+        return [p + c for c in "qkvgba"]
+
+    def weights(self, p):
+        yield p + "conv", self.conv, "small", [p + "q.conv", p + "k.conv", p + "v.conv"]
+        yield p + "A_log", self.A_log, "zeros", None
+        yield p + "dt_bias", self.dt_bias, "zeros", None
+        yield p + "norm", self.norm, "ones", None
+
+    def cache(self, num_blocks, num_slots, dtype, device) -> LayerCache:
+        s = self.s
+        return LayerCache(state=torch.zeros(num_slots, *s.state_shape, dtype=torch.float32, device=device),
+                          shift=torch.zeros(num_slots, s.conv_taps - 1, self.conv_cols, dtype=torch.float32, device=device))
+
+    def forward(self, proj, out, meta, cache: LayerCache):
+        s = self.s
+        H, G, D, Dv, C = s.heads, s.kv_heads, s.dim, s.vdim, self.conv_cols
+        if self._taps is None:
+            self._taps, self._rate = self.conv.data.t().contiguous(), torch.exp(self.A_log.data)
+        ga = C + H * Dv
+        qkv, decay, beta = seqmix.causal_conv(proj[:, :C], self._taps, None, cache.shift, meta, torch.float32, act="silu",
+                                              unit=(2 * G, D, G, D ** -0.5),
+                                              gates=("delta", proj[:, ga:ga + 2 * H], self._rate, self.dt_bias.data))
+        o, _ = seqmix.gated_scan(qkv[:, :G * D], qkv[:, G * D:2 * G * D], qkv[:, 2 * G * D:], decay, beta, cache.state, meta,
+                                 H, G, D, Dv, delta=True)
+        seqmix.rms_gate(o, self.norm.data, self.eps, proj[:, C:ga], out.dtype, groups=H, gate_act="silu", out=out,
+                        token_seq=meta.token_seq)
+
+
+class MatrixMemory(nn.Module):
+    """Log gates ``i = cap · tanh((W_i h + b) / cap)``, ``f = logsigmoid(cap · tanh((W_f h + b) / cap))``; ``m ← max(f + m, i)`` from zero;
+    ``S ← exp(f + m' - m) S + exp(i - m) k vᵀ`` (``m'``: the maximum before), ``n`` likewise with ``k``; ``o = Sᵀ q / (max(|n · q|, exp(-m)) + 1e-6)``;
+    per-head root mean square, weight, ``sigmoid(W_g h)``.  In and out columns as for ``DeltaRule``."""
+
+    def __init__(self, spec: MixerSpec, width: int, eps: float, ctx: ParallelContext, dtype, device):
+        super().__init__()
+        self.s, self.eps = spec, eps
+        H, D, Dv = spec.heads, spec.dim, spec.vdim
+        self.in_cols, self.out_cols = 2 * H * D + 2 * H * Dv + 2 * H, H * Dv                 # q | k | v | output gate | i | f
+        self.gate_b, self.norm = _param((2 * H,), ctx, device), _param((H * Dv,), ctx, device)
+
+    def in_sources(self, p):
+        return [p + c for c in "qkvgif"]
+
+    def weights(self, p):
+        yield p + "gates.b", self.gate_b, "zeros", [p + "i.b", p + "f.b"]
+        yield p + "norm", self.norm, "ones", None
+
+    def cache(self, num_blocks, num_slots, dtype, device) -> LayerCache:
+        return LayerCache(state=torch.zeros(num_slots, *self.s.state_shape, dtype=torch.float32, device=device),
+                          aux=torch.zeros(num_slots, self.s.heads, dtype=torch.float32, device=device))     # the running maximum
+
+    def forward(self, proj, out, meta, cache: LayerCache):
+        s = self.s
+        H, D, Dv = s.heads, s.dim, s.vdim
+        HD, gg = H * D, 2 * H * D + H * Dv
+        keep, write, floor = seqmix.max_gates(proj[:, gg + H * Dv:], self.gate_b.data, s.gate_cap, cache.aux, meta)
+        o, nq = seqmix.gated_scan(proj[:, :HD], proj[:, HD:2 * HD], proj[:, 2 * HD:gg], keep, write, cache.state, meta, H, H, D, Dv,
+                                  q_scale=D ** -0.5, normaliser=True)
+        seqmix.rms_gate(o, self.norm.data, self.eps, proj[:, gg:gg + H * Dv], out.dtype, groups=H, out=out, divide=(nq, floor),
+                        token_seq=meta.token_seq)
+
+
+class ConvAttention(nn.Module):
+    """Attention half of ``NormedPair``: reads its columns ``[q | k]`` of the layer's input GEMM, returns ``W_o`` of the heads."""
+
+    def __init__(self, spec: MixerSpec, width: int, eps: float, ctx: ParallelContext, dtype, device):
+        super().__init__()
+        self.s = spec
+        H, G, D = spec.heads, spec.kv_heads, spec.dim
+        self.in_cols = (H + G) * D
+        self.conv = _param((self.in_cols, spec.conv_taps), ctx, device)
+        self.sink = _param((H,), ctx, device)
+        self.o = _matrix(width, H * D, ctx, dtype, device)
+        self._taps = None
+        self.register_buffer("inv_freq", seqmix.banded_inv_freq(spec.rot_base, spec.rot_dims, spec.rot_scaling, device), persistent=False)
+
+    def in_sources(self, p):
+        return [p + "q", p + "k"]
+
+    def weights(self, p):
+        yield p + "conv", self.conv, "small", [p + "q.conv", p + "k.conv"]
+        yield p + "sink", self.sink, "zeros", None
+        yield p + "o", self.o, "normal", None
+
+    def cache(self, num_blocks, num_slots, dtype, device) -> LayerCache:
+        s = self.s
+        rows = (num_blocks, KV_BLOCK_SIZE, s.kv_heads * s.dim)
+        return LayerCache(k=torch.zeros(rows, dtype=dtype, device=device), v=torch.zeros(rows, dtype=dtype, device=device),
+                          shift=torch.zeros(num_slots, s.conv_taps - 1, self.in_cols, dtype=torch.float32, device=device))
+
+    def forward(self, proj, meta, cache: LayerCache):
+        s = self.s
+        H, G, D = s.heads, s.kv_heads, s.dim
+        T = proj.shape[0]
+        if self._taps is None:
+            self._taps = self.conv.data.t().contiguous()
+        q = seqmix.conv_rope_cache(proj, self._taps, cache.shift, meta, self.inv_freq, s.rot_dims, cache.k, cache.v, H, G, D)
+        out = torch.zeros(T, H, D, dtype=proj.dtype, device=proj.device)        # padding rows of a captured step stay zero
+        seqmix.token_attention(out, q.view(T, H, D), None, cache.k, cache.v, meta, G, D, s.scale, sink=self.sink.data)
+        return ops.linear(out.view(T, H * D), self.o.data)
+
+
+class StateSpace(nn.Module):
+    """Recurrent half of ``NormedPair``: columns ``[z | x | B | C | dt]`` of the layer's input GEMM; ``x``, ``B``, ``C`` through a biased
+    convolution and silu; ``dt = softplus(dt + bias)``; per head ``S ← exp(-exp(A_log) dt) S + dt B xᵀ``, ``y = Sᵀ C + D x``; ``y · silu(z)``
+    normed in ``norm_groups`` parts, times a weight, through ``W_o``."""
+
+    def __init__(self, spec: MixerSpec, width: int, eps: float, ctx: ParallelContext, dtype, device):
+        super().__init__()
+        self.s, self.eps = spec, eps
+        H, G, N, Dv = spec.heads, spec.kv_heads, spec.dim, spec.vdim
+        self.inner, self.conv_cols = H * Dv, H * Dv + 2 * G * N
+        self.in_cols = self.inner + self.conv_cols + H
+        self.conv, self.conv_b = _param((self.conv_cols, spec.conv_taps), ctx, device), _param((self.conv_cols,), ctx, device)
+        self.dt_bias, self.A_log, self.skip = (_param((H,), ctx, device) for _ in range(3))
+        self.norm = _param((self.inner,), ctx, device)
+        self.o = _matrix(width, self.inner, ctx, dtype, device)
+        self._taps = self._rate = None
+
+    def in_sources(self, p):
+        return [p + "in"]
+
+    def weights(self, p):
+        yield p + "conv", self.conv, "small", None
+        yield p + "conv.b", self.conv_b, "zeros", None
+        yield p + "dt_bias", self.dt_bias, "zeros", None
+        yield p + "A_log", self.A_log, "zeros", None
+        yield p + "D", self.skip, "ones", None
+        yield p + "norm", self.norm, "ones", None
+        yield p + "o", self.o, "normal", None
+
+    def cache(self, num_blocks, num_slots, dtype, device) -> LayerCache:
+        s = self.s
+        return LayerCache(state=torch.zeros(num_slots, *s.state_shape, dtype=torch.float32, device=device),
+                          shift=torch.zeros(num_slots, s.conv_taps - 1, self.conv_cols, dtype=torch.float32, device=device))
+
+    def forward(self, proj, meta, cache: LayerCache):
+        s = self.s
+        H, G, N, Dv, inner = s.heads, s.kv_heads, s.dim, s.vdim, self.inner
+        if self._taps is None:
+            self._taps, self._rate = self.conv.data.t().contiguous(), torch.exp(self.A_log.data)
+        C = self.conv_cols
+        xbc, decay, dt = seqmix.causal_conv(proj[:, inner:inner + C], self._taps, self.conv_b.data, cache.shift, meta, torch.float32,
+                                            act="silu", gates=("ssd", proj[:, inner + C:], self._rate, self.dt_bias.data))
+        x, B, Cc = xbc[:, :inner], xbc[:, inner:inner + G * N], xbc[:, inner + G * N:]
+        y, _ = seqmix.gated_scan(Cc, B, x, decay, dt, cache.state, meta, H, G, N, Dv)
+        y = seqmix.rms_gate(y, self.norm.data, self.eps, proj[:, :inner], proj.dtype, groups=s.norm_groups, gate_act="silu",
+                            skip=(x, self.skip.data), gate_first=True, token_seq=meta.token_seq)
+        return ops.linear(y, self.o.data)
+
+
+class NormedPair(nn.Module):
+    """``½ (rms(left(h)) · w_l + rms(right(h)) · w_r)``; ``forward`` returns both outputs before their norms (the layer's next residual
+    update applies norms, weights and the half in fp32)."""
+    out_cols = 0                # its halves have output projections of their own
+
+    def __init__(self, spec: MixerSpec, width: int, eps: float, ctx: ParallelContext, dtype, device):
+        super().__init__()
+        kinds = tuple(p.kind for p in spec.parts)
+        if kinds != ("conv_attention", "ssd"):
+            raise ValueError(f"the normed pair is convolved attention beside a state-space mixer, not {kinds}")
+        self.left = ConvAttention(spec.parts[0], width, eps, ctx, dtype, device)
+        self.right = StateSpace(spec.parts[1], width, eps, ctx, dtype, device)
+        self.left_w, self.right_w = _param((width,), ctx, device), _param((width,), ctx, device)
+        self.in_cols = self.left.in_cols + self.right.in_cols
+
+    def in_sources(self, p):
+        return self.left.in_sources(p + "left.") + self.right.in_sources(p + "right.")
+
+    def weights(self, p):
+        yield from self.left.weights(p + "left.")
+        yield from self.right.weights(p + "right.")
+        yield p + "left.out", self.left_w, "ones", None
+        yield p + "right.out", self.right_w, "ones", None
+
+    def cache(self, num_blocks, num_slots, dtype, device) -> LayerCache:
+        return LayerCache(parts=tuple(m.cache(num_blocks, num_slots, dtype, device) for m in (self.left, self.right)))
+
+    def forward(self, proj, meta, cache: LayerCache):
+        n = self.left.in_cols
+        return self.left(proj[:, :n], meta, cache.parts[0]), self.right(proj[:, n:], meta, cache.parts[1])
+
+
 MIXERS = {"gated_attention": GatedAttention, "retention": Retention, "attention": WindowAttention, "latent_attention": LatentAttention, "lightning": LightningAttention,
           "sink_attention": SinkTalkAttention, "time_mix": TimeMix, "parallel": DualMixer, "rglru": GatedLinearRecurrence,
-          "gated_latent_attention": GatedLatentAttention}
+          "gated_latent_attention": GatedLatentAttention, "delta": DeltaRule, "mlstm": MatrixMemory, "conv_attention": ConvAttention,
+          "ssd": StateSpace, "normed_pair": NormedPair}
 
 
 class DenseFF(nn.Module):
@@ -725,6 +946,71 @@ class HyperLayer(nn.Module):
         h2 = seqmix.stream_mix_norm(x, y, self.hc1.mix.data, self.hc1.w_out.data, self.hc2.w_in.data, self.norm2.data, self.eps,
                                     self.w_offset, self.dtype, self.center)
         return self.ff(h2), self.hc2
+
+
+class TanhNorm(nn.Module):
+    """``tanh(α x) · w + b`` with a scalar ``α``: no statistics of the row."""
+
+    def __init__(self, n: int, ctx, device):
+        super().__init__()
+        self.alpha, self.w, self.b = _param((1,), ctx, device), _param((n,), ctx, device), _param((n,), ctx, device)
+
+    def weights(self, p):
+        yield p, self.w, "ones", None
+        yield p + ".b", self.b, "zeros", None
+        yield p + ".alpha", self.alpha, "half", None
+
+    def read(self, x, pending, mult: float, eps: float, out_dtype):
+        """``x += mult · pending`` (the previous layer's output, see ``SingleNormLayer``), then the norm of ``x``."""
+        y, pair = pending if pending is not None else (None, None)
+        return seqmix.residual_tanh_norm(x, y, pair, mult, self.alpha.data, self.w.data, self.b.data, eps, out_dtype)
+
+
+class SingleNormLayer(nn.Module):
+    """``x += m · (mixer(h) + W_down gelu_tanh(W_up h))`` with ``h = tanh_norm(x)``.  The rows of every projection that reads ``h`` — the
+    feed-forward's and the mixer's — are one GEMM; where the mixer's output projection adds straight into the sum, it and
+    ``W_down`` are one GEMM over both activations side by side as well.  ``forward`` returns ``(y, pair)``: what the next
+    ``TanhNorm.read`` adds — ``y`` (None: nothing) and, for ``NormedPair``, the two outputs still to be normed and averaged."""
+    ALIGN = 16                  # the fused projection's rows are padded to a multiple of this (the decode GEMM's tile)
+
+    def __init__(self, spec: MixerSpec, width: int, eps: float, ctx: ParallelContext, dtype, device):
+        super().__init__()
+        self.spec, self.ff = spec, spec.ff
+        if spec.ff and (spec.ff_kind, spec.ff_act) != ("dense", "gelu_tanh_plain"):
+            raise ValueError(f"single-norm layers take a dense tanh-GELU feed-forward, not {spec.ff_kind!r} / {spec.ff_act!r}")
+        self.norm1 = TanhNorm(width, ctx, device)
+        self.mixer = MIXERS[spec.kind](spec, width, eps, ctx, dtype, device)
+        used = spec.ff + self.mixer.in_cols
+        self.pad = -used % self.ALIGN
+        self.inp = _matrix(used + self.pad, width, ctx, dtype, device)                      # feed-forward | mixer | alignment rows
+        self.fused_out = self.mixer.out_cols > 0
+        k = self.mixer.out_cols + spec.ff
+        self.out = _matrix(width, k, ctx, dtype, device) if k else None
+
+    def weights(self, p):
+        yield from self.norm1.weights(p + "norm1")
+        up = [p + "mlp.up"] if self.ff else []
+        yield p + "in", self.inp, "normal", up + self.mixer.in_sources(p + "mix.") + ([f"@zeros:{self.pad}"] if self.pad else [])
+        yield from self.mixer.weights(p + "mix.")
+        if self.out is not None:
+            cols = ([p + "mix.o"] if self.fused_out else []) + ([p + "mlp.down"] if self.ff else [])
+            yield p + "out", self.out, "normal", ["@cols"] + cols
+
+    def cache(self, num_blocks, num_slots, dtype, device) -> LayerCache:
+        return self.mixer.cache(num_blocks, num_slots, dtype, device)
+
+    def forward(self, h, meta, cache: LayerCache):
+        F, n, m = self.ff, self.mixer.in_cols, self.mixer.out_cols
+        both = ops.linear(h, self.inp.data)
+        if not self.fused_out:
+            pair = self.mixer(both[:, F:F + n], meta, cache)
+            y = ops.linear(seqmix.gelu_rows(both[:, :F]), self.out.data) if F else None
+            return y, (*pair, self.mixer.left_w.data, self.mixer.right_w.data)
+        acts = torch.empty(h.shape[0], m + F, dtype=h.dtype, device=h.device)
+        self.mixer(both[:, F:F + n], acts[:, :m], meta, cache)
+        if F:
+            seqmix.gelu_rows(both[:, :F], out=acts[:, m:])
+        return ops.linear(acts, self.out.data), None
 
 
 class GatedParallelLayer(nn.Module):

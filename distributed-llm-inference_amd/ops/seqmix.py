@@ -101,22 +101,44 @@ def add_ln(x: torch.Tensor, y: torch.Tensor, w: torch.Tensor, b: torch.Tensor, e
 
 
 def rms_gate(o: torch.Tensor, w: Optional[torch.Tensor], eps: float, gate: torch.Tensor, out_dtype: torch.dtype, groups: int = 1,
-             gate_act: str = "sigmoid") -> torch.Tensor:
+             gate_act: str = "sigmoid", out: Optional[torch.Tensor] = None, divide: Optional[tuple] = None, skip: Optional[tuple] = None,
+             gate_first: bool = False, token_seq: Optional[torch.Tensor] = None) -> torch.Tensor:
     """``o / rms(o) · w · act(gate)`` per row (``o`` fp32 ``[T, N]``, or — what the GPU scan returns — planes of partial
     sums ``[parts, T, N]`` whose sum is the row; ``gate`` a row-strided view).  ``groups`` > 1: every one of that many equal
-    slices of the row is divided by its own root mean square; ``w`` None: no weight; ``gate_act``: ``"sigmoid"`` or ``"silu"``."""
+    slices of the row is divided by its own root mean square; ``w`` None: no weight, ``[N / groups]``: one weight for all
+    slices; ``gate_act``: ``"sigmoid"`` or ``"silu"``.  ``divide = (d, floor)`` fp32 ``[T, heads]``: head ``h``'s slice of ``o`` is first
+    divided by ``max(|d|, floor) + 1e-6``.  ``skip = (x [T, N] fp32 view, c [heads])``: ``c[h] · x`` is added first.  ``gate_first``: the
+    gate multiplies in front of the norm.  ``out``: result rows (a row-strided view); ``token_seq``: rows with a negative entry
+    become zeros on the GPU."""
     assert gate_act in ("sigmoid", "silu")
     if o.is_cuda:
-        return _hip().sm_rms_gate(o, w, eps, gate, out_dtype == torch.bfloat16, groups, gate_act == "silu")
+        d, floor = divide if divide is not None else (None, None)
+        x, c = skip if skip is not None else (None, None)
+        return _hip().sm_rms_gate(o, w, eps, gate, out_dtype == torch.bfloat16, groups, gate_act == "silu", out, d, floor, x, c,
+                                  gate_first, token_seq)
     if o.dim() == 3:
         o = o.sum(0)
     T, N = o.shape
-    g = o.view(T, groups, N // groups)
-    y = (g * torch.rsqrt((g * g).mean(-1, keepdim=True) + eps)).reshape(T, N)
-    if w is not None:
-        y = y * w
+    if divide is not None:
+        den = torch.maximum(divide[0].abs(), divide[1]) + 1e-6
+        o = (o.view(T, den.shape[1], -1) / den.unsqueeze(2)).view(T, N)
+    if skip is not None:
+        H = skip[1].numel()
+        o = o + (skip[0].reshape(T, H, N // H) * skip[1].view(1, H, 1)).reshape(T, N)
     z = gate.float()
-    return (y * (torch.sigmoid(z) if gate_act == "sigmoid" else torch.nn.functional.silu(z))).to(out_dtype)
+    act = torch.sigmoid(z) if gate_act == "sigmoid" else torch.nn.functional.silu(z)
+    if gate_first:
+        o = o * act
+    g = o.view(T, groups, N // groups)
+    y = g * torch.rsqrt((g * g).mean(-1, keepdim=True) + eps)
+    if w is not None:
+        y = y * (w if w.numel() == N // groups else w.view(groups, N // groups))
+    y = y.reshape(T, N)
+    y = (y if gate_first else y * act).to(out_dtype)
+    if out is None:
+        return y
+    out.copy_(y)
+    return out
 
 
 def relu2(x: torch.Tensor) -> torch.Tensor:
@@ -666,14 +688,25 @@ def gated_experts(h: torch.Tensor, ids: torch.Tensor, wts: torch.Tensor, gate_up
 # (``models/mixers.py``: ``GatedLinearRecurrence``, ``GatedLatentAttention``, ``ScoreRoutedFF``).  GPU kernels:
 # ``csrc/kernels/recurmix.hip`` (``torch.ops.dli.rm_*``) beside extensions of the kernels above.
 def causal_conv(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor], state: torch.Tensor, meta,
-                out_dtype: torch.dtype) -> torch.Tensor:
+                out_dtype: torch.dtype, act: str = "none", unit: Optional[tuple] = None, gates: Optional[tuple] = None):
     """``x [T, C]`` (a row-strided view); ``w [taps, C]`` fp32 (tap-major: the last row weighs the token itself).  Row ``t`` of
     the result is ``bias + Σ_j w[j] · x[t - taps + 1 + j]`` over the rows of the same sequence: rows above inside a chunk, the
     sequence's ``state`` rows ``[slots, taps-1, C]`` (its last ``taps-1`` inputs, oldest first) before a chunk's start, zero
-    before position 0.  The state rows are then moved on to the sequence's last ``taps-1`` inputs of this step."""
+    before position 0.  The state rows are then moved on to the sequence's last ``taps-1`` inputs of this step.
+
+    ``act="silu"``: applied to the result.  ``unit = (n, d, scaled, scale)``: the first ``n · d`` columns are ``n`` vectors brought to
+    unit length, ``v / sqrt(Σ v² + 1e-6)``, the first ``scaled`` of them times ``scale``.  ``gates = (kind, g, rate, gate_bias)`` (``g`` a view
+    with ``x``'s row stride; ``rate``, ``gate_bias`` fp32 ``[H]``) also returns two fp32 ``[T, H]`` tensors, the log decay and the input
+    weight of every head for ``gated_scan``: ``"delta"``, ``g = [β | decay]`` columns — ``-rate · softplus(decay + gate_bias)`` and
+    ``sigmoid(β)``; ``"ssd"``, ``g`` = step sizes — ``-rate · dt`` and ``dt = softplus(g + gate_bias)``."""
+    assert act in ("none", "silu")
     if _act_ok(x):
-        return _hip().rm_causal_conv(x, w, bias, state, meta.positions, meta.token_seq, meta.query_start_loc, meta.state_slots,
-                                     meta.counts, meta.num_seqs, out_dtype == torch.bfloat16)
+        kind, g, rate, gb = gates if gates is not None else ("", None, None, None)
+        n, d, scaled, scale = unit if unit is not None else (0, 1, 0, 1.0)
+        out, decay, weight = _hip().rm_causal_conv(x, w, bias, state, meta.positions, meta.token_seq, meta.query_start_loc, meta.state_slots,
+                                                   meta.counts, meta.num_seqs, out_dtype == torch.bfloat16, act == "silu", n, d, scaled,
+                                                   scale, {"": 0, "delta": 1, "ssd": 2}[kind], g, rate, gb, meta.num_prefill_tiles > 0)
+        return (out, decay, weight) if gates is not None else out
     taps, C = w.shape
     xf = x.float()
     out = torch.zeros(x.shape[0], C)
@@ -690,7 +723,23 @@ def causal_conv(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor], 
             state[slot] = ext[n:]
     if bias is not None:
         out = out + bias
-    return out.to(out_dtype)
+    if act == "silu":
+        out = torch.nn.functional.silu(out)
+    if unit is not None:
+        n, d, scaled, scale = unit
+        v = out[:, :n * d].reshape(-1, n, d)
+        v = v * torch.rsqrt((v * v).sum(-1, keepdim=True) + 1e-6)
+        v[:, :scaled] *= scale
+        out = torch.cat([v.reshape(-1, n * d), out[:, n * d:]], dim=1)
+    out = out.to(out_dtype)
+    if gates is None:
+        return out
+    kind, g, rate, gb = gates
+    if kind == "delta":
+        H = rate.numel()
+        return out, -rate * torch.nn.functional.softplus(g[:, H:].float() + gb, threshold=1e9), torch.sigmoid(g[:, :H].float())
+    dt = torch.nn.functional.softplus(g.float() + gb, threshold=1e9)
+    return out, -rate * dt, dt
 
 
 def rglru_scan(z: torch.Tensor, u: torch.Tensor, y: torch.Tensor, gate_bias: torch.Tensor, rate: torch.Tensor, state: torch.Tensor,
@@ -789,3 +838,136 @@ def softmax_all_route(h: torch.Tensor, router: torch.Tensor, choice_bias: Option
     ids = ids[:, :top]
     w = torch.gather(sc, 1, ids)
     return ids.int(), w / (w.sum(-1, keepdim=True) + 1e-20)
+
+
+# ====================================================================================== single-norm layers, gated matrix states
+# Ops of stacks whose layers read one tanh norm with mixer and feed-forward side by side, and of the mixers with a gated matrix
+# state per head (``models/mixers.py``: ``DeltaRule``, ``MatrixMemory``, ``StateSpace``) and convolved attention (``ConvAttention``).
+# GPU kernels: ``csrc/kernels/gatemix.hip`` (``torch.ops.dli.gm_*``) beside extensions of the kernels above.
+def residual_tanh_norm(x: torch.Tensor, y: Optional[torch.Tensor], pair: Optional[tuple], mult: float, alpha: torch.Tensor, w: torch.Tensor,
+                       b: torch.Tensor, eps: float, out_dtype: torch.dtype) -> torch.Tensor:
+    """In place on the fp32 stream ``x [T, W]``: ``x += mult · (y + ½ (rms(l) · wl + rms(r) · wr))`` — ``y`` and ``pair = (l, r, wl, wr)``
+    both optional, ``rms(v) = v / sqrt(mean(v²) + eps)`` — then returns ``tanh(alpha · x) · w + b`` in ``out_dtype``."""
+    if x.is_cuda:
+        l, r, wl, wr = pair if pair is not None else (None, None, None, None)
+        return _hip().gm_residual_tanh_norm(x, y, l, r, wl, wr, mult, alpha, w, b, eps, out_dtype == torch.bfloat16)
+    add = None
+    if pair is not None:
+        l, r, wl, wr = pair
+        l, r = l.float(), r.float()
+        add = 0.5 * (l * torch.rsqrt((l * l).mean(-1, keepdim=True) + eps) * wl + r * torch.rsqrt((r * r).mean(-1, keepdim=True) + eps) * wr)
+    if y is not None:
+        add = y.float() if add is None else add + y.float()
+    if add is not None:
+        x.add_(add, alpha=mult)
+    return (torch.tanh(alpha * x) * w + b).to(out_dtype)
+
+
+def gelu_rows(x: torch.Tensor, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """tanh-form GELU of a row-strided 2-D view, into ``out`` (row-strided view) or a contiguous tensor."""
+    if _act_ok(x):
+        return _hip().gm_gelu_rows(x, out)
+    y = torch.nn.functional.gelu(x.float(), approximate="tanh").to(x.dtype)
+    if out is None:
+        return y
+    out.copy_(y)
+    return out
+
+
+def banded_inv_freq(base: float, dims: int, scaling: tuple = (), device="cpu") -> torch.Tensor:
+    """Rotation frequencies of ``dims`` rotated entries (float64 ``[dims/2]``).  ``scaling = (factor, original, high, low)``: pairs whose
+    wavelength is below ``original / high`` keep their frequency, those above ``original / low`` have it divided by ``factor``, with a
+    blend in ``original / wavelength`` between the two."""
+    import math
+    f = rotary_inv_freq(base, dims, "cpu")
+    if scaling:
+        factor, original, high, low = scaling
+        turns = original * f / (2.0 * math.pi)                             # original / wavelength
+        s = (turns - low) / (high - low) if high != low else (turns >= low).double()
+        f = torch.where(turns > high, f, torch.where(turns < low, f / factor, (1.0 - s) * f / factor + s * f))
+    return f.to(device)
+
+
+def conv_rope_cache(qk: torch.Tensor, w: torch.Tensor, state: torch.Tensor, meta, inv_freq: torch.Tensor, rot_dims: int,
+                    k_cache: torch.Tensor, v_cache: torch.Tensor, H: int, G: int, D: int) -> torch.Tensor:
+    """``qk [T, (H+G)·D]`` (row-strided view) = query and key projections.  Both pass the causal convolution of ``causal_conv`` (no
+    bias; its ``state`` rows); the convolved keys go to ``v_cache``; then entries ``i`` and ``i + rot_dims/2`` of every head are turned by
+    ``position · inv_freq[i]``, the keys go to ``k_cache`` (token-major rows ``slot_mapping``, < 0: skipped) and the queries are
+    returned (``[T, H·D]``)."""
+    if _act_ok(qk):
+        return _hip().rm_conv_rope_cache(qk, w, state, meta.positions, meta.token_seq, meta.query_start_loc, meta.state_slots, meta.counts,
+                                         meta.num_seqs, inv_freq if rot_dims else None, rot_dims, meta.slot_mapping, k_cache, v_cache,
+                                         H, G, D, meta.num_prefill_tiles > 0)
+    T = qk.shape[0]
+    c = causal_conv(qk, w, None, state, meta, torch.float32).view(T, H + G, D)
+    rot = _turn_half(c, meta.positions[:T], inv_freq, 1.0, rot_dims) if rot_dims else c
+    keep = meta.slot_mapping[:T] >= 0
+    s = meta.slot_mapping[:T][keep].long()
+    k_cache.view(-1, G * D)[s] = rot[:, H:].reshape(T, G * D)[keep].to(k_cache.dtype)
+    v_cache.view(-1, G * D)[s] = c[:, H:].reshape(T, G * D)[keep].to(v_cache.dtype)
+    return rot[:, :H].reshape(T, H * D).to(qk.dtype)
+
+
+def max_gates(g: torch.Tensor, bias: torch.Tensor, cap: float, state: torch.Tensor, meta):
+    """Exponential gating with a running maximum.  ``g [T, ≥ 2H]`` (row-strided view) = input and forget gate columns before their
+    ``bias`` fp32 ``[2H]``: ``i = cap · tanh((g_i + b_i) / cap)``, ``f = logsigmoid(cap · tanh((g_f + b_f) / cap))``.  Per sequence and head,
+    ``m ← max(f + m, i)`` from ``state[slot, h]`` (zero at position 0), written back after the step's last token.  Returns fp32
+    ``[T, H]``: the log decay ``f + m_before - m``, the input weight ``exp(i - m)`` and ``exp(-m)``."""
+    H = bias.numel() // 2
+    if _act_ok(g):
+        return _hip().gm_max_gates(g, bias, cap, state, meta.positions, meta.query_start_loc, meta.state_slots, meta.counts, meta.num_seqs,
+                                   meta.num_prefill_tiles > 0)
+    z = cap * torch.tanh((g[:, :2 * H].float() + bias) / cap)
+    i, f = z[:, :H], torch.nn.functional.logsigmoid(z[:, H:])
+    T = g.shape[0]
+    keep, write, floor = (torch.zeros(T, H) for _ in range(3))
+    for _i, t0, t1, slot in _seq_rows(meta):
+        m = state[slot].clone() if int(meta.positions[t0]) > 0 else torch.zeros(H)
+        for t in range(t0, t1):
+            new = torch.maximum(f[t] + m, i[t])
+            keep[t], write[t], floor[t] = f[t] + m - new, torch.exp(i[t] - new), torch.exp(-new)
+            m = new
+        state[slot] = m
+    return keep, write, floor
+
+
+def gated_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.Tensor, weight: torch.Tensor, state: torch.Tensor, meta,
+               H: int, G: int, D: int, Dv: int, delta: bool = False, q_scale: float = 1.0, normaliser: bool = False):
+    """Linear recurrence with a gated matrix state.  ``q``, ``k`` ``[T, G·D]`` and ``v`` ``[T, H·Dv]`` (row-strided views; head ``h`` uses q / k
+    head ``h // (H/G)``); ``decay`` (logarithms) and ``weight`` fp32 ``[T, H]``.  Per sequence and head, token by token in fp32, with ``S``
+    the sequence's ``state[slot, h]`` ``[D, Dv]`` (zero at position 0), written back after the step's last token:
+    ``S ← exp(decay) S``; ``u = weight · v``, with ``delta`` ``u = weight · (v - Sᵀ k)``; ``S ← S + k uᵀ``; ``o = q_scale · Sᵀ q``.  ``normaliser``:
+    ``n ← exp(decay) n + weight · k`` is kept behind ``S`` (``state [slots, H, D·(Dv+1)]``).  Returns ``(o fp32 [T, H·Dv], q_scale · n · q fp32
+    [T, H] or None)``."""
+    if _act_ok(q):
+        # chunks of two tokens or more run block by block over the step's 64-token tiles on the matrix cores
+        tiles = meta.num_prefill_tiles if BLOCK_SCAN else 0
+        o, nq = _hip().gm_gated_scan(q, k, v, decay, weight, state, meta.positions, meta.query_start_loc, meta.state_slots, meta.counts,
+                                     meta.num_seqs, H, G, D, Dv, delta, q_scale, normaliser, meta.prefill_tile_seq if tiles else None,
+                                     meta.prefill_tile_q0 if tiles else None, tiles)
+        return o, (nq if normaliser else None)
+    T = q.shape[0]
+    rep = H // G
+    qf, kf = (t.float().reshape(T, G, D).repeat_interleave(rep, dim=1) for t in (q, k))
+    vf = v.float().reshape(T, H, Dv)
+    if normaliser:
+        vf = torch.cat([vf, torch.ones(T, H, 1)], dim=2)
+    cols = vf.shape[2]
+    o = torch.zeros(T, H, cols)
+    for _i, t0, t1, slot in _seq_rows(meta):
+        S = torch.zeros(H, D, cols)
+        if int(meta.positions[t0]) > 0:
+            flat = state[slot].view(H, D * cols)
+            S[:, :, :Dv] = flat[:, :D * Dv].view(H, D, Dv)
+            if normaliser:
+                S[:, :, Dv] = flat[:, D * Dv:]
+        for t in range(t0, t1):
+            S = torch.exp(decay[t]).view(H, 1, 1) * S
+            u = vf[t] - torch.einsum("hde,hd->he", S, kf[t]) if delta else vf[t]
+            S = S + kf[t].unsqueeze(2) * (weight[t].unsqueeze(1) * u).unsqueeze(1)
+            o[t] = torch.einsum("hde,hd->he", S, qf[t]) * q_scale
+        flat = state[slot].view(H, D * cols)
+        flat[:, :D * Dv] = S[:, :, :Dv].reshape(H, D * Dv)
+        if normaliser:
+            flat[:, D * Dv:] = S[:, :, Dv]
+    return o[:, :, :Dv].reshape(T, H * Dv), (o[:, :, Dv] if normaliser else None)

@@ -829,7 +829,7 @@ class ModelRunner:
         same recurrent / token-shift state both times — cache pages, in contrast, are rewritten with the same values)."""
         if not self.stateful:
             return []
-        return [(t, t[:n].clone()) for c in self.kv_caches for t in (c.state, c.shift) if t is not None]
+        return [(t, t[:n].clone()) for c in self.kv_caches for t in c.state_tensors()]
 
     @staticmethod
     def _restore_state_rows(saved: list) -> None:
