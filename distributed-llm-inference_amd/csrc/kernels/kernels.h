@@ -74,8 +74,10 @@ void launch_sm_ln_shift(const float* x, const float* add, float* xout, const flo
                         const int* counts, int rows, int seqs, float eps, int W, void* out, bool out_bf16, hipStream_t stream);
 void launch_sm_add_ln(float* x, const void* y, bool y_bf16, int64_t y_stride, const float* w1, const float* b1, float mult,
                       const float* w2, const float* b2, float eps, int rows, int W, void* out, bool out_bf16, hipStream_t stream);
-void launch_sm_rms_gate(const float* o, int parts, const float* w, float eps, const void* gate, bool gate_bf16, int64_t gate_stride,
-                        int rows, int N, void* out, bool out_bf16, int groups, bool silu, hipStream_t stream);
+void launch_sm_rms_gate(const float* o, int parts, const float* w, int wn, float eps, const void* gate, bool gate_bf16,
+                        int64_t gate_stride, int rows, int N, void* out, int64_t out_stride, bool out_bf16, int groups, bool silu,
+                        const float* div, const float* floor_, int dheads, const float* skip, int64_t skip_stride, const float* skip_c,
+                        int sheads, bool gate_first, const int* token_seq, hipStream_t stream);
 int sm_lightning_parts(int D);
 void launch_sm_relu2(const void* x, void* out, int64_t n, bool bf16, hipStream_t stream);
 void launch_sm_softcap(const void* x, bool bf16, float* out, float cap, int64_t n, hipStream_t stream);
@@ -193,7 +195,13 @@ void launch_hm_softmax_route(const void* h, bool bf16, int64_t h_stride, const f
 int rm_max_taps();
 void launch_rm_causal_conv(const void* x, bool bf16, int64_t x_stride, const float* w, const float* bias, int taps, float* state,
                            const int* positions, const int* token_seq, const int* qsl, const int* state_slots, const int* counts,
-                           int rows, int seqs, int C, void* out, bool out_bf16, hipStream_t stream);
+                           int rows, int seqs, int C, void* out, bool out_bf16, bool silu, int unit_n, int unit_d, int unit_scaled,
+                           float unit_scale, int gate_kind, int gate_heads, const void* gate, const float* gate_rate,
+                           const float* gate_bias, float* decay, float* weight, bool chunks, hipStream_t stream);
+void launch_rm_conv_rope_cache(const void* x, bool bf16, int64_t x_stride, const float* w, int taps, float* state, const int* positions,
+                               const int* token_seq, const int* qsl, const int* state_slots, const int* counts, int rows, int seqs,
+                               const double* freq, int rot_dims, const int* slot_mapping, void* k_cache, void* v_cache, int H, int G,
+                               int D, void* q, bool chunks, hipStream_t stream);
 void launch_rm_rglru_scan(const void* z, const void* u, const void* y, bool bf16, int64_t y_stride, const float* gate_bias,
                           const float* rate, float* state, const int* positions, const int* qsl, const int* state_slots,
                           const int* counts, int rows, int seqs, int B, int n, void* out, bool out_bf16, const int* tile_seq,
@@ -212,5 +220,22 @@ void launch_dm_relu2_rows(const void* x, bool bf16, int64_t x_stride, int rows, 
 void launch_dm_gated_combine(float* x, float mult, const void* p0, const void* p1, float s0, float s1, const void* g1, int64_t g1_stride,
                              const float* b1, const void* ff, const void* shared, const float* sg, const void* g2, int64_t g2_stride,
                              const float* b2, bool bf16, int rows, int W, hipStream_t stream);
+
+// single-norm layers, gated matrix states (gatemix.hip)
+void launch_gm_residual_tanh_norm(float* x, const void* y, const void* l, const void* r, bool bf16, const float* wl, const float* wr,
+                                  float mult, const float* alpha, const float* w, const float* b, float eps, int rows, int W, void* out,
+                                  bool out_bf16, hipStream_t stream);
+void launch_gm_gelu_rows(const void* x, bool bf16, int64_t x_stride, int rows, int F, void* out, int64_t o_stride, hipStream_t stream);
+void launch_gm_max_gates(const void* g, bool bf16, int64_t g_stride, const float* bias, float cap, float* state, const int* positions,
+                         const int* qsl, const int* state_slots, const int* counts, int seqs, int H, float* keep, float* write,
+                         float* floor_, bool chunks, hipStream_t stream);
+int gm_step_max_dim();
+int gm_block_max_dim();
+int64_t gm_scan_ws_floats(int rows, int seqs, int H, bool delta);
+void launch_gm_gated_scan(const void* q, int64_t q_stride, const void* k, int64_t k_stride, const void* v, int64_t v_stride, bool bf16,
+                          const float* decay, const float* weight, float* state, const int* positions, const int* qsl,
+                          const int* state_slots, const int* counts, int seqs, int H, int G, int D, int Dv, bool delta, float q_scale,
+                          bool normaliser, float* out, float* nq, const int* tile_seq, const int* tile_q0, int num_tiles, float* ws,
+                          hipStream_t stream);
 
 }  // namespace dli

@@ -1,6 +1,7 @@
 // Kernels of the stacks that alternate gated linear recurrences with gated latent attention (models/mixers.py:
 // GatedLinearRecurrence, GatedLatentAttention; ops/seqmix.py): the causal per-channel convolution in front of the recurrence
-// with its per-sequence input rows, the recurrence itself (gates, decay, state, output branch), the norms / rotation / cache
+// with its per-sequence input rows (optionally with silu, unit-length vectors and step gates behind it, or with rotation and
+// cache write for the attention that convolves its queries and keys), the recurrence itself (gates, decay, state, output branch), the norms / rotation / cache
 // write of the attention's latents, the rotation of its queries and its element-wise output gate.  (Attention with a sink,
 // the layer norm over several stream copies, score routing and the clamped experts of these stacks are extensions of the
 // kernels in seqmix.hip / hypermix.hip / dualmix.hip.)
@@ -74,58 +75,132 @@ template <typename A, int V> struct Vec {
 };
 
 // ------------------------------------------------------------------------------------------------ convolution
-// out[t, c] = bias[c] + Σ_j w[j, c] · x[t - taps + 1 + j, c] over the rows of the token's own sequence: rows of this step's
+// out[t, c] = act(bias[c] + Σ_j w[j, c] · x[t - taps + 1 + j, c]) over the rows of the token's own sequence: rows of this step's
 // chunk, the sequence's state rows (its last taps-1 inputs, oldest first: positions p0-taps+1 … p0-1 for a chunk starting at
 // p0) before the chunk, nothing before position 0 (so a reused slot needs no clearing).  One workgroup per token; a thread
-// keeps one channel per trip, so all taps of a channel are coalesced row reads.
+// keeps V channels per trip, so all taps of a channel are coalesced row reads.
+//
+// Where the step brings one token of a sequence, the thread that owns a channel also moves its state rows on.  unit.n > 0: the
+// first n · d results are n vectors that leave at unit length (the first `scaled` of them times `scale`); they wait in LDS for
+// their sums.  gate.kind > 0: log decay and input weight of the token's heads (see GateArgs).
+struct ConvUnit {
+  int n, d, scaled;
+  float scale;
+};
+// g: columns with x's row stride; kind 1: [β | decay] → weight = sigmoid(β), decay = -rate · softplus(decay + bias); kind 2: step sizes →
+// weight = softplus(g + bias), decay = -rate · weight.  decay / weight: fp32 [T, H].
+template <typename A> struct GateArgs {
+  int kind, H;
+  const A* g;
+  const float *rate, *bias;
+  float *decay, *weight;
+};
+
+// the convolution of V channels from c on: x / state pointers as above, d <= back → row of the chunk, else state row
+template <typename A, int V>
+__device__ __forceinline__ Vec<float, V> conv_taps(const A* xr, int64_t x_stride, const float* w, const float* bias, int taps,
+                                                   const float* st, int p, int back, int C, int c) {
+  Vec<float, V> a;
+  if (bias != nullptr) a.load(bias + c);
+  else
+#pragma unroll
+    for (int k = 0; k < V; ++k) a.v[k] = 0.f;
+#pragma unroll 4
+  for (int j = max(taps - 1 - p, 0); j < taps; ++j) {             // taps that would reach before position 0 are skipped
+    const int d = taps - 1 - j;                                    // how far back the tap reaches
+    Vec<float, V> v, wj;
+    if (d <= back) {
+      Vec<A, V> xv;
+      xv.load(xr - (int64_t)d * x_stride + c);
+#pragma unroll
+      for (int k = 0; k < V; ++k) v.v[k] = xv.v[k];
+    } else {
+      v.load(st + (int64_t)(taps - 1 - (d - back)) * C + c);
+    }
+    wj.load(w + (int64_t)j * C + c);
+#pragma unroll
+    for (int k = 0; k < V; ++k) a.v[k] += wj.v[k] * v.v[k];
+  }
+  return a;
+}
+
+// state rows of a sequence whose step is the one token xr: up by one, the token last (one thread per V channels)
+template <typename A, int V>
+__device__ __forceinline__ void shift_rows(const A* xr, float* st, int taps, int C, int c) {
+  for (int r = 0; r + 1 < taps; ++r) {
+    Vec<float, V> v;
+    if (r + 2 < taps) {
+      v.load(st + (int64_t)(r + 1) * C + c);
+    } else {
+      Vec<A, V> xv;
+      xv.load(xr + c);
+#pragma unroll
+      for (int k = 0; k < V; ++k) v.v[k] = xv.v[k];
+    }
+    v.store(st + (int64_t)r * C + c);
+  }
+}
+
 template <typename A, typename O, int V>
 __global__ __launch_bounds__(NT) void causal_conv_kernel(const A* __restrict__ x, int64_t x_stride, const float* __restrict__ w,
-                                                         const float* __restrict__ bias, int taps, const float* __restrict__ state,
+                                                         const float* __restrict__ bias, int taps, float* state,
                                                          const int* __restrict__ positions, const int* __restrict__ token_seq,
                                                          const int* __restrict__ qsl, const int* __restrict__ state_slots, int C,
-                                                         O* __restrict__ out) {
+                                                         O* __restrict__ out, int silu, ConvUnit unit, GateArgs<A> gate) {
+  extern __shared__ float vecs[];                                 // [unit.n · unit.d]
   const int64_t t = blockIdx.x;
   const int seq = token_seq[t];
   if (seq < 0 || state_slots[seq] < 0) {                         // padding row
     for (int c = threadIdx.x; c < C; c += NT) stf<O>(out + t * C + c, 0.f);
+    if (gate.kind != 0)
+      for (int h = threadIdx.x; h < gate.H; h += NT) gate.decay[t * gate.H + h] = gate.weight[t * gate.H + h] = 0.f;
     return;
   }
   const int p = positions[t];
   const int back = (int)t - qsl[seq];                             // rows of the chunk above this one
-  const float* st = state + (int64_t)state_slots[seq] * (taps - 1) * C;
+  const bool single = qsl[seq + 1] - qsl[seq] == 1;
+  float* st = state + (int64_t)state_slots[seq] * (taps - 1) * C;
   const A* xr = x + t * x_stride;
+  const int nu = unit.n * unit.d;
   for (int c = threadIdx.x * V; c < C; c += NT * V) {
-    Vec<float, V> a;
-    if (bias != nullptr) a.load(bias + c);
-    else
+    Vec<float, V> a = conv_taps<A, V>(xr, x_stride, w, bias, taps, st, p, back, C, c);
+    if (single) shift_rows<A, V>(xr, st, taps, C, c);
+    if (silu)
 #pragma unroll
-      for (int k = 0; k < V; ++k) a.v[k] = 0.f;
-#pragma unroll 4
-    for (int j = max(taps - 1 - p, 0); j < taps; ++j) {           // taps that would reach before position 0 are skipped
-      const int d = taps - 1 - j;                                  // how far back the tap reaches
-      Vec<float, V> v, wj;
-      if (d <= back) {
-        Vec<A, V> xv;
-        xv.load(xr - (int64_t)d * x_stride + c);
-#pragma unroll
-        for (int k = 0; k < V; ++k) v.v[k] = xv.v[k];
-      } else {
-        v.load(st + (int64_t)(taps - 1 - (d - back)) * C + c);
-      }
-      wj.load(w + (int64_t)j * C + c);
-#pragma unroll
-      for (int k = 0; k < V; ++k) a.v[k] += wj.v[k] * v.v[k];
+      for (int k = 0; k < V; ++k) a.v[k] *= sigmoid_f(a.v[k]);
+    if (c < nu) {
+      a.store(vecs + c);
+      continue;
     }
     Vec<O, V> o;
 #pragma unroll
     for (int k = 0; k < V; ++k) o.v[k] = a.v[k];
     o.store(out + t * C + c);
   }
+  if (gate.kind != 0) {
+    const A* gr = gate.g + t * x_stride;
+    for (int h = threadIdx.x; h < gate.H; h += NT) {
+      const float z = ldf<A>(gr + (gate.kind == 1 ? gate.H + h : h)) + gate.bias[h];
+      const float sp = fmaxf(z, 0.f) + log1pf(expf(-fabsf(z)));  // softplus
+      gate.decay[t * gate.H + h] = -gate.rate[h] * sp;
+      gate.weight[t * gate.H + h] = gate.kind == 1 ? 1.f / (1.f + expf(-ldf<A>(gr + h))) : sp;
+    }
+  }
+  if (nu == 0) return;
+  __syncthreads();
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  for (int u = wave; u < unit.n; u += NT / 64) {                  // a wave per vector
+    const float* row = vecs + u * unit.d;
+    float ss = 0.f;
+    for (int i = lane; i < unit.d; i += 64) ss += row[i] * row[i];
+    const float inv = (u < unit.scaled ? unit.scale : 1.f) / sqrtf(wave_sum(ss) + 1e-6f);
+    for (int i = lane; i < unit.d; i += 64) stf<O>(out + t * C + u * unit.d + i, row[i] * inv);
+  }
 }
 
-// One workgroup per batch row, after the kernel above has read the old rows: the state becomes the sequence's last taps-1
-// inputs.  New row r holds chunk row n-(taps-1)+r when that exists, else old row n+r (written in increasing r by the thread
-// that owns the column, so an old row is read before its turn to be replaced).
+// One workgroup per batch row with two tokens or more, after the convolution has read the old rows: the state becomes the
+// sequence's last taps-1 inputs.  New row r holds chunk row n-(taps-1)+r when that exists, else old row n+r (written in
+// increasing r by the thread that owns the column, so an old row is read before its turn to be replaced).
 template <typename A>
 __global__ __launch_bounds__(NT) void conv_rows_kernel(const A* __restrict__ x, int64_t x_stride, int taps, float* __restrict__ state,
                                                        const int* __restrict__ qsl, const int* __restrict__ state_slots,
@@ -134,13 +209,86 @@ __global__ __launch_bounds__(NT) void conv_rows_kernel(const A* __restrict__ x, 
   if (seq >= counts[3]) return;
   const int slot = state_slots[seq];
   const int t0 = qsl[seq], n = qsl[seq + 1] - t0;
-  if (slot < 0 || n <= 0) return;
+  if (slot < 0 || n < 2) return;                                  // single tokens: moved on by the convolution itself
   float* st = state + (int64_t)slot * (taps - 1) * C;
-  for (int c = threadIdx.x; c < C; c += NT)
+  for (int c = blockIdx.y * NT + threadIdx.x; c < C; c += NT * gridDim.y)
     for (int r = 0; r < taps - 1; ++r) {
       const int i = n - (taps - 1) + r;
       st[(int64_t)r * C + c] = i >= 0 ? ldf<A>(x + (int64_t)(t0 + i) * x_stride + c) : st[(int64_t)(n + r) * C + c];
     }
+}
+
+// Query and key projections [H | G heads of D] through the convolution; the convolved keys are the values (v_cache row); entries
+// i and i + rot_dims/2 of every head turned by position · freq[i] (angles in double until reduced), queries to q, keys to the
+// k_cache row.  One workgroup per token; a thread takes V pairs (or V entries past the rotated ones) per trip.
+template <typename A, int V>
+__global__ __launch_bounds__(NT) void conv_rope_cache_kernel(const A* __restrict__ x, int64_t x_stride, const float* __restrict__ w,
+                                                             int taps, float* state, const int* __restrict__ positions,
+                                                             const int* __restrict__ token_seq, const int* __restrict__ qsl,
+                                                             const int* __restrict__ state_slots, const double* __restrict__ freq,
+                                                             int rot_dims, const int* __restrict__ slot_mapping, A* __restrict__ k_cache,
+                                                             A* __restrict__ v_cache, int H, int G, int D, A* __restrict__ q) {
+  extern __shared__ float sh[];          // cos[rot_dims/2], sin[rot_dims/2]
+  const int64_t t = blockIdx.x;
+  const int seq = token_seq[t];
+  if (seq < 0 || state_slots[seq] < 0) {
+    for (int c = threadIdx.x; c < H * D; c += NT) stf<A>(q + t * H * D + c, 0.f);
+    return;
+  }
+  const int p = positions[t], half = rot_dims >> 1, C = (H + G) * D;
+  for (int i = threadIdx.x; i < half; i += NT) {
+    double a = (double)p * freq[i];
+    a -= 6.283185307179586476925 * floor(a * 0.15915494309189533577);    // reduced in double, then exact enough in fp32
+    double sn, cs;
+    sincos(a, &sn, &cs);
+    sh[i] = (float)cs;
+    sh[half + i] = (float)sn;
+  }
+  __syncthreads();
+  const int back = (int)t - qsl[seq];
+  const bool single = qsl[seq + 1] - qsl[seq] == 1;
+  float* st = state + (int64_t)state_slots[seq] * (taps - 1) * C;
+  const A* xr = x + t * x_stride;
+  const int slot = slot_mapping[t];
+  const int per = (D - half) / V;                                 // work items of a head: pairs first, then single entries
+  for (int idx = threadIdx.x; idx < (H + G) * per; idx += NT) {
+    const int h = idx / per, i = (idx - h * per) * V;
+    const bool pair = i < half;
+    const int c = h * D + (pair ? i : i + half);
+    Vec<float, V> a = conv_taps<A, V>(xr, x_stride, w, nullptr, taps, st, p, back, C, c);
+    if (single) shift_rows<A, V>(xr, st, taps, C, c);
+    Vec<float, V> b;
+    if (pair) {
+      b = conv_taps<A, V>(xr, x_stride, w, nullptr, taps, st, p, back, C, c + half);
+      if (single) shift_rows<A, V>(xr, st, taps, C, c + half);
+    }
+    A* dst = h < H ? q + t * H * D + c : (slot >= 0 ? k_cache + (int64_t)slot * G * D + (c - H * D) : nullptr);
+    if (dst == nullptr) continue;
+    Vec<A, V> o;
+    if (h >= H) {
+      A* vd = v_cache + (int64_t)slot * G * D + (c - H * D);
+#pragma unroll
+      for (int k = 0; k < V; ++k) o.v[k] = a.v[k];
+      o.store(vd);
+      if (pair) {
+#pragma unroll
+        for (int k = 0; k < V; ++k) o.v[k] = b.v[k];
+        o.store(vd + half);
+      }
+    }
+    if (!pair) {
+#pragma unroll
+      for (int k = 0; k < V; ++k) o.v[k] = a.v[k];
+      o.store(dst);
+      continue;
+    }
+#pragma unroll
+    for (int k = 0; k < V; ++k) o.v[k] = a.v[k] * sh[i + k] - b.v[k] * sh[half + i + k];
+    o.store(dst);
+#pragma unroll
+    for (int k = 0; k < V; ++k) o.v[k] = b.v[k] * sh[i + k] + a.v[k] * sh[half + i + k];
+    o.store(dst + half);
+  }
 }
 
 // ------------------------------------------------------------------------------------------------ recurrence
@@ -457,19 +605,42 @@ static bool al16(const void* p) { return p == nullptr || reinterpret_cast<uintpt
 
 void launch_rm_causal_conv(const void* x, bool bf16, int64_t x_stride, const float* w, const float* bias, int taps, float* state,
                            const int* positions, const int* token_seq, const int* qsl, const int* state_slots, const int* counts,
-                           int rows, int seqs, int C, void* out, bool out_bf16, hipStream_t stream) {
+                           int rows, int seqs, int C, void* out, bool out_bf16, bool silu, int unit_n, int unit_d, int unit_scaled,
+                           float unit_scale, int gate_kind, int gate_heads, const void* gate, const float* gate_rate,
+                           const float* gate_bias, float* decay, float* weight, bool chunks, hipStream_t stream) {
   if (rows == 0) return;
-  if (C % 4 == 0 && x_stride % 4 == 0 && al16(x) && al16(w) && al16(bias) && al16(state) && al16(out))
-    RM_BF16(bf16, A, RM_BF16(out_bf16, O, hipLaunchKernelGGL((causal_conv_kernel<A, O, 4>), dim3(rows), dim3(NT), 0, stream, (const A*)x,
-                                                             x_stride, w, bias, taps, state, positions, token_seq, qsl, state_slots, C,
-                                                             (O*)out)));
-  else
-    RM_BF16(bf16, A, RM_BF16(out_bf16, O, hipLaunchKernelGGL((causal_conv_kernel<A, O, 1>), dim3(rows), dim3(NT), 0, stream, (const A*)x,
-                                                             x_stride, w, bias, taps, state, positions, token_seq, qsl, state_slots, C,
-                                                             (O*)out)));
-  if (taps > 1 && seqs > 0)
-    RM_BF16(bf16, A, hipLaunchKernelGGL(conv_rows_kernel<A>, dim3(seqs), dim3(NT), 0, stream, (const A*)x, x_stride, taps, state, qsl,
-                                        state_slots, counts, C));
+  const ConvUnit unit{unit_n, unit_d, unit_scaled, unit_scale};
+  const int nu = unit_n * unit_d;
+#define RM_CONV(VV)                                                                                                                  \
+  RM_BF16(bf16, A, RM_BF16(out_bf16, O, hipLaunchKernelGGL((causal_conv_kernel<A, O, VV>), dim3(rows), dim3(NT), nu * sizeof(float), \
+                                                           stream, (const A*)x, x_stride, w, bias, taps, state, positions, token_seq, \
+                                                           qsl, state_slots, C, (O*)out, silu ? 1 : 0, unit,                          \
+                                                           (GateArgs<A>{gate_kind, gate_heads, (const A*)gate, gate_rate, gate_bias,  \
+                                                                        decay, weight}))))
+  if (C % 4 == 0 && nu % 4 == 0 && x_stride % 4 == 0 && al16(x) && al16(w) && al16(bias) && al16(state) && al16(out)) RM_CONV(4);
+  else RM_CONV(1);
+#undef RM_CONV
+  if (taps > 1 && seqs > 0 && chunks)
+    RM_BF16(bf16, A, hipLaunchKernelGGL(conv_rows_kernel<A>, dim3(seqs, std::min((C + NT - 1) / NT, 16)), dim3(NT), 0, stream, (const A*)x,
+                                        x_stride, taps, state, qsl, state_slots, counts, C));
+}
+
+void launch_rm_conv_rope_cache(const void* x, bool bf16, int64_t x_stride, const float* w, int taps, float* state, const int* positions,
+                               const int* token_seq, const int* qsl, const int* state_slots, const int* counts, int rows, int seqs,
+                               const double* freq, int rot_dims, const int* slot_mapping, void* k_cache, void* v_cache, int H, int G,
+                               int D, void* q, bool chunks, hipStream_t stream) {
+  if (rows == 0) return;
+  const int half = rot_dims / 2, C = (H + G) * D;
+#define RM_CR(VV)                                                                                                                      \
+  RM_BF16(bf16, A, hipLaunchKernelGGL((conv_rope_cache_kernel<A, VV>), dim3(rows), dim3(NT), std::max(rot_dims, 2) * sizeof(float),    \
+                                      stream, (const A*)x, x_stride, w, taps, state, positions, token_seq, qsl, state_slots, freq,    \
+                                      rot_dims, slot_mapping, (A*)k_cache, (A*)v_cache, H, G, D, (A*)q))
+  if (half % 4 == 0 && D % 4 == 0 && x_stride % 4 == 0 && al16(x) && al16(w) && al16(state) && al16(k_cache) && al16(v_cache) && al16(q)) RM_CR(4);
+  else RM_CR(1);
+#undef RM_CR
+  if (taps > 1 && seqs > 0 && chunks)
+    RM_BF16(bf16, A, hipLaunchKernelGGL(conv_rows_kernel<A>, dim3(seqs, std::min((C + NT - 1) / NT, 16)), dim3(NT), 0, stream, (const A*)x,
+                                        x_stride, taps, state, qsl, state_slots, counts, C));
 }
 
 int64_t rm_rglru_ws_floats(int rows, int seqs, int C) { return (int64_t)((rows >> 6) + seqs + 1) * 2 * C; }

@@ -294,28 +294,85 @@ __global__ __launch_bounds__(NT) void add_ln_kernel(float* __restrict__ x, const
   }
 }
 
-// o: `parts` planes of partial sums [parts][T][N] (the scan cuts the state rows into parts); the row is their sum
-template <typename G, typename O>
+// o: `parts` planes of partial sums [parts][T][N] (the scan cuts the state rows into parts); the row is their sum.  Every one of
+// `groups` equal slices is divided by its own root mean square, times w ([N], or [N / groups] shared by the slices), times the
+// activated gate.  Options (null / 0: off): head h's entries first divided by max(|div[t, h]|, floor[t, h]) + 1e-6 (dheads heads);
+// skip_c[h] · skip[t, :] added (sheads heads); the gate in front of the norm; rows of padding (token_seq < 0) zeroed.
+template <typename G, typename O, int V>
 __global__ __launch_bounds__(NT) void rms_gate_kernel(const float* __restrict__ o, int parts, int64_t part_stride,
-                                                      const float* __restrict__ w, float eps, const G* __restrict__ gate,
-                                                      int64_t gate_stride, int N, O* __restrict__ out, int groups, int silu) {
+                                                      const float* __restrict__ w, int wn, float eps, const G* __restrict__ gate,
+                                                      int64_t gate_stride, int N, O* __restrict__ out, int64_t out_stride, int groups,
+                                                      int silu, const float* __restrict__ div, const float* __restrict__ floor_,
+                                                      int dheads, const float* __restrict__ skip, int64_t skip_stride,
+                                                      const float* __restrict__ skip_c, int sheads, int gate_first,
+                                                      const int* __restrict__ token_seq) {
   extern __shared__ float sh[];
   __shared__ float red[NT / 64];
   const int64_t t = blockIdx.x;
-  float s = 0.f;
-  for (int i = threadIdx.x; i < N; i += NT) {
-    float v = o[t * N + i];
-    for (int p = 1; p < parts; ++p) v += o[p * part_stride + t * N + i];
-    sh[i] = v;
-    s += v * v;
+  if (token_seq != nullptr && token_seq[t] < 0) {
+    for (int i = threadIdx.x; i < N; i += NT) stf<O>(out + t * out_stride + i, 0.f);
+    return;
   }
+  auto load = [](const auto* p, float* d) {
+    if constexpr (V == 4) {
+      const f32x4 v = ld4(p);
+      d[0] = v[0]; d[1] = v[1]; d[2] = v[2]; d[3] = v[3];
+    } else {
+      d[0] = ldf(p);
+    }
+  };
+  auto activate = [&](float g) {
+    const float a = 1.f / (1.f + expf(-g));
+    return silu ? g * a : a;
+  };
+  float s = 0.f;
+  for (int i = threadIdx.x * V; i < N; i += NT * V) {
+    float v[V], u[V];
+    load(o + t * N + i, v);
+    for (int p = 1; p < parts; ++p) {
+      load(o + p * part_stride + t * N + i, u);
+#pragma unroll
+      for (int j = 0; j < V; ++j) v[j] += u[j];
+    }
+    if (div != nullptr) {
+#pragma unroll
+      for (int j = 0; j < V; ++j) {
+        const int64_t h = t * dheads + (i + j) / (N / dheads);
+        v[j] /= fmaxf(fabsf(div[h]), floor_[h]) + 1e-6f;
+      }
+    }
+    if (skip != nullptr) {
+      load(skip + t * skip_stride + i, u);
+#pragma unroll
+      for (int j = 0; j < V; ++j) v[j] += skip_c[(i + j) / (N / sheads)] * u[j];
+    }
+    if (gate_first) {
+      load(gate + t * gate_stride + i, u);
+#pragma unroll
+      for (int j = 0; j < V; ++j) v[j] *= activate(u[j]);
+    }
+#pragma unroll
+    for (int j = 0; j < V; ++j) {
+      sh[i + j] = v[j];
+      s += v[j] * v[j];
+    }
+  }
+  const int wmask = wn > 0 ? wn : 1;
+  auto emit = [&](int c, float inv) {
+    float g[V];
+    if (!gate_first) load(gate + t * gate_stride + c, g);
+    float y[V];
+#pragma unroll
+    for (int j = 0; j < V; ++j) {
+      y[j] = sh[c + j] * inv * (w != nullptr ? w[(c + j) % wmask] : 1.f);
+      if (!gate_first) y[j] *= activate(g[j]);
+    }
+    if constexpr (V == 4) st4<O>(out + t * out_stride + c, f32x4{y[0], y[1], y[2], y[3]});
+    else stf<O>(out + t * out_stride + c, y[0]);
+  };
   if (groups <= 1) {
     const float inv = 1.f / sqrtf(block_sum<NT>(s, red) / (float)N + eps);
-    for (int i = threadIdx.x; i < N; i += NT) {
-      const float g = ldf<G>(gate + t * gate_stride + i);
-      const float a = 1.f / (1.f + expf(-g));
-      stf<O>(out + t * N + i, sh[i] * inv * (w != nullptr ? w[i] : 1.f) * (silu ? g * a : a));
-    }
+    for (int i = threadIdx.x * V; i < N; i += NT * V) emit(i, inv);
     return;
   }
   // every slice of N / groups entries has its own statistic: a wave per slice
@@ -327,12 +384,7 @@ __global__ __launch_bounds__(NT) void rms_gate_kernel(const float* __restrict__ 
     float q = 0.f;
     for (int i = lane; i < Dg; i += 64) q += row[i] * row[i];
     const float inv = 1.f / sqrtf(wave_sum(q) / (float)Dg + eps);
-    for (int i = lane; i < Dg; i += 64) {
-      const int c = gi * Dg + i;
-      const float g = ldf<G>(gate + t * gate_stride + c);
-      const float a = 1.f / (1.f + expf(-g));
-      stf<O>(out + t * N + c, row[i] * inv * (w != nullptr ? w[c] : 1.f) * (silu ? g * a : a));
-    }
+    for (int i = lane * V; i < Dg; i += 64 * V) emit(gi * Dg + i, inv);
   }
 }
 
@@ -1235,14 +1287,25 @@ void launch_sm_add_ln(float* x, const void* y, bool y_bf16, int64_t y_stride, co
                                                                                 y_stride, w1, b1, mult, w2, b2, eps, W, (O*)out)));
 }
 
-void launch_sm_rms_gate(const float* o, int parts, const float* w, float eps, const void* gate, bool gate_bf16, int64_t gate_stride,
-                        int rows, int N, void* out, bool out_bf16, int groups, bool silu, hipStream_t stream) {
+void launch_sm_rms_gate(const float* o, int parts, const float* w, int wn, float eps, const void* gate, bool gate_bf16,
+                        int64_t gate_stride, int rows, int N, void* out, int64_t out_stride, bool out_bf16, int groups, bool silu,
+                        const float* div, const float* floor_, int dheads, const float* skip, int64_t skip_stride, const float* skip_c,
+                        int sheads, bool gate_first, const int* token_seq, hipStream_t stream) {
   if (rows == 0) return;
   const int64_t ps = (int64_t)rows * N;
-  SM_DISPATCH_BF16(gate_bf16, G, SM_DISPATCH_BF16(out_bf16, O, hipLaunchKernelGGL((rms_gate_kernel<G, O>), dim3(rows), dim3(NT),
-                                                                                   N * sizeof(float), stream, o, parts, ps, w, eps,
-                                                                                   (const G*)gate, gate_stride, N, (O*)out, groups,
-                                                                                   silu ? 1 : 0)));
+  auto al = [](const void* p, uintptr_t a) { return reinterpret_cast<uintptr_t>(p) % a == 0; };
+  const bool wide = N % 4 == 0 && (N / groups) % 4 == 0 && gate_stride % 4 == 0 && out_stride % 4 == 0 && skip_stride % 4 == 0 &&
+                    al(o, 16) && al(gate, gate_bf16 ? 8 : 16) && al(out, out_bf16 ? 8 : 16) && al(skip, 16);
+#define SM_RG(VV)                                                                                                                     \
+  SM_DISPATCH_BF16(gate_bf16, G, SM_DISPATCH_BF16(out_bf16, O, hipLaunchKernelGGL((rms_gate_kernel<G, O, VV>), dim3(rows), dim3(NT),   \
+                                                                                   N * sizeof(float), stream, o, parts, ps, w, wn, eps, \
+                                                                                   (const G*)gate, gate_stride, N, (O*)out, out_stride, \
+                                                                                   groups, silu ? 1 : 0, div, floor_, dheads, skip,   \
+                                                                                   skip_stride, skip_c, sheads, gate_first ? 1 : 0,   \
+                                                                                   token_seq)))
+  if (wide) SM_RG(4);
+  else SM_RG(1);
+#undef SM_RG
 }
 
 void launch_sm_relu2(const void* x, void* out, int64_t n, bool bf16, hipStream_t stream) {

@@ -9,10 +9,15 @@ const double* rot_freq(const Tensor& freq, int64_t rot_dims) {
   return freq.data_ptr<double>();
 }
 
-// x [T, C] (row-strided view) → bias + Σ_j w[j] · x[t - taps + 1 + j] within each sequence; state [slots, taps-1, C] fp32 moves on
-Tensor rm_causal_conv(const Tensor& x, const Tensor& w, const c10::optional<Tensor>& bias, Tensor state, const Tensor& positions,
-                      const Tensor& token_seq, const Tensor& qsl, const Tensor& state_slots, const Tensor& counts, int64_t num_seqs,
-                      bool out_bf16) {
+// x [T, C] (row-strided view) → act(bias + Σ_j w[j] · x[t - taps + 1 + j]) within each sequence; state [slots, taps-1, C] fp32 moves
+// on.  unit_n vectors of unit_d leading columns leave at unit length; gate_kind 1 / 2: log decay and input weight of the heads
+// from the gate columns (x's row stride).  chunks: the step may bring more than one token of a sequence.
+std::tuple<Tensor, Tensor, Tensor> rm_causal_conv(const Tensor& x, const Tensor& w, const c10::optional<Tensor>& bias, Tensor state,
+                                                  const Tensor& positions, const Tensor& token_seq, const Tensor& qsl,
+                                                  const Tensor& state_slots, const Tensor& counts, int64_t num_seqs, bool out_bf16,
+                                                  bool silu, int64_t unit_n, int64_t unit_d, int64_t unit_scaled, double unit_scale,
+                                                  int64_t gate_kind, const c10::optional<Tensor>& gate, const c10::optional<Tensor>& rate,
+                                                  const c10::optional<Tensor>& gate_bias, bool chunks) {
   const bool bf = act_bf16(x, "x");
   check_rows(x, "x");
   const int64_t T = x.size(0), C = x.size(1);
@@ -26,11 +31,71 @@ Tensor rm_causal_conv(const Tensor& x, const Tensor& w, const c10::optional<Tens
   check_i32(token_seq, "token_seq");
   TORCH_CHECK(token_seq.numel() >= T, "token_seq shorter than the batch");
   check_step_meta(positions, qsl, state_slots, counts, T, num_seqs);
+  TORCH_CHECK(unit_n >= 0 && unit_d >= 1 && unit_n * unit_d <= C && unit_n * unit_d * 4 <= kSmMaxLds, "unit vectors too wide");
+  int64_t H = 0;
+  const void* gp = nullptr;
+  const float *rp = nullptr, *gbp = nullptr;
+  Tensor decay, weight;
+  if (gate_kind != 0) {
+    TORCH_CHECK((gate_kind == 1 || gate_kind == 2) && gate.has_value() && rate.has_value() && gate_bias.has_value(), "gates need columns, rates and biases");
+    H = rate->numel();
+    check_f32(*rate, "rate", H);
+    check_f32(*gate_bias, "gate_bias", H);
+    check_act_like(*gate, bf, "gate");
+    check_rows(*gate, "gate");
+    TORCH_CHECK(gate->size(0) == T && gate->size(1) >= (gate_kind == 1 ? 2 * H : H), "gate columns missing");
+    TORCH_CHECK(gate->stride(0) == x.stride(0) || T <= 1, "gate columns must share x's row stride");
+    gp = gate->data_ptr();
+    rp = rate->data_ptr<float>();
+    gbp = gate_bias->data_ptr<float>();
+  }
+  decay = at::empty({gate_kind != 0 ? T : 0, H}, x.options().dtype(at::kFloat));
+  weight = at::empty({gate_kind != 0 ? T : 0, H}, x.options().dtype(at::kFloat));
   Tensor out = at::empty({T, C}, x.options().dtype(out_bf16 ? at::kBFloat16 : at::kFloat));
   dli::launch_rm_causal_conv(x.data_ptr(), bf, x.stride(0), w.data_ptr<float>(), bp, (int)taps, state.data_ptr<float>(),
                              positions.data_ptr<int>(), token_seq.data_ptr<int>(), qsl.data_ptr<int>(), state_slots.data_ptr<int>(),
-                             counts.data_ptr<int>(), (int)T, (int)num_seqs, (int)C, out.data_ptr(), out_bf16, cur_stream(x));
-  return out;
+                             counts.data_ptr<int>(), (int)T, (int)num_seqs, (int)C, out.data_ptr(), out_bf16, silu, (int)unit_n, (int)unit_d,
+                             (int)unit_scaled, (float)unit_scale, (int)gate_kind, (int)H, gp, rp, gbp, decay.data_ptr<float>(),
+                             weight.data_ptr<float>(), chunks, cur_stream(x));
+  return {out, decay, weight};
+}
+
+// query / key projections [H | G heads of D] → convolution → values (v_cache), rotation → queries (returned), keys (k_cache)
+Tensor rm_conv_rope_cache(const Tensor& x, const Tensor& w, Tensor state, const Tensor& positions, const Tensor& token_seq, const Tensor& qsl,
+                          const Tensor& state_slots, const Tensor& counts, int64_t num_seqs, const c10::optional<Tensor>& freq,
+                          int64_t rot_dims, const Tensor& slot_mapping, Tensor k_cache, Tensor v_cache, int64_t H, int64_t G, int64_t D,
+                          bool chunks) {
+  const bool bf = act_bf16(x, "x");
+  check_rows(x, "x");
+  const int64_t T = x.size(0), C = (H + G) * D;
+  TORCH_CHECK(H > 0 && G > 0 && D > 0 && x.size(1) == C, "x must be [T, (H+G)·D]");
+  check_f32(w, "w");
+  TORCH_CHECK(w.dim() == 2 && w.size(1) == C && w.size(0) >= 1 && w.size(0) <= dli::rm_max_taps(), "w must be [taps, C], taps in 1..",
+              dli::rm_max_taps());
+  const int64_t taps = w.size(0);
+  check_f32(state, "state");
+  TORCH_CHECK(state.dim() == 3 && state.size(1) == taps - 1 && state.size(2) == C, "state must be [slots, taps-1, C]");
+  check_i32(token_seq, "token_seq");
+  check_i32(slot_mapping, "slot_mapping");
+  TORCH_CHECK(token_seq.numel() >= T && slot_mapping.numel() >= T, "step metadata shorter than the batch");
+  check_step_meta(positions, qsl, state_slots, counts, T, num_seqs);
+  TORCH_CHECK(rot_dims >= 0 && rot_dims % 2 == 0 && rot_dims <= D && rot_dims * 4 <= kSmMaxLds, "rot_dims must be even and at most D");
+  const double* fp = nullptr;
+  if (rot_dims > 0) {
+    TORCH_CHECK(freq.has_value(), "rotation needs frequencies");
+    fp = rot_freq(*freq, rot_dims);
+  }
+  for (const Tensor* c : {&k_cache, &v_cache}) {
+    check_act_like(*c, bf, "cache");
+    TORCH_CHECK(c->is_contiguous() && c->dim() == 3 && c->size(1) == kSmPageTokens && c->size(2) == G * D,
+                "caches must be contiguous [pages, page tokens, G·D]");
+  }
+  Tensor q = at::empty({T, H * D}, x.options());
+  dli::launch_rm_conv_rope_cache(x.data_ptr(), bf, x.stride(0), w.data_ptr<float>(), (int)taps, state.data_ptr<float>(),
+                                 positions.data_ptr<int>(), token_seq.data_ptr<int>(), qsl.data_ptr<int>(), state_slots.data_ptr<int>(),
+                                 counts.data_ptr<int>(), (int)T, (int)num_seqs, fp, (int)rot_dims, slot_mapping.data_ptr<int>(),
+                                 k_cache.data_ptr(), v_cache.data_ptr(), (int)H, (int)G, (int)D, q.data_ptr(), chunks, cur_stream(x));
+  return q;
 }
 
 // z [B, T, 2n] gate pre-activations, u [T, B·n], y [T, B·n] (row-strided view), gate_bias fp32 [2, B·n], rate fp32 [B·n],

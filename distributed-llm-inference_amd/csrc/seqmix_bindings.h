@@ -92,20 +92,61 @@ Tensor sm_add_ln(Tensor x, const Tensor& y, const Tensor& w, const Tensor& b, do
 }
 
 Tensor sm_rms_gate(const Tensor& o, const c10::optional<Tensor>& w, double eps, const Tensor& gate, bool out_bf16, int64_t groups,
-                   bool silu) {
+                   bool silu, const c10::optional<Tensor>& out_rows, const c10::optional<Tensor>& div, const c10::optional<Tensor>& floor_,
+                   const c10::optional<Tensor>& skip, const c10::optional<Tensor>& skip_c, bool gate_first,
+                   const c10::optional<Tensor>& token_seq) {
   check_f32(o, "o");
   TORCH_CHECK(o.dim() == 2 || o.dim() == 3, "o must be [T, N] or planes of partial sums [parts, T, N]");
   const int64_t parts = o.dim() == 3 ? o.size(0) : 1;
   const int64_t T = o.size(-2), N = o.size(-1);
   TORCH_CHECK(N * 4 <= kSmMaxLds, "row too wide");
-  const float* wp = opt_f32(w, "w", N);
   TORCH_CHECK(groups >= 1 && N % groups == 0, "the row does not divide into that many groups");
+  const int64_t wn = w.has_value() ? w->numel() : 0;
+  TORCH_CHECK(wn == 0 || wn == N || wn == N / groups, "w must have N entries, or N / groups");
+  const float* wp = opt_f32(w, "w", wn);
   const bool gbf = act_bf16(gate, "gate");
   check_rows(gate, "gate");
   TORCH_CHECK(gate.size(0) == T && gate.size(1) == N, "gate must be [T, N]");
-  Tensor out = at::empty({T, N}, o.options().dtype(out_bf16 ? at::kBFloat16 : at::kFloat));
-  dli::launch_sm_rms_gate(o.data_ptr<float>(), (int)parts, wp, (float)eps, gate.data_ptr(), gbf, gate.stride(0), (int)T, (int)N,
-                          out.data_ptr(), out_bf16, (int)groups, silu, cur_stream(o));
+  Tensor out;
+  if (out_rows.has_value()) {
+    out = *out_rows;
+    TORCH_CHECK(out.is_cuda() && out.scalar_type() == (out_bf16 ? at::kBFloat16 : at::kFloat), "out has the wrong type");
+    check_rows(out, "out");
+    TORCH_CHECK(out.size(0) == T && out.size(1) == N, "out must be [T, N]");
+  } else {
+    out = at::empty({T, N}, o.options().dtype(out_bf16 ? at::kBFloat16 : at::kFloat));
+  }
+  TORCH_CHECK(div.has_value() == floor_.has_value() && skip.has_value() == skip_c.has_value(), "options come in pairs");
+  const float *dp = nullptr, *fp = nullptr, *sp = nullptr, *cp = nullptr;
+  int64_t dheads = 1, sheads = 1, sstride = 0;
+  if (div.has_value()) {
+    TORCH_CHECK(div->dim() == 2 && div->size(0) == T && div->size(1) >= 1 && N % div->size(1) == 0, "div must be [T, heads]");
+    dheads = div->size(1);
+    check_f32(*div, "div", T * dheads);
+    check_f32(*floor_, "floor", T * dheads);
+    dp = div->data_ptr<float>();
+    fp = floor_->data_ptr<float>();
+  }
+  if (skip.has_value()) {
+    TORCH_CHECK(skip->is_cuda() && skip->scalar_type() == at::kFloat, "skip must be a float32 GPU tensor");
+    check_rows(*skip, "skip");
+    TORCH_CHECK(skip->size(0) == T && skip->size(1) == N, "skip must be [T, N]");
+    sheads = skip_c->numel();
+    TORCH_CHECK(sheads >= 1 && N % sheads == 0, "the row does not divide into the skip's heads");
+    check_f32(*skip_c, "skip_c", sheads);
+    sp = skip->data_ptr<float>();
+    cp = skip_c->data_ptr<float>();
+    sstride = skip->stride(0);
+  }
+  const int* tsp = nullptr;
+  if (token_seq.has_value()) {
+    check_i32(*token_seq, "token_seq");
+    TORCH_CHECK(token_seq->numel() >= T, "token_seq shorter than the batch");
+    tsp = token_seq->data_ptr<int>();
+  }
+  dli::launch_sm_rms_gate(o.data_ptr<float>(), (int)parts, wp, (int)wn, (float)eps, gate.data_ptr(), gbf, gate.stride(0), (int)T, (int)N,
+                          out.data_ptr(), out.stride(0), out_bf16, (int)groups, silu, dp, fp, (int)dheads, sp, sstride, cp, (int)sheads,
+                          gate_first, tsp, cur_stream(o));
   return out;
 }
 

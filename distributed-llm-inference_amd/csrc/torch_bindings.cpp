@@ -583,6 +583,7 @@ void ar_all_gather(int64_t st, const Tensor& inp, Tensor out) {
 #include "dualmix_bindings.h"
 #include "hypermix_bindings.h"
 #include "recurmix_bindings.h"
+#include "gatemix_bindings.h"
 
 }  // namespace
 
@@ -592,7 +593,8 @@ TORCH_LIBRARY(dli, m) {
         "Tensor token_seq, Tensor qsl, Tensor state_slots, Tensor counts, int num_seqs, bool out_bf16) -> (Tensor, Tensor)", &sm_ln_shift);
   m.def("sm_add_ln(Tensor(a!) x, Tensor y, Tensor w, Tensor b, float eps, float mult, Tensor? w2, Tensor? b2, bool out_bf16) -> Tensor",
         &sm_add_ln);
-  m.def("sm_rms_gate(Tensor o, Tensor? w, float eps, Tensor gate, bool out_bf16, int groups=1, bool silu=False) -> Tensor", &sm_rms_gate);
+  m.def("sm_rms_gate(Tensor o, Tensor? w, float eps, Tensor gate, bool out_bf16, int groups, bool silu, Tensor(a!)? out, Tensor? div, "
+        "Tensor? floor, Tensor? skip, Tensor? skip_c, bool gate_first, Tensor? token_seq) -> Tensor", &sm_rms_gate);
   m.def("sm_relu2(Tensor x) -> Tensor", &sm_relu2);
   m.def("sm_softcap(Tensor x, float cap) -> Tensor", &sm_softcap);
   m.def("sm_qk_norm_cache(Tensor(a!) qkv, Tensor qw, Tensor kw, float eps, Tensor slot_mapping, Tensor(b!) k_cache, Tensor(c!) v_cache, "
@@ -639,7 +641,12 @@ TORCH_LIBRARY(dli, m) {
   m.def("hm_act_mul(Tensor x, bool silu) -> Tensor", &hm_act_mul);
   m.def("hm_softmax_route(Tensor h, Tensor router, Tensor? bias, int K, bool all=False) -> (Tensor, Tensor)", &hm_softmax_route);
   m.def("rm_causal_conv(Tensor x, Tensor w, Tensor? bias, Tensor(a!) state, Tensor positions, Tensor token_seq, Tensor qsl, "
-        "Tensor state_slots, Tensor counts, int num_seqs, bool out_bf16) -> Tensor", &rm_causal_conv);
+        "Tensor state_slots, Tensor counts, int num_seqs, bool out_bf16, bool silu, int unit_n, int unit_d, int unit_scaled, "
+        "float unit_scale, int gate_kind, Tensor? gate, Tensor? rate, Tensor? gate_bias, bool chunks) -> (Tensor, Tensor, Tensor)",
+        &rm_causal_conv);
+  m.def("rm_conv_rope_cache(Tensor x, Tensor w, Tensor(a!) state, Tensor positions, Tensor token_seq, Tensor qsl, Tensor state_slots, "
+        "Tensor counts, int num_seqs, Tensor? freq, int rot_dims, Tensor slot_mapping, Tensor(b!) k_cache, Tensor(c!) v_cache, int H, "
+        "int G, int D, bool chunks) -> Tensor", &rm_conv_rope_cache);
   m.def("rm_rglru_scan(Tensor z, Tensor u, Tensor y, Tensor gate_bias, Tensor rate, Tensor(a!) state, Tensor positions, Tensor qsl, "
         "Tensor state_slots, Tensor counts, int num_seqs, bool out_bf16, Tensor? tile_seq=None, Tensor? tile_q0=None, int num_tiles=0) "
         "-> Tensor", &rm_rglru_scan);
@@ -649,6 +656,14 @@ TORCH_LIBRARY(dli, m) {
         &rm_rotate_heads);
   m.def("rm_gate_heads(Tensor o, Tensor gate) -> Tensor", &rm_gate_heads);
   m.def("rm_clamped_experts(Tensor h, Tensor ids, Tensor wts, Tensor gate_up, Tensor down, float limit) -> Tensor", &rm_clamped_experts);
+  m.def("gm_residual_tanh_norm(Tensor(a!) x, Tensor? y, Tensor? l, Tensor? r, Tensor? wl, Tensor? wr, float mult, Tensor alpha, Tensor w, "
+        "Tensor b, float eps, bool out_bf16) -> Tensor", &gm_residual_tanh_norm);
+  m.def("gm_gelu_rows(Tensor x, Tensor(a!)? out) -> Tensor", &gm_gelu_rows);
+  m.def("gm_max_gates(Tensor g, Tensor bias, float cap, Tensor(a!) state, Tensor positions, Tensor qsl, Tensor state_slots, Tensor counts, "
+        "int num_seqs, bool chunks) -> (Tensor, Tensor, Tensor)", &gm_max_gates);
+  m.def("gm_gated_scan(Tensor q, Tensor k, Tensor v, Tensor decay, Tensor weight, Tensor(a!) state, Tensor positions, Tensor qsl, "
+        "Tensor state_slots, Tensor counts, int num_seqs, int H, int G, int D, int Dv, bool delta, float q_scale, bool normaliser, "
+        "Tensor? tile_seq, Tensor? tile_q0, int num_tiles) -> (Tensor, Tensor)", &gm_gated_scan);
   m.def("dm_relu2_rows(Tensor x) -> Tensor", &dm_relu2_rows);
   m.def("dm_set_grouped_experts(bool on) -> ()", &dm_set_grouped_experts);
   m.def("dm_gated_combine(Tensor(a!) x, float mult, Tensor p0, Tensor p1, float s0, float s1, Tensor g1, Tensor b1, Tensor? ff, "
