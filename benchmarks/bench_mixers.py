@@ -32,6 +32,13 @@ latent attention (512-wide latent + 64 rotated, queries through a latent of 3/4 
 + 8 clamped experts and 2 identity experts, 2 per token, of the Mixtral expert width — beside ``rodelix-latent_attention``
 (mixer) and ``mixtral`` (experts); ``sinilorn`` = a recurrence (dense), a latent layer and a latent layer on the second
 one's cache rows (both with experts).
+
+``--models rodelix-lightning,nefarax-delta,nefarax-mlstm,rodelix-attention,nefarax-pair,nefarax`` compares the Nefarax stacks (one
+tanh norm per layer, mixer and plain tanh-GELU feed-forward of 1.5× the Llama FFN width side by side) with their closest families:
+``nefarax-delta`` = the gated delta rule (half as many q / k heads as value heads, heads of 128 × 128, four-tap convolutions) and
+``nefarax-mlstm`` = mLSTM (heads of 128 × 128) — both beside ``rodelix-lightning``, the framework's other ``[128, 128]`` state per head;
+``nefarax-pair`` = convolved attention beside a Mamba-2 recurrence (inner width twice the model width in heads of 64, state 128) —
+beside ``rodelix-attention`` (attention) and ``rodelix-lightning`` (recurrence); ``nefarax`` = one layer of each.
 """
 from __future__ import annotations
 
@@ -108,8 +115,22 @@ def sinilorn_raw(width, heads, kv, ffn, kinds):
             "layers": [mk[k] for k in kinds]}
 
 
+def nefarax_raw(width, heads, kv, ffn, kinds):
+    ff = {"kind": "dense", "ff": ffn * 3 // 2}
+    mk = {
+        "delta": {"type": "delta", "mlp": ff, "mixer": {"heads": heads, "kv_heads": heads // 2, "dim": 128, "vdim": 128, "conv": 4}},
+        "mlstm": {"type": "mlstm", "mlp": ff, "mixer": {"heads": heads, "dim": 128, "vdim": 128, "gate_cap": 12.0}},
+        "pair": {"type": "parallel", "mlp": ff,
+                 "mixer": {"left": {"heads": heads, "kv_heads": kv, "dim": 128, "vdim": 128, "conv": 4, "scale": 128 ** -0.5,
+                                    "rot": {"base": 500000.0, "dims": 128, "scaling": {"factor": 8.0, "high": 4.0, "low": 1.0, "original": 8192}}},
+                           "right": {"heads": 2 * width // 64, "vdim": 64, "state": 128, "groups": 1, "conv": 4, "norm_groups": 1}}},
+    }
+    return {"architecture": "Nefarax", "vocab": 32000, "width": width, "residual_mult": 0.5, "norm": {"eps": 1e-5},
+            "layers": [mk[k] for k in kinds]}
+
+
 def model_configs(size):
-    from dli_amd.config import ModelConfig, rodelix_config, sevelorn_config, sinilorn_config, vibunex_config
+    from dli_amd.config import ModelConfig, nefarax_config, rodelix_config, sevelorn_config, sinilorn_config, vibunex_config
     s = SIZES[size]
     out = {"llama": ModelConfig(name=f"llama-{size}", arch="llama", vocab_size=32000, hidden_size=s["width"],
                                 intermediate_size=s["ffn"], num_layers=LAYERS, num_heads=s["heads"], num_kv_heads=s["kv"],
@@ -124,6 +145,9 @@ def model_configs(size):
     for name, kinds in (("sinilorn", ("recurrence", "latent", "shared_latent")), ("sinilorn-recurrence", ("recurrence",) * LAYERS),
                         ("sinilorn-latent", ("latent",) * LAYERS)):
         out[name] = sinilorn_config(sinilorn_raw(s["width"], s["heads"], s["kv"], s["ffn"], kinds), name=f"{name}-{size}")
+    for name, kinds in (("nefarax", ("delta", "mlstm", "pair")), ("nefarax-delta", ("delta",) * LAYERS), ("nefarax-mlstm", ("mlstm",) * LAYERS),
+                        ("nefarax-pair", ("pair",) * LAYERS)):
+        out[name] = nefarax_config(nefarax_raw(s["width"], s["heads"], s["kv"], s["ffn"], kinds), name=f"{name}-{size}")
     kinds = ("attention", "lightning", "latent_attention")
     out["rodelix"] = rodelix_config(rodelix_raw(s["width"], s["heads"], s["kv"], s["ffn"], kinds), name=f"rodelix-{size}")
     for k in kinds:

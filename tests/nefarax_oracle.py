@@ -9,8 +9,7 @@ engine agrees with the right one):
 only), ``conv_act`` (no silu behind the delta rule's convolutions), ``unit`` (q and k of the delta rule not brought to unit
 length), ``beta`` (write strength 1), ``decay`` (states never decay), ``erase`` (the delta rule adds without subtracting what
 the key already reads), ``late_read`` (the state is read before the token's write), ``out_norm`` (no per-head norm of a
-recurrence's output), ``gate`` (no output gates), ``cap`` (mLSTM gates not capped), ``m_start`` (running maximum starts at
-minus infinity), ``normaliser`` (mLSTM output not divided), ``rotated_values`` (values are the keys after rotation),
+recurrence's output), ``gate`` (no output gates), ``cap`` (mLSTM gates not capped), ``normaliser`` (mLSTM output not divided), ``rotated_values`` (values are the keys after rotation),
 ``scaling`` (plain frequencies), ``rotation`` (no rotation), ``sink`` (no sink in the denominator), ``skip`` (no ``D x``
 term), ``late_gate`` (the gate comes behind the grouped norm), ``one_group`` (one root mean square over all groups),
 ``dt_bias`` (no bias of the step size), ``half`` (the side-by-side outputs are summed, not averaged), ``side_norm`` (they are
@@ -120,7 +119,7 @@ def mlstm_scan(q, k, v, i, f, faults=()):
     T, H, D = q.shape
     S = torch.zeros(H, D, v.shape[2], dtype=F64)
     n = torch.zeros(H, D, dtype=F64)
-    m = torch.full((H,), -math.inf if "m_start" in faults else 0.0, dtype=F64)
+    m = torch.zeros(H, dtype=F64)
     out = torch.zeros_like(v)
     for t in range(T):
         m_new = torch.maximum(f[t] + m, i[t])
