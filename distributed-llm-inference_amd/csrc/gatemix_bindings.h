@@ -67,7 +67,7 @@ std::tuple<Tensor, Tensor> gm_gated_scan(const Tensor& q, const Tensor& k, const
                                          const c10::optional<Tensor>& tile_q0, int64_t num_tiles) {
   const bool bf = act_bf16(q, "q");
   const int64_t T = q.size(0), cols = Dv + (normaliser ? 1 : 0);
-  TORCH_CHECK(G >= 1 && H >= 1 && H % G == 0 && D >= 1 && Dv >= 1 && D <= dli::gm_step_max_dim(), "head sizes: H a multiple of G, D up to ",
+  TORCH_CHECK(G >= 1 && H >= 1 && H % G == 0 && D >= 1 && Dv >= 1 && D <= dli::gm_step_max_dim() && !(delta && normaliser), "head sizes: H a multiple of G, D up to ",
               dli::gm_step_max_dim());
   check_act_like(k, bf, "k");
   check_act_like(v, bf, "v");

@@ -217,43 +217,49 @@ __global__ __launch_bounds__(NTH) void max_gates_kernel(const A* __restrict__ g,
 }
 
 // ------------------------------------------------------------------------------------------------ recurrence
-// Columns of the state: 0 … Dv-1 belong to the values; with a normaliser column Dv is a value that is always one (its state is kept
-// behind the others, [D] contiguous).  state [slots][H][D · cols].
-__device__ __forceinline__ float* state_at(float* head, int D, int Dv, int d, int e) { return head + (e < Dv ? (int64_t)d * Dv + e : (int64_t)D * Dv + d); }
+// state [slots][H][D · Dv (+ D)]: the [D][Dv] matrix of a head, then (normaliser) its vector n.
 
-// Token by token: one workgroup per (sequence, head, 64 state columns); wave v keeps rows v·DR … of its lane's column in registers.
-// Serves single tokens (and, with single_only = 0, whole chunks: sizes the block path does not take).
+// Token by token: one workgroup per (sequence, head, 64 state columns); wave v keeps rows v·DR … of its lane's column in registers,
+// the workgroup of the first columns also the normaliser.  Serves single tokens (and, with single_only = 0, whole chunks: sizes
+// the block path does not take).
 template <typename A, int DRMAX, bool DELTA>
 __global__ __launch_bounds__(NT) void scan_step_kernel(const A* __restrict__ q, int64_t q_stride, const A* __restrict__ k, int64_t k_stride,
                                                        const A* __restrict__ v, int64_t v_stride, const float* __restrict__ decay,
                                                        const float* __restrict__ weight, float* __restrict__ state,
                                                        const int* __restrict__ positions, const int* __restrict__ qsl,
                                                        const int* __restrict__ state_slots, const int* __restrict__ counts, int H, int G,
-                                                       int D, int Dv, int cols, float q_scale, float* __restrict__ out,
-                                                       float* __restrict__ nq, int single_only) {
-  __shared__ float qs[DRMAX * 4], ks[DRMAX * 4], red[4][64], red2[4][64];
-  const int seq = blockIdx.x, h = blockIdx.y;
+                                                       int D, int Dv, float q_scale, float* __restrict__ out, float* __restrict__ nq,
+                                                       int single_only) {
+  __shared__ float qs[DRMAX * 4], ks[DRMAX * 4], red[4][64], red2[4][64], sred[NT / 64];
+  const int h = blockIdx.x, seq = blockIdx.z;
   if (seq >= counts[3]) return;
   const int t0 = qsl[seq], t1 = qsl[seq + 1];
   const int slot = state_slots[seq];
   if (slot < 0 || t1 <= t0 || (single_only && t1 - t0 != 1)) return;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  const int e = blockIdx.z * 64 + lane;
-  const bool active = e < cols;
+  const int e = blockIdx.y * 64 + lane;
+  const bool active = e < Dv, norm = nq != nullptr && blockIdx.y == 0;
   const int g = h / (H / G);
   const int DR = (D + 3) >> 2, d0 = wave * DR, dn = min(DR, D - d0);
-  float* head = state + ((int64_t)slot * H + h) * D * cols;
+  float* head = state + ((int64_t)slot * H + h) * D * (Dv + (nq != nullptr ? 1 : 0));
   const bool carry = positions[t0] > 0;
   float S[DRMAX];
 #pragma unroll
-  for (int i = 0; i < DRMAX; ++i) S[i] = (carry && active && i < dn) ? *state_at(head, D, Dv, d0 + i, e) : 0.f;
+  for (int i = 0; i < DRMAX; ++i) S[i] = (carry && active && i < dn) ? head[(int64_t)(d0 + i) * Dv + e] : 0.f;
+  constexpr int NN = (DRMAX * 4 + NT - 1) / NT;
+  float nv[NN];
+#pragma unroll
+  for (int i = 0; i < NN; ++i) {
+    const int d = threadIdx.x + NT * i;
+    nv[i] = (norm && carry && d < D) ? head[(int64_t)D * Dv + d] : 0.f;
+  }
   for (int t = t0; t < t1; ++t) {
     for (int d = threadIdx.x; d < D; d += NT) {
       qs[d] = ldf<A>(q + (int64_t)t * q_stride + g * D + d);
       ks[d] = ldf<A>(k + (int64_t)t * k_stride + g * D + d);
     }
     const float a = expf(decay[(int64_t)t * H + h]), wt = weight[(int64_t)t * H + h];
-    float ve = active ? (e < Dv ? ldf<A>(v + (int64_t)t * v_stride + (int64_t)h * Dv + e) : 1.f) : 0.f;
+    float ve = active ? ldf<A>(v + (int64_t)t * v_stride + (int64_t)h * Dv + e) : 0.f;
     __syncthreads();
     float seen = 0.f;
 #pragma unroll
@@ -276,16 +282,31 @@ __global__ __launch_bounds__(NT) void scan_step_kernel(const A* __restrict__ q, 
         o += S[i] * qs[d0 + i];
       }
     red2[wave][lane] = o;
-    __syncthreads();
-    if (wave == 0 && active) {
-      o = ((red2[0][lane] + red2[1][lane]) + (red2[2][lane] + red2[3][lane])) * q_scale;
-      if (e < Dv) out[((int64_t)t * H + h) * Dv + e] = o;
-      else nq[(int64_t)t * H + h] = o;
+    if (norm) {
+      float p = 0.f;
+#pragma unroll
+      for (int i = 0; i < NN; ++i) {
+        const int d = threadIdx.x + NT * i;
+        if (d < D) {
+          nv[i] = a * nv[i] + wt * ks[d];
+          p += nv[i] * qs[d];
+        }
+      }
+      p = block_sum<NT>(p, sred) * q_scale;
+      if (threadIdx.x == 0) nq[(int64_t)t * H + h] = p;
     }
+    __syncthreads();
+    if (wave == 0 && active)
+      out[((int64_t)t * H + h) * Dv + e] = ((red2[0][lane] + red2[1][lane]) + (red2[2][lane] + red2[3][lane])) * q_scale;
   }
 #pragma unroll
   for (int i = 0; i < DRMAX; ++i)
-    if (active && i < dn) *state_at(head, D, Dv, d0 + i, e) = S[i];
+    if (active && i < dn) head[(int64_t)(d0 + i) * Dv + e] = S[i];
+#pragma unroll
+  for (int i = 0; i < NN; ++i) {
+    const int d = threadIdx.x + NT * i;
+    if (norm && d < D) head[(int64_t)D * Dv + d] = nv[i];
+  }
 }
 
 // Chunks of two tokens or more, in blocks of 64 tokens.  With P_t = Σ_{s ≤ t} decay_s inside the block and S0 the state at its start,
@@ -294,7 +315,10 @@ __global__ __launch_bounds__(NT) void scan_step_kernel(const A* __restrict__ q, 
 // U = (I + M)⁻¹ diag(w) (V - diag(exp P) K S0) with M strictly lower triangular.
 //   scan_block_kernel: per (block, head), all blocks side by side: A = tril(exp(P_t - P_j) q_t · k_j), (I + M)⁻¹ and the vectors
 //     exp(P), exp(P_end - P), w → workspace
-//   scan_walk_kernel: per (sequence, head, 16·CT state columns) over its blocks in order, the state on the matrix cores' accumulators
+//   scan_walk_kernel: per (sequence, head, 16·CT state columns) over its blocks in order, the state on the matrix cores' accumulators;
+//     everything a block reads from memory is fetched while the block before it is computed (one register set: a fragment is
+//     refilled as soon as it has been used).  The normaliser n = exp(P_end) n0 + Σ_j exp(P_end - P_j) w_j k_j and its product with q
+//     ride on the fragments of the first columns' workgroup.
 // Workspace row of a block = (first token >> 6) + batch row (unique: rows of later sequences start at later tokens): per head
 // [64][64] A | delta: [64][64] (I + M)⁻¹ | [3][64] vectors.
 template <bool DELTA> __host__ __device__ constexpr int64_t block_floats() { return (DELTA ? 2 : 1) * BT * BT + 3 * BT; }
@@ -403,15 +427,52 @@ __global__ __launch_bounds__(NT) void scan_block_kernel(const A* __restrict__ q,
   }
 }
 
+// fragments as they come from memory (converted where they are used, so that a fetch ahead does not wait for its data)
+template <typename A> struct Raw;
+template <> struct Raw<float> {
+  using v4 = f32x4;
+  static __device__ __forceinline__ f32x4 cvt(v4 v) { return v; }
+};
+template <> struct Raw<uint16_t> {
+  using v4 = bf16x4;
+  static __device__ __forceinline__ f32x4 cvt(v4 v) {
+    return f32x4{bf2f((uint16_t)v[0]), bf2f((uint16_t)v[1]), bf2f((uint16_t)v[2]), bf2f((uint16_t)v[3])};
+  }
+};
+template <typename A> __device__ __forceinline__ typename Raw<A>::v4 raw4(const A* row, int d, int D, bool wide) {
+  typename Raw<A>::v4 r;
+  if (wide) {
+    if (d < D) return *reinterpret_cast<const typename Raw<A>::v4*>(row + d);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) r[j] = 0;
+    return r;
+  }
+#pragma unroll
+  for (int j = 0; j < 4; ++j) r[j] = d + j < D ? row[d + j] : A(0);
+  return r;
+}
+// workgroup barrier for data exchanged through LDS only: fetches from memory stay in flight
+__device__ __forceinline__ void lds_barrier() {
+  asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+  __builtin_amdgcn_s_barrier();
+  asm volatile("" ::: "memory");
+}
+// sum over the four lane groups l>>4 (every lane gets it)
+__device__ __forceinline__ float group_sum(float v) {
+  v += __shfl_xor(v, 16, 64);
+  return v + __shfl_xor(v, 32, 64);
+}
+
 template <typename A, bool DELTA, int DTMAX, int CT>
 __global__ __launch_bounds__(NT) void scan_walk_kernel(const A* __restrict__ q, int64_t q_stride, const A* __restrict__ k, int64_t k_stride,
                                                        const A* __restrict__ v, int64_t v_stride, float* __restrict__ state,
                                                        const int* __restrict__ positions, const int* __restrict__ qsl,
                                                        const int* __restrict__ state_slots, const int* __restrict__ counts, int H, int G,
-                                                       int D, int Dv, int cols, int wide, float q_scale, const float* __restrict__ ws,
+                                                       int D, int Dv, int wide, float q_scale, const float* __restrict__ ws,
                                                        float* __restrict__ out, float* __restrict__ nq) {
   extern __shared__ __align__(16) float sh[];
-  const int seq = blockIdx.x, h = blockIdx.y;
+  __shared__ float wts[2][BT], ews[2][BT], ns[GM_BLOCK_MAX_D];       // (normaliser) w, exp(P_end - P) w, n at the block's start
+  const int h = blockIdx.x, seq = blockIdx.z;                        // a head's column slices share an XCD (its q / k stay in one L2)
   if (seq >= counts[3]) return;
   const int s0 = qsl[seq], n = qsl[seq + 1] - s0;
   const int slot = state_slots[seq];
@@ -424,9 +485,80 @@ __global__ __launch_bounds__(NT) void scan_walk_kernel(const A* __restrict__ q, 
   float* Rt = St + 16 * CT * DS;                          // [columns][BS]: right-hand sides of the delta rule
   float* Ut = Rt + (DELTA ? 16 * CT * BS : 0);            // [columns][BS]: u
   float* Us = Ut + 16 * CT * BS;                          // [columns][BS]: exp(P_end - P) u
-  const int e0 = blockIdx.z * 16 * CT;
-  float* head = state + ((int64_t)slot * H + h) * D * cols;
+  const int e0 = blockIdx.y * 16 * CT;
+  const bool norm = !DELTA && nq != nullptr && blockIdx.y == 0;
+  float* head = state + ((int64_t)slot * H + h) * D * (Dv + (nq != nullptr ? 1 : 0));
   const bool carry = positions[s0] > 0;
+  const int blocks = (n + BT - 1) / BT;
+
+  using R4 = typename Raw<A>::v4;
+  R4 qf[DTMAX], kf[DELTA ? DTMAX : 1], kt[DW][4];
+  A vf[CT][4];
+  f32x4 ia[DELTA ? 4 : 1], aa[4], ep, er, wt;
+  float pend = 0.f, wl = 0.f, el = 0.f, epc = 0.f;
+  auto base_of = [&](int b) { return ws + ((int64_t)(((s0 + BT * b) >> 6) + seq) * H + h) * block_floats<DELTA>(); };
+  auto fetch_rows = [&](int b) {                          // q (and k) rows 16·wave + c; rows past the chunk repeat its last token
+    const int64_t tr = s0 + min(BT * b + 16 * wave + c, n - 1);
+    const A* qr = q + tr * q_stride + g * D;
+    const A* kr = k + tr * k_stride + g * D;
+#pragma unroll
+    for (int i = 0; i < DTMAX; ++i)
+      if (i < DT) {
+        qf[i] = raw4<A>(qr, 16 * i + 4 * g4, D, wide);
+        if (DELTA) kf[i] = raw4<A>(kr, 16 * i + 4 * g4, D, wide);
+      }
+  };
+  auto fetch_values = [&](int b) {
+#pragma unroll
+    for (int ct = 0; ct < CT; ++ct) {
+      const int e = min(e0 + 16 * ct + c, Dv - 1);
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+        vf[ct][r] = v[(int64_t)(s0 + min(BT * b + 16 * wave + 4 * g4 + r, n - 1)) * v_stride + (int64_t)h * Dv + e];
+    }
+  };
+  auto fetch_vectors = [&](int b) {
+    const float* wv = base_of(b) + (DELTA ? 2 : 1) * BT * BT;
+    ep = ld4<float>(wv + 16 * wave + 4 * g4);
+    er = ld4<float>(wv + BT + 16 * wave + 4 * g4);
+    wt = ld4<float>(wv + 2 * BT + 16 * wave + 4 * g4);
+    pend = wv[BT - 1];
+    if (norm) {
+      wl = wv[2 * BT + lane];
+      el = wv[BT + lane];
+      epc = wv[16 * wave + c];
+    }
+  };
+  auto fetch_inverse = [&](int b) {
+    const float* wi = base_of(b) + BT * BT;
+#pragma unroll
+    for (int s = 0; s < 4; ++s)
+      if (DELTA && s <= wave) ia[s] = ld4<float>(wi + (16 * wave + c) * BT + 16 * s + 4 * g4);
+  };
+  auto fetch_scores = [&](int b) {
+    const float* wa = base_of(b);
+#pragma unroll
+    for (int s = 0; s < 4; ++s)
+      if (s <= wave) aa[s] = ld4<float>(wa + (16 * wave + c) * BT + 16 * s + 4 * g4);
+  };
+  auto fetch_columns = [&](int b) {                       // kᵀ of this wave's state row tiles
+#pragma unroll
+    for (int i = 0; i < DW; ++i)
+      if (wave + 4 * i < DT) {
+        const int d = min(16 * (wave + 4 * i) + c, D - 1);
+#pragma unroll
+        for (int s = 0; s < 4; ++s)
+#pragma unroll
+          for (int j = 0; j < 4; ++j) kt[i][s][j] = k[(int64_t)(s0 + min(BT * b + 16 * s + 4 * g4 + j, n - 1)) * k_stride + g * D + d];
+      }
+  };
+  fetch_rows(0);
+  fetch_vectors(0);
+  fetch_values(0);
+  fetch_inverse(0);
+  fetch_scores(0);
+  fetch_columns(0);
+
   f32x4 S[DW][CT];
 #pragma unroll
   for (int i = 0; i < DW; ++i)
@@ -435,73 +567,72 @@ __global__ __launch_bounds__(NT) void scan_walk_kernel(const A* __restrict__ q, 
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int d = 16 * (wave + 4 * i) + 4 * g4 + r, e = e0 + 16 * ct + c;
-        S[i][ct][r] = (carry && d < D && e < cols) ? *state_at(head, D, Dv, d, e) : 0.f;
+        S[i][ct][r] = (carry && d < D && e < Dv) ? head[(int64_t)d * Dv + e] : 0.f;
       }
-  const int blocks = (n + BT - 1) / BT;
+  if (norm)
+    for (int d = threadIdx.x; d < DT * 16; d += NT) ns[d] = (carry && d < D) ? head[(int64_t)D * Dv + d] : 0.f;
+
   for (int b = 0; b < blocks; ++b) {
     const int t0 = s0 + BT * b, nn = min(BT, n - BT * b);
-    const float* wa = ws + ((int64_t)((t0 >> 6) + seq) * H + h) * block_floats<DELTA>();
-    const float* wi = wa + BT * BT;
-    const float* wv = wa + (DELTA ? 2 : 1) * BT * BT;
+    const bool more = b + 1 < blocks;
 #pragma unroll
     for (int i = 0; i < DW; ++i)
       if (wave + 4 * i < DT)
 #pragma unroll
         for (int ct = 0; ct < CT; ++ct) *reinterpret_cast<f32x4*>(St + (16 * ct + c) * DS + 16 * (wave + 4 * i) + 4 * g4) = S[i][ct];
-    __syncthreads();
+    if (norm && wave == 0) {
+      wts[b & 1][lane] = wl;
+      ews[b & 1][lane] = wl * el;
+    }
+    lds_barrier();
     // rows 16·wave … of K S0 and Q S0
     f32x4 ks[CT], o[CT];
+    float pn = 0.f;
 #pragma unroll
     for (int ct = 0; ct < CT; ++ct) ks[ct] = o[ct] = f32x4{0.f, 0.f, 0.f, 0.f};
-    const int64_t tr = t0 + min(16 * wave + c, nn - 1);
-    const A* qr = q + tr * q_stride + g * D;
-    const A* kr = k + tr * k_stride + g * D;
 #pragma unroll
     for (int i = 0; i < DTMAX; ++i)
       if (i < DT) {
         const int d = 16 * i + 4 * g4;
-        const f32x4 qa = row4(qr, d, D, wide);
+        const f32x4 qa = Raw<A>::cvt(qf[i]);
         f32x4 ka;
-        if (DELTA) ka = row4(kr, d, D, wide);
+        if (DELTA) ka = Raw<A>::cvt(kf[i]);
 #pragma unroll
         for (int ct = 0; ct < CT; ++ct) {
           const f32x4 sb = *reinterpret_cast<const f32x4*>(St + (16 * ct + c) * DS + d);
           o[ct] = mfma_k16(qa, sb, o[ct]);
           if (DELTA) ks[ct] = mfma_k16(ka, sb, ks[ct]);
         }
+        if (norm) pn += (qa[0] * ns[d] + qa[1] * ns[d + 1]) + (qa[2] * ns[d + 2] + qa[3] * ns[d + 3]);
       }
-    const f32x4 ep = ld4<float>(wv + 16 * wave + 4 * g4), er = ld4<float>(wv + BT + 16 * wave + 4 * g4),
-                wt = ld4<float>(wv + 2 * BT + 16 * wave + 4 * g4);
-    const float pend = wv[BT - 1];
+    if (more) fetch_rows(b + 1);
     f32x4 u[CT];
 #pragma unroll
     for (int ct = 0; ct < CT; ++ct) {
-      const int e = e0 + 16 * ct + c;
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
-        const int i = 16 * wave + 4 * g4 + r;
-        float x = 0.f;
-        if (i < nn && e < cols) x = e < Dv ? ldf<A>(v + (int64_t)(t0 + i) * v_stride + (int64_t)h * Dv + e) : 1.f;
+        float x = ldf<A>(&vf[ct][r]);
         if (DELTA) x -= ep[r] * ks[ct][r];
-        u[ct][r] = i < nn ? wt[r] * x : 0.f;
+        u[ct][r] = 16 * wave + 4 * g4 + r < nn ? wt[r] * x : 0.f;
         o[ct][r] *= ep[r] * q_scale;
       }
     }
+    if (more) fetch_values(b + 1);
     if (DELTA) {
 #pragma unroll
       for (int ct = 0; ct < CT; ++ct) {
         *reinterpret_cast<f32x4*>(Rt + (16 * ct + c) * BS + 16 * wave + 4 * g4) = u[ct];
         u[ct] = f32x4{0.f, 0.f, 0.f, 0.f};
       }
-      __syncthreads();
+      lds_barrier();
 #pragma unroll
       for (int s = 0; s < 4; ++s)
         if (s <= wave) {
-          const f32x4 ia = ld4<float>(wi + (16 * wave + c) * BT + 16 * s + 4 * g4);
 #pragma unroll
           for (int ct = 0; ct < CT; ++ct)
-            u[ct] = mfma_k16(ia, *reinterpret_cast<const f32x4*>(Rt + (16 * ct + c) * BS + 16 * s + 4 * g4), u[ct]);
+            u[ct] = mfma_k16(ia[s], *reinterpret_cast<const f32x4*>(Rt + (16 * ct + c) * BS + 16 * s + 4 * g4), u[ct]);
         }
+      if (more) fetch_inverse(b + 1);
     }
 #pragma unroll
     for (int ct = 0; ct < CT; ++ct) {
@@ -509,25 +640,35 @@ __global__ __launch_bounds__(NT) void scan_walk_kernel(const A* __restrict__ q, 
       *reinterpret_cast<f32x4*>(p) = u[ct];
       *reinterpret_cast<f32x4*>(p + (Us - Ut)) = f32x4{u[ct][0] * er[0], u[ct][1] * er[1], u[ct][2] * er[2], u[ct][3] * er[3]};
     }
-    __syncthreads();
+    lds_barrier();
+    float rs = 0.f;
 #pragma unroll
     for (int s = 0; s < 4; ++s)
       if (s <= wave) {
-        const f32x4 aa = ld4<float>(wa + (16 * wave + c) * BT + 16 * s + 4 * g4);
 #pragma unroll
         for (int ct = 0; ct < CT; ++ct)
-          o[ct] = mfma_k16(aa, *reinterpret_cast<const f32x4*>(Ut + (16 * ct + c) * BS + 16 * s + 4 * g4), o[ct]);
+          o[ct] = mfma_k16(aa[s], *reinterpret_cast<const f32x4*>(Ut + (16 * ct + c) * BS + 16 * s + 4 * g4), o[ct]);
+        if (norm) {
+          const float* w4 = wts[b & 1] + 16 * s + 4 * g4;
+          rs += (aa[s][0] * w4[0] + aa[s][1] * w4[1]) + (aa[s][2] * w4[2] + aa[s][3] * w4[3]);
+        }
       }
+    if (norm) {
+      const float x = group_sum(epc * q_scale * pn + rs);
+      if (g4 == 0 && 16 * wave + c < nn) nq[(int64_t)(t0 + 16 * wave + c) * H + h] = x;
+    }
+    const float pe = pend;
+    if (more) {
+      fetch_scores(b + 1);
+      fetch_vectors(b + 1);
+    }
 #pragma unroll
     for (int ct = 0; ct < CT; ++ct) {
       const int e = e0 + 16 * ct + c;
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int i = 16 * wave + 4 * g4 + r;
-        if (i < nn && e < cols) {
-          if (e < Dv) out[((int64_t)(t0 + i) * H + h) * Dv + e] = o[ct][r];
-          else nq[(int64_t)(t0 + i) * H + h] = o[ct][r];
-        }
+        if (i < nn && e < Dv) out[((int64_t)(t0 + i) * H + h) * Dv + e] = o[ct][r];
       }
     }
     // S ← exp(P_end) S + Kᵀ (exp(P_end - P) u): this wave's row tiles, k running over the block's tokens
@@ -535,30 +676,42 @@ __global__ __launch_bounds__(NT) void scan_walk_kernel(const A* __restrict__ q, 
     for (int i = 0; i < DW; ++i)
       if (wave + 4 * i < DT) {
         const int d = 16 * (wave + 4 * i) + c;
+        float kn = 0.f;
 #pragma unroll
         for (int ct = 0; ct < CT; ++ct)
 #pragma unroll
-          for (int r = 0; r < 4; ++r) S[i][ct][r] *= pend;
+          for (int r = 0; r < 4; ++r) S[i][ct][r] *= pe;
 #pragma unroll
         for (int s = 0; s < 4; ++s) {
-          f32x4 kt;
-#pragma unroll
-          for (int j = 0; j < 4; ++j) kt[j] = d < D ? ldf<A>(k + (int64_t)(t0 + min(16 * s + 4 * g4 + j, nn - 1)) * k_stride + g * D + d) : 0.f;
+          f32x4 ka = Raw<A>::cvt(kt[i][s]);
+          if (d >= D) ka = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
           for (int ct = 0; ct < CT; ++ct)
-            S[i][ct] = mfma_k16(kt, *reinterpret_cast<const f32x4*>(Us + (16 * ct + c) * BS + 16 * s + 4 * g4), S[i][ct]);
+            S[i][ct] = mfma_k16(ka, *reinterpret_cast<const f32x4*>(Us + (16 * ct + c) * BS + 16 * s + 4 * g4), S[i][ct]);
+          if (norm) {
+            const float* w4 = ews[b & 1] + 16 * s + 4 * g4;
+            kn += (ka[0] * w4[0] + ka[1] * w4[1]) + (ka[2] * w4[2] + ka[3] * w4[3]);
+          }
+        }
+        if (norm) {
+          kn = group_sum(kn);
+          if (g4 == 0) ns[d] = pe * ns[d] + kn;
         }
       }
+    if (more) fetch_columns(b + 1);
   }
 #pragma unroll
-  for (int i = 0; i < DW; ++i)
+  for (int i = 0; i < DW; ++i) {
 #pragma unroll
     for (int ct = 0; ct < CT; ++ct)
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int d = 16 * (wave + 4 * i) + 4 * g4 + r, e = e0 + 16 * ct + c;
-        if (d < D && e < cols) *state_at(head, D, Dv, d, e) = S[i][ct][r];
+        if (d < D && e < Dv) head[(int64_t)d * Dv + e] = S[i][ct][r];
       }
+    const int d = 16 * (wave + 4 * i) + c;
+    if (norm && g4 == 0 && d < D) head[(int64_t)D * Dv + d] = ns[d];
+  }
 }
 
 }  // namespace
@@ -628,12 +781,12 @@ int64_t gm_scan_ws_floats(int rows, int seqs, int H, bool delta) {
 template <typename A, bool DELTA>
 static void gated_scan(const A* q, int64_t q_stride, const A* k, int64_t k_stride, const A* v, int64_t v_stride, const float* decay,
                        const float* weight, float* state, const int* positions, const int* qsl, const int* state_slots,
-                       const int* counts, int seqs, int H, int G, int D, int Dv, int cols, float q_scale, float* out, float* nq,
+                       const int* counts, int seqs, int H, int G, int D, int Dv, float q_scale, float* out, float* nq,
                        const int* tile_seq, const int* tile_q0, int num_tiles, float* ws, hipStream_t stream) {
   const bool blocks = num_tiles > 0 && ws != nullptr && D <= GM_BLOCK_MAX_D;
 #define GM_STEP(DR)                                                                                                                   \
-  hipLaunchKernelGGL((scan_step_kernel<A, DR, DELTA>), dim3(seqs, H, (cols + 63) / 64), dim3(NT), 0, stream, q, q_stride, k, k_stride, \
-                     v, v_stride, decay, weight, state, positions, qsl, state_slots, counts, H, G, D, Dv, cols, q_scale, out, nq,     \
+  hipLaunchKernelGGL((scan_step_kernel<A, DR, DELTA>), dim3(H, (Dv + 63) / 64, seqs), dim3(NT), 0, stream, q, q_stride, k, k_stride, \
+                     v, v_stride, decay, weight, state, positions, qsl, state_slots, counts, H, G, D, Dv, q_scale, out, nq,           \
                      blocks ? 1 : 0)
   const int dr = (D + 3) / 4;
   if (dr <= 8) GM_STEP(8);
@@ -643,16 +796,16 @@ static void gated_scan(const A* q, int64_t q_stride, const A* k, int64_t k_strid
   else GM_STEP(128);
 #undef GM_STEP
   if (!blocks) return;
-  const int wide = D % 4 == 0 && q_stride % 4 == 0 && k_stride % 4 == 0 && al16(q) && al16(k);
+  const int wide = D % 4 == 0 && q_stride % 4 == 0 && k_stride % 4 == 0 && al16(q) && al16(k);     // 4 entries at a time
   hipLaunchKernelGGL((scan_block_kernel<A, DELTA>), dim3(num_tiles, H), dim3(NT), 0, stream, q, q_stride, k, k_stride, decay, weight, qsl,
                      state_slots, counts, tile_seq, tile_q0, num_tiles, H, G, D, wide, q_scale, ws);
-  const int ct = H * ((cols + 31) / 32) >= 128 ? 2 : 1;   // 32 state columns per workgroup where that still leaves enough of them
+  const int ct = H * ((Dv + 31) / 32) >= 128 ? 2 : 1;   // 32 state columns per workgroup where that still leaves enough of them
   const int DS = ((D + 15) / 16) * 16 + 4;
   const size_t lds = (size_t)16 * ct * (DS + (DELTA ? 3 : 2) * BS) * sizeof(float);
-  const dim3 grid(seqs, H, (cols + 16 * ct - 1) / (16 * ct));
+  const dim3 grid(H, (Dv + 16 * ct - 1) / (16 * ct), seqs);
 #define GM_WALK(DT, CTV)                                                                                                               \
   hipLaunchKernelGGL((scan_walk_kernel<A, DELTA, DT, CTV>), grid, dim3(NT), lds, stream, q, q_stride, k, k_stride, v, v_stride, state,  \
-                     positions, qsl, state_slots, counts, H, G, D, Dv, cols, wide, q_scale, ws, out, nq)
+                     positions, qsl, state_slots, counts, H, G, D, Dv, wide, q_scale, ws, out, nq)
 #define GM_WALK_D(DT)          \
   do {                         \
     if (ct == 2) GM_WALK(DT, 2); \
@@ -671,10 +824,10 @@ void launch_gm_gated_scan(const void* q, int64_t q_stride, const void* k, int64_
                           bool normaliser, float* out, float* nq, const int* tile_seq, const int* tile_q0, int num_tiles, float* ws,
                           hipStream_t stream) {
   if (seqs == 0) return;
-  const int cols = Dv + (normaliser ? 1 : 0);
+  if (!normaliser) nq = nullptr;
 #define GM_SCAN(DELTA)                                                                                                                 \
   GM_BF16(bf16, A, (gated_scan<A, DELTA>((const A*)q, q_stride, (const A*)k, k_stride, (const A*)v, v_stride, decay, weight, state,     \
-                                         positions, qsl, state_slots, counts, seqs, H, G, D, Dv, cols, q_scale, out, nq, tile_seq,     \
+                                         positions, qsl, state_slots, counts, seqs, H, G, D, Dv, q_scale, out, nq, tile_seq,           \
                                          tile_q0, num_tiles, ws, stream)))
   if (delta) GM_SCAN(true);
   else GM_SCAN(false);

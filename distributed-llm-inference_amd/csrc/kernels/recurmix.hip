@@ -82,7 +82,7 @@ template <typename A, int V> struct Vec {
 //
 // Where the step brings one token of a sequence, the thread that owns a channel also moves its state rows on.  unit.n > 0: the
 // first n · d results are n vectors that leave at unit length (the first `scaled` of them times `scale`); they wait in LDS for
-// their sums.  gate.kind > 0: log decay and input weight of the token's heads (see GateArgs).
+// their sums.  gridDim.y workgroups share a token's channels, `span` each.  gate.kind > 0: log decay and input weight of the token's heads (see GateArgs).
 struct ConvUnit {
   int n, d, scaled;
   float scale;
@@ -146,13 +146,14 @@ __global__ __launch_bounds__(NT) void causal_conv_kernel(const A* __restrict__ x
                                                          const float* __restrict__ bias, int taps, float* state,
                                                          const int* __restrict__ positions, const int* __restrict__ token_seq,
                                                          const int* __restrict__ qsl, const int* __restrict__ state_slots, int C,
-                                                         O* __restrict__ out, int silu, ConvUnit unit, GateArgs<A> gate) {
-  extern __shared__ float vecs[];                                 // [unit.n · unit.d]
+                                                         O* __restrict__ out, int silu, ConvUnit unit, GateArgs<A> gate, int span) {
+  extern __shared__ float vecs[];                                 // this workgroup's vectors
   const int64_t t = blockIdx.x;
   const int seq = token_seq[t];
+  const int c0 = blockIdx.y * span, c1 = min(c0 + span, C);       // span: a multiple of unit.d where there are vectors
   if (seq < 0 || state_slots[seq] < 0) {                         // padding row
-    for (int c = threadIdx.x; c < C; c += NT) stf<O>(out + t * C + c, 0.f);
-    if (gate.kind != 0)
+    for (int c = c0 + threadIdx.x; c < c1; c += NT) stf<O>(out + t * C + c, 0.f);
+    if (gate.kind != 0 && blockIdx.y == 0)
       for (int h = threadIdx.x; h < gate.H; h += NT) gate.decay[t * gate.H + h] = gate.weight[t * gate.H + h] = 0.f;
     return;
   }
@@ -162,14 +163,14 @@ __global__ __launch_bounds__(NT) void causal_conv_kernel(const A* __restrict__ x
   float* st = state + (int64_t)state_slots[seq] * (taps - 1) * C;
   const A* xr = x + t * x_stride;
   const int nu = unit.n * unit.d;
-  for (int c = threadIdx.x * V; c < C; c += NT * V) {
+  for (int c = c0 + threadIdx.x * V; c < c1; c += NT * V) {
     Vec<float, V> a = conv_taps<A, V>(xr, x_stride, w, bias, taps, st, p, back, C, c);
     if (single) shift_rows<A, V>(xr, st, taps, C, c);
     if (silu)
 #pragma unroll
       for (int k = 0; k < V; ++k) a.v[k] *= sigmoid_f(a.v[k]);
     if (c < nu) {
-      a.store(vecs + c);
+      a.store(vecs + (c - c0));
       continue;
     }
     Vec<O, V> o;
@@ -177,7 +178,7 @@ __global__ __launch_bounds__(NT) void causal_conv_kernel(const A* __restrict__ x
     for (int k = 0; k < V; ++k) o.v[k] = a.v[k];
     o.store(out + t * C + c);
   }
-  if (gate.kind != 0) {
+  if (gate.kind != 0 && blockIdx.y == gridDim.y - 1) {
     const A* gr = gate.g + t * x_stride;
     for (int h = threadIdx.x; h < gate.H; h += NT) {
       const float z = ldf<A>(gr + (gate.kind == 1 ? gate.H + h : h)) + gate.bias[h];
@@ -186,11 +187,12 @@ __global__ __launch_bounds__(NT) void causal_conv_kernel(const A* __restrict__ x
       gate.weight[t * gate.H + h] = gate.kind == 1 ? 1.f / (1.f + expf(-ldf<A>(gr + h))) : sp;
     }
   }
-  if (nu == 0) return;
+  if (c0 >= nu) return;
   __syncthreads();
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  for (int u = wave; u < unit.n; u += NT / 64) {                  // a wave per vector
-    const float* row = vecs + u * unit.d;
+  const int u0 = c0 / unit.d, u1 = min((c1 + unit.d - 1) / unit.d, unit.n);
+  for (int u = u0 + wave; u < u1; u += NT / 64) {                 // a wave per vector
+    const float* row = vecs + (u - u0) * unit.d;
     float ss = 0.f;
     for (int i = lane; i < unit.d; i += 64) ss += row[i] * row[i];
     const float inv = (u < unit.scaled ? unit.scale : 1.f) / sqrtf(wave_sum(ss) + 1e-6f);
@@ -611,12 +613,15 @@ void launch_rm_causal_conv(const void* x, bool bf16, int64_t x_stride, const flo
   if (rows == 0) return;
   const ConvUnit unit{unit_n, unit_d, unit_scaled, unit_scale};
   const int nu = unit_n * unit_d;
+  // about one trip per thread; a vector stays in one workgroup
+  const int step = nu > 0 ? (unit_d % 4 == 0 ? unit_d : 4 * unit_d) : 4;
+  const int span = (4 * NT + step - 1) / step * step;
 #define RM_CONV(VV)                                                                                                                  \
-  RM_BF16(bf16, A, RM_BF16(out_bf16, O, hipLaunchKernelGGL((causal_conv_kernel<A, O, VV>), dim3(rows), dim3(NT), nu * sizeof(float), \
+  RM_BF16(bf16, A, RM_BF16(out_bf16, O, hipLaunchKernelGGL((causal_conv_kernel<A, O, VV>), dim3(rows, (C + span - 1) / span), dim3(NT), std::min(nu, span) * sizeof(float), \
                                                            stream, (const A*)x, x_stride, w, bias, taps, state, positions, token_seq, \
                                                            qsl, state_slots, C, (O*)out, silu ? 1 : 0, unit,                          \
                                                            (GateArgs<A>{gate_kind, gate_heads, (const A*)gate, gate_rate, gate_bias,  \
-                                                                        decay, weight}))))
+                                                                        decay, weight}), span)))
   if (C % 4 == 0 && nu % 4 == 0 && x_stride % 4 == 0 && al16(x) && al16(w) && al16(bias) && al16(state) && al16(out)) RM_CONV(4);
   else RM_CONV(1);
 #undef RM_CONV

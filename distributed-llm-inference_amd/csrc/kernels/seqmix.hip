@@ -388,6 +388,39 @@ __global__ __launch_bounds__(NT) void rms_gate_kernel(const float* __restrict__ 
   }
 }
 
+// The same for slices of 4 · LP entries (LP lanes own one, a power of two up to 64) without planes, skip or leading gate: a slice
+// lives in registers, one pass, a grid over groups of four entries.
+template <typename G, typename O>
+__global__ __launch_bounds__(NT) void slice_gate_kernel(const float* __restrict__ o, const float* __restrict__ w, int wn, float eps,
+                                                        const G* __restrict__ gate, int64_t gate_stride, int64_t items, int N, int LP,
+                                                        O* __restrict__ out, int64_t out_stride, int silu, const float* __restrict__ div,
+                                                        const float* __restrict__ floor_, int dheads, const int* __restrict__ token_seq) {
+  const int64_t i = (int64_t)blockIdx.x * NT + threadIdx.x;
+  if (i >= items) return;                                  // items is a multiple of LP: whole slices leave together
+  const int64_t t = i / (N / 4);
+  const int c = (int)(i - t * (N / 4)) * 4;
+  const bool pad = token_seq != nullptr && token_seq[t] < 0;
+  f32x4 v = ld4<float>(o + t * N + c);
+  const f32x4 g = ld4<G>(gate + t * gate_stride + c);
+  if (div != nullptr) {                                    // (slices do not straddle heads: the launcher checks)
+    const int64_t h = t * dheads + c / (N / dheads);
+    const float inv = 1.f / (fmaxf(fabsf(div[h]), floor_[h]) + 1e-6f);
+    v = f32x4{v[0] * inv, v[1] * inv, v[2] * inv, v[3] * inv};
+  }
+  f32x4 ww = {1.f, 1.f, 1.f, 1.f};
+  if (w != nullptr) ww = ld4<float>(w + (wn == N ? c : c % wn));
+  float q = (v[0] * v[0] + v[1] * v[1]) + (v[2] * v[2] + v[3] * v[3]);
+  for (int s = LP >> 1; s > 0; s >>= 1) q += __shfl_xor(q, s, 64);
+  const float inv = 1.f / sqrtf(q / (float)(4 * LP) + eps);
+  f32x4 y;
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    const float a = 1.f / (1.f + expf(-g[j]));
+    y[j] = pad ? 0.f : v[j] * inv * ww[j] * (silu ? g[j] * a : a);
+  }
+  st4<O>(out + t * out_stride + c, y);
+}
+
 template <typename A>
 __global__ __launch_bounds__(NT) void relu2_kernel(const A* __restrict__ x, A* __restrict__ out, int64_t n) {
   for (int64_t i = (int64_t)blockIdx.x * NT + threadIdx.x; i < n; i += (int64_t)gridDim.x * NT) {
@@ -1296,6 +1329,16 @@ void launch_sm_rms_gate(const float* o, int parts, const float* w, int wn, float
   auto al = [](const void* p, uintptr_t a) { return reinterpret_cast<uintptr_t>(p) % a == 0; };
   const bool wide = N % 4 == 0 && (N / groups) % 4 == 0 && gate_stride % 4 == 0 && out_stride % 4 == 0 && skip_stride % 4 == 0 &&
                     al(o, 16) && al(gate, gate_bf16 ? 8 : 16) && al(out, out_bf16 ? 8 : 16) && al(skip, 16);
+  const int lp = N / groups / 4;
+  if (wide && parts == 1 && skip == nullptr && !gate_first && groups > 1 && lp <= 64 && (lp & (lp - 1)) == 0 && (w == nullptr || al(w, 16)) &&
+      (div == nullptr || dheads == groups)) {
+    const int64_t items = (int64_t)rows * N / 4;
+    SM_DISPATCH_BF16(gate_bf16, G, SM_DISPATCH_BF16(out_bf16, O, hipLaunchKernelGGL((slice_gate_kernel<G, O>), dim3((unsigned)((items + NT - 1) / NT)),
+                                                                                     dim3(NT), 0, stream, o, w, wn, eps, (const G*)gate, gate_stride,
+                                                                                     items, N, lp, (O*)out, out_stride, silu ? 1 : 0, div, floor_,
+                                                                                     dheads, token_seq)));
+    return;
+  }
 #define SM_RG(VV)                                                                                                                     \
   SM_DISPATCH_BF16(gate_bf16, G, SM_DISPATCH_BF16(out_bf16, O, hipLaunchKernelGGL((rms_gate_kernel<G, O, VV>), dim3(rows), dim3(NT),   \
                                                                                    N * sizeof(float), stream, o, parts, ps, w, wn, eps, \

@@ -31,7 +31,7 @@ std::tuple<Tensor, Tensor, Tensor> rm_causal_conv(const Tensor& x, const Tensor&
   check_i32(token_seq, "token_seq");
   TORCH_CHECK(token_seq.numel() >= T, "token_seq shorter than the batch");
   check_step_meta(positions, qsl, state_slots, counts, T, num_seqs);
-  TORCH_CHECK(unit_n >= 0 && unit_d >= 1 && unit_n * unit_d <= C && unit_n * unit_d * 4 <= kSmMaxLds, "unit vectors too wide");
+  TORCH_CHECK(unit_n >= 0 && unit_d >= 1 && unit_n * unit_d <= C && (4 * unit_d + 1024) * 4 <= kSmMaxLds, "unit vectors too wide");
   int64_t H = 0;
   const void* gp = nullptr;
   const float *rp = nullptr, *gbp = nullptr;
