@@ -14,6 +14,8 @@
                                                       # side benchmark: Sevelorn stacks beside their closest families
     python bench.py --mixers --models rodelix-lightning,sinilorn-recurrence,rodelix-latent_attention,sinilorn-latent,mixtral,sinilorn
                                                       # side benchmark: Sinilorn stacks beside their closest families
+    python bench.py --mixers --models rodelix-lightning,nefarax-delta,nefarax-mlstm,rodelix-attention,nefarax-pair,nefarax
+                                                      # side benchmark: Nefarax stacks beside their closest families
 
 One rank per GPU.  ``--tp`` consecutive ranks form one tensor-parallel replica (``dp = gpus / tp`` replicas);
 every replica serves its share (round-robin, the router's stateless policy) of ONE global BurstGPT-like trace

@@ -207,7 +207,7 @@ def run_one(mcfg, prompt, batch, new_tokens, device="cuda", graphs=True):
     sync()
     t_decode = time.perf_counter() - t0
     made = sum(r.num_output for r in reqs) - done0
-    return {"model": mcfg.name, "params_per_layer_M": round((mcfg.param_count() - 2 * mcfg.vocab_size * mcfg.hidden_size) / LAYERS / 1e6, 1),
+    return {"model": mcfg.name, "params_per_layer_M": round((mcfg.param_count() - (1 if mcfg.tie_embeddings else 2) * mcfg.vocab_size * mcfg.hidden_size) / LAYERS / 1e6, 1),
             "prompt": prompt, "batch": batch, "prefill_tokens_per_s": round(batch * prompt / t_prefill),
             "prefill_ms": round(t_prefill * 1e3, 2), "decode_tokens_per_s": round(made / t_decode),
             "decode_ms_per_step": round(t_decode / max(steps, 1) * 1e3, 3), "decode_steps": steps,
