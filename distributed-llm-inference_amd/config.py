@@ -42,15 +42,21 @@ class MixerSpec:
     ``gate_cap``, a normaliser vector beside the ``[D, Dv]`` state and a running maximum per head), ``"conv_attention"``
     (causal grouped-query attention whose q and k pass a convolution and half-split rotation; the values are the keys before
     rotation; a per-head sink in the denominator), ``"ssd"`` (Mamba-2: ``heads`` heads of ``vdim`` channels over ``kv_heads``
-    groups of ``dim`` state columns, gate before a norm over ``norm_groups`` parts) or ``"normed_pair"`` (the two mixers in
-    ``parts`` read the same input; half the sum of their outputs, each RMS-normed over the width)."""
+    groups of ``dim`` state columns, gate before a norm over ``norm_groups`` parts), ``"normed_pair"`` (the two mixers in
+    ``parts`` read the same input; half the sum of their outputs, each RMS-normed over the width), ``"masked_attention"``
+    (grouped-query softmax attention, q and k normed per head, half-split rotation of the leading ``rot_dims`` entries, keys
+    visible within a ``chunk`` or a ``window`` with ``keep_first`` kept tokens, scores soft-capped at ``score_cap``, a per-head
+    ``sink`` in the denominator; ``maps`` = 2: differential attention, two maps over the same values), ``"channel_delta"`` (the
+    gated delta rule with a decay per key channel from a projection of rank ``lora``, sigmoid output gate from one of rank
+    ``gate_lora``) or ``"scaled_pair"`` (the two mixers in ``parts`` read the same input; their outputs are summed with the weights
+    ``part_scales``)."""
     kind: str
     heads: int
     dim: int                            # per-head query / key size (latent attention: the unrotated part)
     vdim: int
     kv_heads: int = 0                   # attention: key / value heads
     scale: float = 1.0                  # multiplies q·k
-    window: int = 0                     # attention, gated latent attention: a query sees itself and the window-1 tokens before it (0: all)
+    window: int = 0                     # attention, gated latent / masked attention: a query sees itself and the window-1 tokens before it (0: all)
     kv_rank: int = 0                    # latent attention: size of the cached latent
     rot_dim: int = 0                    # latent attention: size of the rotated query / key part
     rot_base: float = 10000.0
@@ -58,9 +64,9 @@ class MixerSpec:
     decay: tuple = ()                   # lightning: per-head state decay
     rot_scaling: tuple = ()             # sink / gated latent attention: (factor, original length, fast turns, slow turns) or ();
                                         # conv attention: (factor, original length, high, low)
-    lora: int = 0                       # time mix: rank of the decay projection
-    parts: tuple = ()                   # parallel: the mixers run side by side (MixerSpec each)
-    part_scales: tuple = ()             # parallel: weight of every part's output
+    lora: int = 0                       # time mix, channel delta: rank of the decay projection
+    parts: tuple = ()                   # parallel, scaled / normed pair: the mixers run side by side (MixerSpec each)
+    part_scales: tuple = ()             # parallel, scaled pair: weight of every part's output
     ff: int = 0                         # feed-forward inner width (0: the layer has none); routed: of ONE expert
     ff_kind: str = "dense"              # "dense" | "moe" (sigmoid-routed squared-ReLU experts + optional gated shared expert)
     experts: int = 0                    # moe: number of routed experts
@@ -68,22 +74,31 @@ class MixerSpec:
     router_scale: float = 1.0           # moe: multiplies the chosen experts' scores
     shared_ff: int = 0                  # moe: inner width of the expert every token takes (0: none)
     kv_from: int = -1                   # gated (latent) attention: index of the layer whose cached rows this layer reads (-1: its own)
-    ff_act: str = "relu2"               # feed-forward activation: "relu2" | "gelu_tanh" / "silu" (gated) | "clamped" (gated experts)
+    ff_act: str = "relu2"               # feed-forward activation: "relu2" | "gelu_tanh" / "silu" (gated) | "clamped" (gated)
                                         # | "gelu_tanh_plain" (not gated)
     router: str = "sigmoid"             # moe: "sigmoid" (scores, not renormalised) | "softmax" (biased logits, softmax over the chosen)
                                         # | "softmax_all" (softmax over all logits, a choice bias, renormalised over the chosen)
     q_rank: int = 0                     # gated latent attention: size of the normed query latent
-    sink: bool = False                  # gated latent attention: a learned per-head logit in the softmax denominator
-    conv_taps: int = 0                  # rglru, delta, ssd, conv attention: taps of the causal convolution behind the projections
+    sink: bool = False                  # gated latent / masked attention: a learned per-head logit in the softmax denominator
+    conv_taps: int = 0                  # rglru, (channel) delta, ssd, conv attention: taps of the causal convolution behind the projections
     identity_experts: int = 0           # moe ("softmax_all"): trailing router outputs whose expert returns its input
-    ff_limit: float = 0.0               # moe ("clamped" experts): bound of the gate (above) and of the up projection (both sides)
+    ff_limit: float = 0.0               # "clamped": bound of the gate (above) and of the up projection (both sides)
     ff_bias: bool = False               # dense feed-forward: the three projections have biases
     gate_cap: float = 0.0               # mlstm: soft bound of the gates' pre-activations
     norm_groups: int = 1                # ssd: equal parts of the inner width that are normed on their own
+    chunk: int = 0                      # masked attention: keys of the query's own stretch of this many positions only (0: off)
+    keep_first: int = 0                 # masked attention: first tokens of the sequence that stay visible behind the window
+    score_cap: float = 0.0              # masked attention: score ← cap · tanh(score / cap) (0: off)
+    qk_weight: bool = False             # masked attention: the per-head norms of q and k have weights
+    maps: int = 1                       # masked attention: 2 = map 1 minus a learned multiple of map 2, normed per head
+    map_diff: float = 0.0               # masked attention, two maps: constant part of that multiple
+    gate_lora: int = 0                  # channel delta: rank of the output gate's projection
+    weights_of: int = -1                # index of the layer whose parameters this layer uses, with a cache of its own (-1: its own)
 
     @property
     def stateful(self) -> bool:
-        return (self.kind in ("lightning", "time_mix", "retention", "rglru", "delta", "mlstm", "ssd", "conv_attention")
+        return (self.kind in ("lightning", "time_mix", "retention", "rglru", "delta", "mlstm", "ssd", "conv_attention",
+                              "channel_delta")
                 or any(p.stateful for p in self.parts))
 
     @property
@@ -94,7 +109,9 @@ class MixerSpec:
             return self.kv_heads * self.dim, self.kv_heads * self.vdim
         if self.kind == "conv_attention":
             return self.kv_heads * self.dim, self.kv_heads * self.dim
-        if self.kind in ("parallel", "normed_pair"):
+        if self.kind == "masked_attention":
+            return self.kv_heads * self.maps * self.dim, self.kv_heads * self.vdim
+        if self.kind in ("parallel", "normed_pair", "scaled_pair"):
             return tuple(sum(w) for w in zip(*(p.cache_row for p in self.parts)))
         if self.kind == "latent_attention" or (self.kind == "gated_latent_attention" and self.kv_from < 0):
             return self.kv_rank + self.rot_dim, 0
@@ -102,13 +119,14 @@ class MixerSpec:
 
     @property
     def state_shape(self) -> tuple:
-        if self.kind in ("parallel", "normed_pair"):
+        if self.kind in ("parallel", "normed_pair", "scaled_pair"):
             return next((p.state_shape for p in self.parts if p.state_shape), ())
         if self.kind == "mlstm":                # the state's columns, then the normaliser
             return (self.heads, self.dim * (self.vdim + 1))
         if self.kind == "rglru":
             return (self.heads * self.dim,)
-        return (self.heads, self.dim, self.vdim) if self.kind in ("lightning", "time_mix", "retention", "delta", "ssd") else ()
+        return (self.heads, self.dim, self.vdim) if self.kind in ("lightning", "time_mix", "retention", "delta", "ssd",
+                                                                      "channel_delta") else ()
 
 
 @dataclass
@@ -179,6 +197,8 @@ class ModelConfig:
             return 2 * v * h + h + sum(_hyper_layer_params(m, h, self.streams, self.conv_taps) for m in self.layer_specs)
         if self.arch == "nefarax":
             return v * h + 2 * h + 1 + sum(_nefarax_layer_params(m, h) for m in self.layer_specs)
+        if self.arch == "mozalix":
+            return 2 * v * h + h + sum(_mozalix_layer_params(m, h) for m in self.layer_specs if m.weights_of < 0)
         if self.arch == "sinilorn":
             return 2 * v * h + h + sum(_sinilorn_layer_params(m, h, self.streams) for m in self.layer_specs)
         if self.layer_specs:
@@ -264,6 +284,20 @@ def _nefarax_layer_params(m: MixerSpec, h: int) -> int:
     cb = inner + 2 * b.kv_heads * b.dim
     return (tot + 2 * h + ca * (h + a.conv_taps) + a.heads + h * a.heads * a.dim
             + h * (inner + cb + b.heads) + cb * (b.conv_taps + 1) + 3 * b.heads + inner + h * inner)
+
+
+def _mozalix_layer_params(m: MixerSpec, h: int) -> int:
+    """Parameters of one Mozalix layer (norms, mixer, feed-forward)."""
+    tot = h + (3 * h * m.ff + 2 * m.ff + 2 * h if m.ff else 0)
+    for p in m.parts or (m,):
+        if p.kind == "masked_attention":
+            tot += h * (p.heads * p.maps * p.dim + p.kv_heads * (p.maps * p.dim + p.vdim)) + p.heads * p.vdim * h \
+                + (2 * p.dim if p.qk_weight else 0) + (p.heads if p.sink else 0) + (4 * p.dim if p.maps == 2 else 0)
+        else:
+            qk, v, d = p.kv_heads * p.dim, p.heads * p.vdim, p.heads * p.dim
+            tot += (h + p.conv_taps) * (2 * qk + v) + h * (p.heads + p.lora + p.gate_lora) + d * p.lora + v * p.gate_lora + p.heads + d \
+                + p.vdim + v * h
+    return tot
 
 
 def _rodelix_spec(entry: dict) -> MixerSpec:
@@ -502,8 +536,70 @@ def nefarax_config(cfg: dict, name: str = "nefarax", dtype: str = "bfloat16") ->
                        residual_mult=float(cfg.get("residual_mult", 1.0)))
 
 
+def _mozalix_attention(m: dict, need, **kw) -> MixerSpec:
+    rot, mask = m.get("rot") or {}, m.get("mask") or {}
+    s = MixerSpec(kind="masked_attention", heads=int(m["heads"]), kv_heads=int(m["kv_heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]),
+                  scale=float(m["scale"]), rot_base=float(rot.get("base", 10000.0)), rot_dims=int(rot.get("dims", 0)), **kw)
+    need(s.kv_heads >= 1 and s.heads % s.kv_heads == 0, f"{s.heads} query heads over {s.kv_heads} key/value heads")
+    need(s.rot_dims % 2 == 0 and 0 <= s.rot_dims <= s.dim, f"{s.rot_dims} rotated entries of {s.dim}")
+    need(int(mask.get("size", 0)) >= 1, "the mask needs a size")
+    need(s.keep_first >= 0, f"{s.keep_first} kept tokens")
+    return s
+
+
+def _mozalix_spec(entry: dict, index: int, layers: list, shapes: dict) -> MixerSpec:
+    def need(ok, what):
+        if not ok:
+            raise ValueError(f"layer {index}: {what}")
+
+    owner, chain = index, {index}
+    while layers[owner].get("weights_of") is not None:
+        owner = int(layers[owner]["weights_of"])
+        need(0 <= owner < len(layers) and owner not in chain, f"weights of layer {owner}")
+        need(all(entry.get(k) == layers[owner].get(k) for k in ("type", "mixer", "mlp")), f"differs from layer {owner}, whose weights it uses")
+        chain.add(owner)
+    m, mlp, kind = entry["mixer"], entry.get("mlp"), entry["type"]
+    ff = {}
+    if mlp:
+        need(mlp.get("kind") == "dense", f"unknown feed-forward kind {mlp.get('kind')!r}")
+        ff = dict(ff=int(mlp["ff"]), ff_kind="dense", ff_act="clamped", ff_limit=float(mlp["limit"]), ff_bias=True)
+        need(ff["ff_limit"] > 0.0, "the feed-forward's limit must be positive")
+    ff["weights_of"] = owner if owner != index else -1
+    if kind == "attention":
+        return _mozalix_attention(m, need, chunk=int(m["mask"]["size"]), sink=True, qk_weight=True, **ff)
+    if kind == "attention_2":
+        return _mozalix_attention(m, need, window=int(m["mask"]["size"]), qk_weight=True, maps=2, map_diff=float(m["diff"]), **ff)
+    need(kind == "parallel", f"unknown mixer type {kind!r}")
+    a, b = m["left"], m["right"]
+    left = _mozalix_attention(a, need, window=int(a["mask"]["size"]), keep_first=int(a["mask"].get("keep_first", 0)),
+                              score_cap=float(a["softcap"]))
+    need(left.score_cap > 0.0, "the soft cap must be positive")
+    # the ranks of the low-rank projections are tensor shapes, not configuration entries
+    rank = {}
+    for key, name in (("lora", "a1"), ("gate_lora", "g1")):
+        rank[key] = int(b.get(key) or shapes.get(f"l{owner}.mix.right.{name}", (0,))[0])
+        need(rank[key] >= 1, f"the rank of right.{name} is neither in the configuration nor a checkpoint tensor's shape")
+    right = MixerSpec(kind="channel_delta", heads=int(b["heads"]), kv_heads=int(b["kv_heads"]), dim=int(b["dim"]), vdim=int(b["vdim"]),
+                      conv_taps=int(b["conv"]), **rank)
+    need(right.heads % right.kv_heads == 0, f"{right.heads} heads over {right.kv_heads} query/key heads")
+    need(right.conv_taps >= 1, "a convolution has at least the current token's tap")
+    return MixerSpec(kind="scaled_pair", heads=left.heads, dim=left.dim, vdim=left.vdim, kv_heads=left.kv_heads, parts=(left, right),
+                     part_scales=(float(m["left_scale"]), float(m["right_scale"])), **ff)
+
+
+def mozalix_config(cfg: dict, name: str = "mozalix", dtype: str = "bfloat16", shapes: Optional[dict] = None) -> ModelConfig:
+    """``ModelConfig`` of a Mozalix checkpoint from the dict its ``config.json`` holds (``shapes``: tensor name → shape of the
+    checkpoint, for the ranks the configuration leaves to the tensors)."""
+    specs = tuple(_mozalix_spec(e, i, cfg["layers"], shapes or {}) for i, e in enumerate(cfg["layers"]))
+    return ModelConfig(name=name, arch="mozalix", vocab_size=int(cfg["vocab"]), hidden_size=int(cfg["width"]),
+                       intermediate_size=max([s.ff for s in specs] + [0]), num_layers=len(specs), num_heads=specs[0].heads,
+                       num_kv_heads=max(specs[0].kv_heads, 1), head_dim=specs[0].dim, max_position=1 << 24,
+                       rms_eps=float(cfg["norm"]["eps"]), dtype=dtype, bos_token_id=0, eos_token_id=-1, layer_specs=specs,
+                       embed_scale=float((cfg.get("embedding") or {}).get("scale", 1.0)))
+
+
 _CONFIG_READERS = {"Rodelix": rodelix_config, "Vibunex": vibunex_config, "Sevelorn": sevelorn_config, "Sinilorn": sinilorn_config,
-                   "Nefarax": nefarax_config}
+                   "Nefarax": nefarax_config, "Mozalix": mozalix_config}
 
 
 def safetensors_shapes(path: str) -> dict:
@@ -532,7 +628,7 @@ def load_model_config(path: str, dtype: Optional[str] = None) -> ModelConfig:
     if arch not in _CONFIG_READERS:
         raise ValueError(f"no reader for architecture {arch!r} (have {sorted(_CONFIG_READERS)})")
     kw = {"dtype": dtype} if dtype else {}
-    if arch == "Vibunex":
+    if arch in ("Vibunex", "Mozalix"):
         kw["shapes"] = safetensors_shapes(path)
     return _CONFIG_READERS[arch](raw, name=os.path.basename(os.path.normpath(path)) or arch.lower(), **kw)
 
@@ -659,6 +755,24 @@ MODEL_PRESETS: dict[str, ModelConfig] = {
                                 "rot": {"base": 10000.0, "dims": 8, "scaling": {"factor": 4.0, "high": 4.0, "low": 1.0, "original": 64}}},
                        "right": {"heads": 3, "vdim": 16, "state": 24, "groups": 1, "conv": 4, "norm_groups": 2}}}]},
         name="tiny-nefarax", dtype="float32"),
+    # post-norm layers on the unnormed stream: chunked attention with a sink, differential window attention, and soft-capped
+    # attention beside a delta rule with channel decays; the last layer runs on the first one's weights
+    "tiny-mozalix": mozalix_config({
+        "vocab": 272, "width": 88, "embedding": {"scale": 1.5}, "norm": {"eps": 1e-5},
+        "layers": [
+            {"type": "attention", "mlp": {"kind": "dense", "ff": 104, "limit": 3.0},
+             "mixer": {"heads": 6, "kv_heads": 2, "dim": 16, "vdim": 24, "scale": 0.25, "mask": {"size": 45}, "rot": {"base": 10000.0, "dims": 8}}},
+            {"type": "attention_2", "mlp": {"kind": "dense", "ff": 72, "limit": 1.5},
+             "mixer": {"heads": 4, "kv_heads": 2, "dim": 16, "vdim": 32, "scale": 0.2, "diff": 0.4, "mask": {"size": 29},
+                       "rot": {"base": 5000.0, "dims": 16}}},
+            {"type": "parallel", "mlp": None,
+             "mixer": {"left_scale": 0.8, "right_scale": 0.7,
+                       "left": {"heads": 3, "kv_heads": 1, "dim": 24, "vdim": 16, "scale": 0.3, "softcap": 8.0,
+                                "mask": {"size": 21, "keep_first": 3}},
+                       "right": {"heads": 4, "kv_heads": 2, "dim": 16, "vdim": 24, "conv": 3, "lora": 8, "gate_lora": 12}}},
+            {"type": "attention", "weights_of": 0, "mlp": {"kind": "dense", "ff": 104, "limit": 3.0},
+             "mixer": {"heads": 6, "kv_heads": 2, "dim": 16, "vdim": 24, "scale": 0.25, "mask": {"size": 45}, "rot": {"base": 10000.0, "dims": 8}}}]},
+        name="tiny-mozalix", dtype="float32"),
     "tiny-opt": ModelConfig(name="tiny-opt", arch="opt", vocab_size=512, hidden_size=64,
                             intermediate_size=128, num_layers=2, num_heads=4, num_kv_heads=4,
                             head_dim=16, max_position=512, pos_offset=2, tie_embeddings=True,

@@ -17,6 +17,7 @@ from ..config import ModelConfig
 from ..parallel.state import SINGLE, ParallelContext
 from .layers import random_full_tensor
 from .llama import LlamaForCausalLM
+from .mozalix import MozalixForCausalLM
 from .nefarax import NefaraxForCausalLM
 from .opt import OPTForCausalLM
 from .rodelix import RodelixForCausalLM
@@ -26,7 +27,7 @@ from .vibunex import VibunexForCausalLM
 
 _ARCH = {"llama": LlamaForCausalLM, "mixtral": LlamaForCausalLM, "opt": OPTForCausalLM, "rodelix": RodelixForCausalLM,
          "vibunex": VibunexForCausalLM, "sevelorn": SevelornForCausalLM, "sinilorn": SinilornForCausalLM,
-         "nefarax": NefaraxForCausalLM}
+         "nefarax": NefaraxForCausalLM, "mozalix": MozalixForCausalLM}
 
 
 def torch_dtype(name: str) -> torch.dtype:
@@ -62,6 +63,9 @@ def init_random(model, seed: int = 0) -> None:
             w.init_const(0.5)
         elif kind == "eye":
             w.load_full(torch.eye(w.full_shape[0], dtype=torch.float32, device=w.data.device))
+        elif kind == "block_diag":                           # unit-gain blocks, zeros beside them
+            w.load_full(torch.block_diag(*(random_full_tensor(f"{name}.{i}", b, torch.float32, w.data.device, seed, b[1] ** -0.5)
+                                           for i, b in enumerate(w.blocks))))
         elif kind == "small":                                # per-head constants of order one (kept positive)
             w.load_full(random_full_tensor(name, w.full_shape, torch.float32, w.data.device, seed, 1.0).abs() * 0.5)
         elif w.data.dim() in (2, 3) and hasattr(model, "checkpoint_sources"):
@@ -127,6 +131,8 @@ def load_safetensors(model, path: str) -> None:
             keys = fused.get(name, [name])
             if keys[0] == "@cols":                                   # matrices side by side: concatenated along their columns
                 full = torch.cat([shards.get(k) for k in keys[1:]], dim=1)
+            elif keys[0] == "@diag":                                 # matrices along the diagonal, zeros beside them
+                full = torch.block_diag(*(shards.get(k) for k in keys[1:]))
             elif isinstance(keys[0], (list, tuple)):                   # stacked: one slice per entry (each a concatenation)
                 full = torch.stack([shards.cat(ks) for ks in keys])
             else:

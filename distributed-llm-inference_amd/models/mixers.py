@@ -49,6 +49,14 @@ without bias; the mixer optionally also through a short causal convolution over 
 ``SingleNormLayer`` runs one of these five and an optional tanh-GELU feed-forward on the same norm ``tanh(α x) · w + b`` of
 the stream: ``x += m · (mixer(h) + ff(h))`` — one input GEMM and, but for the pair, one output GEMM for both.
 
+* ``MaskedAttention`` – grouped-query attention with per-head q / k norms, partial half-split rotation, a chunk mask or a window with
+  kept first tokens, optionally soft-capped scores, a sink, or two differential maps over the same values;
+* ``ChannelDelta`` – the gated delta rule with a decay per key channel from a low-rank projection;
+* ``ScaledPair`` – these two on the same input, outputs summed with fixed weights.
+
+``PostNormLayer`` runs one of these three and an optional clamped feed-forward with biases, each reading the stream itself:
+``x += norm1(mixer(x))``, ``x += norm2(ff(x))`` (RMS, ``1 + w``).
+
 ``MixerLayer`` wraps one of the first three (and an optional dense feed-forward) in the sandwich
 ``x += m · norm_b(sublayer(norm(x)))`` with token shift in front of the mixer.  The residual stream ``x`` is
 fp32; GEMM operands are the model dtype.  Tensor parallelism is not implemented for these stacks.
@@ -725,10 +733,153 @@ class NormedPair(nn.Module):
         return self.left(proj[:, :n], meta, cache.parts[0]), self.right(proj[:, n:], meta, cache.parts[1])
 
 
+class MaskedAttention(nn.Module):
+    """Columns ``[q | k | v]`` of the layer's input GEMM, heads' outputs (times ``out_scale``) into ``out`` — in and out columns as for
+    ``DeltaRule``.  q and k are divided by their root mean square per head (times a shared weight where ``qk_weight``), then rotated.
+    ``maps`` = 2: q and k hold two vectors per head; ``o = a₁ - λ a₂`` with ``λ = exp(lq1 · lk1) - exp(lq2 · lk2) + map_diff``, divided by its root
+    mean square per head, times ``1 - map_diff``."""
+
+    def __init__(self, spec: MixerSpec, width: int, eps: float, ctx: ParallelContext, dtype, device, out_scale: float = 1.0):
+        super().__init__()
+        self.s, self.eps, self.out_scale = spec, eps, out_scale
+        H, G, D, Dv, M = spec.heads, spec.kv_heads, spec.dim, spec.vdim, spec.maps
+        assert M in (1, 2) and H % G == 0 and spec.rot_dims % 2 == 0 and spec.rot_dims <= D
+        assert M == 1 or not (spec.sink or spec.score_cap), "differential maps have plain softmaxes"
+        self.in_cols, self.out_cols = (H + G) * M * D + G * Dv, H * Dv
+        self.q_norm, self.k_norm = (_param((D,), ctx, device), _param((D,), ctx, device)) if spec.qk_weight else (None, None)
+        self.sink = _param((H,), ctx, device) if spec.sink else None
+        self.lam = _param((4, D), ctx, device) if M == 2 else None
+        self._lam = None                                                                     # derived at first use (after loading)
+        self.register_buffer("inv_freq", seqmix.rotary_inv_freq(spec.rot_base, spec.rot_dims, device), persistent=False)
+
+    def in_sources(self, p):
+        return [p + c for c in "qkv"]
+
+    def out_sources(self, p):
+        return [p + "o"]
+
+    def weights(self, p):
+        if self.q_norm is not None:
+            yield p + "q.norm", self.q_norm, "ones", None
+            yield p + "k.norm", self.k_norm, "ones", None
+        if self.sink is not None:
+            yield p + "sink", self.sink, "zeros", None
+        if self.lam is not None:
+            yield p + "lam", self.lam, "zeros", [[p + s] for s in ("lq1", "lk1", "lq2", "lk2")]
+
+    def cache(self, num_blocks, num_slots, dtype, device) -> LayerCache:
+        k, v = self.s.cache_row
+        return LayerCache(k=torch.zeros(num_blocks, KV_BLOCK_SIZE, k, dtype=dtype, device=device),
+                          v=torch.zeros(num_blocks, KV_BLOCK_SIZE, v, dtype=dtype, device=device))
+
+    def forward(self, proj, out, meta, cache: LayerCache):
+        s = self.s
+        H, G, D, Dv, M = s.heads, s.kv_heads, s.dim, s.vdim, s.maps
+        T = proj.shape[0]
+        if M == 2 and self._lam is None:
+            a = self.lam.data
+            self._lam = torch.exp((a[0] * a[1]).sum()) - torch.exp((a[2] * a[3]).sum()).reshape(1) + s.map_diff
+        qw, kw = (self.q_norm.data, self.k_norm.data) if self.q_norm is not None else (None, None)
+        q = seqmix.head_norm_rope_cache(proj, qw, kw, self.eps, meta.positions, self.inv_freq, s.rot_dims, meta.slot_mapping, cache.k, cache.v,
+                                        H, G, D, Dv, M)
+        if M == 1:
+            seqmix.token_attention(out.unflatten(1, (H, Dv)), q, None, cache.k, cache.v, meta, G, Dv, s.scale, s.window,
+                                   sink=self.sink.data if self.sink is not None else None, chunk=s.chunk, keep_first=s.keep_first,
+                                   cap=s.score_cap, out_scale=self.out_scale)
+            return
+        o = torch.empty(T, 2 * H, Dv, dtype=torch.float32, device=out.device)
+        seqmix.token_attention(o, q, None, cache.k, cache.v, meta, 2 * G, Dv, s.scale, s.window, chunk=s.chunk, keep_first=s.keep_first,
+                               value_heads=G)
+        seqmix.map_combine(o, self._lam, self.eps, (1.0 - s.map_diff) * self.out_scale, G, out, meta.token_seq)
+
+
+class ChannelDelta(nn.Module):
+    """Per head: ``S ← g ⊙ S`` (a decay per row, i.e. key channel), ``u = β (v - Sᵀ k)``, ``S ← S + k uᵀ``, ``o = Sᵀ q``; each head's ``o`` divided by its
+    root mean square, times a weight shared by the heads, times ``sigmoid(W_g2 W_g1 h)``.  ``g = exp(-exp(A) softplus(W_a2 W_a1 h + bias))``.
+    Both low-rank projections are one block-diagonal product over their neighbouring columns.  In and out columns as for
+    ``DeltaRule``; the result is multiplied by ``out_scale``."""
+
+    def __init__(self, spec: MixerSpec, width: int, eps: float, ctx: ParallelContext, dtype, device, out_scale: float = 1.0):
+        super().__init__()
+        self.s, self.eps, self.out_scale = spec, eps, out_scale
+        H, G, D, Dv, R, Rg = spec.heads, spec.kv_heads, spec.dim, spec.vdim, spec.lora, spec.gate_lora
+        assert R >= 1 and Rg >= 1, "the low-rank projections need ranks"
+        self.conv_cols = 2 * G * D + H * Dv
+        self.in_cols, self.out_cols = self.conv_cols + R + Rg + H, H * Dv                       # q | k | v | decay rank | gate rank | β
+        self.low = Weight((H * D + H * Dv, R + Rg), None, ctx, dtype, device)
+        self.low.blocks = ((H * D, R), (H * Dv, Rg))
+        self.conv = _param((self.conv_cols, spec.conv_taps), ctx, device)
+        self.A_log, self.dt_bias, self.norm = _param((H,), ctx, device), _param((H * D,), ctx, device), _param((Dv,), ctx, device)
+        self._taps = self._rate = self._norm = None                                             # derived at first use (after loading)
+
+    def in_sources(self, p):
+        return [p + c for c in ("q", "k", "v", "a1", "g1", "b")]
+
+    def out_sources(self, p):
+        return [p + "o"]
+
+    def weights(self, p):
+        yield p + "low", self.low, "block_diag", ["@diag", p + "a2", p + "g2"]
+        yield p + "conv", self.conv, "small", [p + "q.conv", p + "k.conv", p + "v.conv"]
+        yield p + "A_log", self.A_log, "zeros", None
+        yield p + "dt_bias", self.dt_bias, "zeros", None
+        yield p + "norm", self.norm, "ones", None
+
+    def cache(self, num_blocks, num_slots, dtype, device) -> LayerCache:
+        s = self.s
+        return LayerCache(state=torch.zeros(num_slots, *s.state_shape, dtype=torch.float32, device=device),
+                          shift=torch.zeros(num_slots, s.conv_taps - 1, self.conv_cols, dtype=torch.float32, device=device))
+
+    def forward(self, proj, out, meta, cache: LayerCache):
+        s = self.s
+        H, G, D, Dv, C, R = s.heads, s.kv_heads, s.dim, s.vdim, self.conv_cols, s.lora + s.gate_lora
+        if self._taps is None:
+            self._taps, self._rate, self._norm = self.conv.data.t().contiguous(), torch.exp(self.A_log.data), self.norm.data * self.out_scale
+        low = ops.linear(proj[:, C:C + R], self.low.data)
+        qkv, _, beta = seqmix.causal_conv(proj[:, :C], self._taps, None, cache.shift, meta, torch.float32, act="silu",
+                                          unit=(2 * G, D, G, D ** -0.5), gates=("beta", proj[:, C + R:C + R + H], self._rate, self._rate))
+        o = seqmix.channel_delta_scan(qkv[:, :G * D], qkv[:, G * D:2 * G * D], qkv[:, 2 * G * D:], low[:, :H * D], self._rate,
+                                      self.dt_bias.data, beta, cache.state, meta, H, G, D, Dv)
+        seqmix.rms_gate(o, self._norm, self.eps, low[:, H * D:], out.dtype, groups=H, out=out, token_seq=meta.token_seq)
+
+
+class ScaledPair(nn.Module):
+    """``scale_l · left(h) + scale_r · right(h)``: the scales multiply the halves' activations, so that one GEMM over both side by side
+    (``[W_o left | W_o right]``) is the sum."""
+
+    def __init__(self, spec: MixerSpec, width: int, eps: float, ctx: ParallelContext, dtype, device):
+        super().__init__()
+        kinds = tuple(p.kind for p in spec.parts)
+        if kinds != ("masked_attention", "channel_delta"):
+            raise ValueError(f"the scaled pair is masked attention beside a channel-wise delta rule, not {kinds}")
+        self.left = MaskedAttention(spec.parts[0], width, eps, ctx, dtype, device, spec.part_scales[0])
+        self.right = ChannelDelta(spec.parts[1], width, eps, ctx, dtype, device, spec.part_scales[1])
+        self.in_cols, self.out_cols = self.left.in_cols + self.right.in_cols, self.left.out_cols + self.right.out_cols
+
+    def in_sources(self, p):
+        return self.left.in_sources(p + "left.") + self.right.in_sources(p + "right.")
+
+    def out_sources(self, p):
+        return self.left.out_sources(p + "left.") + self.right.out_sources(p + "right.")
+
+    def weights(self, p):
+        yield from self.left.weights(p + "left.")
+        yield from self.right.weights(p + "right.")
+
+    def cache(self, num_blocks, num_slots, dtype, device) -> LayerCache:
+        return LayerCache(parts=tuple(m.cache(num_blocks, num_slots, dtype, device) for m in (self.left, self.right)))
+
+    def forward(self, proj, out, meta, cache: LayerCache):
+        n, m = self.left.in_cols, self.left.out_cols
+        self.left(proj[:, :n], out[:, :m], meta, cache.parts[0])
+        self.right(proj[:, n:n + self.right.in_cols], out[:, m:], meta, cache.parts[1])
+
+
 MIXERS = {"gated_attention": GatedAttention, "retention": Retention, "attention": WindowAttention, "latent_attention": LatentAttention, "lightning": LightningAttention,
           "sink_attention": SinkTalkAttention, "time_mix": TimeMix, "parallel": DualMixer, "rglru": GatedLinearRecurrence,
           "gated_latent_attention": GatedLatentAttention, "delta": DeltaRule, "mlstm": MatrixMemory, "conv_attention": ConvAttention,
-          "ssd": StateSpace, "normed_pair": NormedPair}
+          "ssd": StateSpace, "normed_pair": NormedPair, "masked_attention": MaskedAttention, "channel_delta": ChannelDelta,
+          "scaled_pair": ScaledPair}
 
 
 class DenseFF(nn.Module):
@@ -782,11 +933,12 @@ class RoutedFF(nn.Module):
 
 
 class GatedDenseFF(nn.Module):
-    """``W_down · (act(W_gate h) ⊙ W_up h)``; gate and up rows are one GEMM."""
+    """``W_down · (act(W_gate h) ⊙ W_up h)``; gate and up rows are one GEMM.  ``act`` "clamped": both sides bounded by ``limit``
+    (``seqmix.act_mul``)."""
 
-    def __init__(self, width: int, ff: int, act: str, ctx, dtype, device, bias: bool = False):
+    def __init__(self, width: int, ff: int, act: str, ctx, dtype, device, bias: bool = False, limit: float = 0.0):
         super().__init__()
-        self.act = act
+        self.act, self.limit = act, limit
         self.gate_up, self.down = _matrix(2 * ff, width, ctx, dtype, device), _matrix(width, ff, ctx, dtype, device)
         self.gate_up_b = Weight((2 * ff,), None, ctx, dtype, device) if bias else None
         self.down_b = Weight((width,), None, ctx, dtype, device) if bias else None
@@ -800,8 +952,9 @@ class GatedDenseFF(nn.Module):
 
     def forward(self, h):
         if self.gate_up_b is None:
-            return ops.linear(seqmix.act_mul(ops.linear(h, self.gate_up.data), self.act), self.down.data)
-        return ops.linear(seqmix.act_mul(ops.linear(h, self.gate_up.data, self.gate_up_b.data), self.act), self.down.data, self.down_b.data)
+            return ops.linear(seqmix.act_mul(ops.linear(h, self.gate_up.data), self.act, self.limit), self.down.data)
+        return ops.linear(seqmix.act_mul(ops.linear(h, self.gate_up.data, self.gate_up_b.data), self.act, self.limit), self.down.data,
+                          self.down_b.data)
 
 
 class SoftmaxRoutedFF(nn.Module):
@@ -1011,6 +1164,49 @@ class SingleNormLayer(nn.Module):
         if F:
             seqmix.gelu_rows(both[:, :F], out=acts[:, m:])
         return ops.linear(acts, self.out.data), None
+
+
+class PostNormLayer(nn.Module):
+    """``x += norm1(mixer(x))``, ``x += norm2(ff(x))`` on the fp32 stream; the sublayers read ``x`` itself.  All projections of the mixer
+    that read it are one GEMM, its output projections one over the halves' activations side by side."""
+    ALIGN = 16                  # the fused projection's rows are padded to a multiple of this (the decode GEMM's tile)
+
+    def __init__(self, spec: MixerSpec, width: int, eps: float, ctx: ParallelContext, dtype, device):
+        super().__init__()
+        self.spec, self.eps, self.dtype = spec, eps, dtype
+        if spec.ff and (spec.ff_kind, spec.ff_act, spec.ff_bias) != ("dense", "clamped", True):
+            raise ValueError(f"post-norm layers take a clamped dense feed-forward with biases, not {spec.ff_kind!r} / {spec.ff_act!r}")
+        self.norm1 = _param((width,), ctx, device)
+        self.mixer = MIXERS[spec.kind](spec, width, eps, ctx, dtype, device)
+        self.pad = -self.mixer.in_cols % self.ALIGN
+        self.inp = _matrix(self.mixer.in_cols + self.pad, width, ctx, dtype, device)
+        self.out = _matrix(width, self.mixer.out_cols, ctx, dtype, device)
+        self.norm2 = _param((width,), ctx, device) if spec.ff else None
+        self.ff = GatedDenseFF(width, spec.ff, spec.ff_act, ctx, dtype, device, bias=True, limit=spec.ff_limit) if spec.ff else None
+
+    def weights(self, p):
+        yield p + "norm1", self.norm1, "zeros", None
+        yield p + "mix.in", self.inp, "normal", self.mixer.in_sources(p + "mix.") + ([f"@zeros:{self.pad}"] if self.pad else [])
+        yield from self.mixer.weights(p + "mix.")
+        yield p + "mix.out", self.out, "normal", ["@cols"] + self.mixer.out_sources(p + "mix.")
+        if self.ff is not None:
+            yield p + "norm2", self.norm2, "zeros", None
+            yield from self.ff.weights(p + "mlp.")
+
+    def cache(self, num_blocks, num_slots, dtype, device) -> LayerCache:
+        return self.mixer.cache(num_blocks, num_slots, dtype, device)
+
+    def forward(self, x, h, meta, cache: LayerCache, final_norm=None):
+        """``x``: fp32 stream ``[T, W]``, updated in place; ``h``: the same in the model dtype.  Returns the new ``x`` in the model dtype, or
+        its norm with the weight ``final_norm`` (the stack's last layer)."""
+        proj = ops.linear(h, self.inp.data)
+        acts = torch.zeros(h.shape[0], self.mixer.out_cols, dtype=h.dtype, device=h.device)      # padding rows of a captured step stay zero
+        self.mixer(proj[:, :self.mixer.in_cols], acts, meta, cache)
+        h = seqmix.post_norm_add(x, ops.linear(acts, self.out.data), self.norm1.data, self.eps, self.dtype,
+                                 final_norm if self.ff is None else None)
+        if self.ff is None:
+            return h
+        return seqmix.post_norm_add(x, self.ff(h), self.norm2.data, self.eps, self.dtype, final_norm)
 
 
 class GatedParallelLayer(nn.Module):

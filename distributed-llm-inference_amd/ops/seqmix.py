@@ -215,7 +215,8 @@ def token_attention(out: torch.Tensor, q1: torch.Tensor, q2: Optional[torch.Tens
                     v_cache: Optional[torch.Tensor], meta, G: int, Dv: int, scale: float, window: int = 0,
                     temp: Optional[torch.Tensor] = None, r1: Optional[torch.Tensor] = None,
                     r2: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None,
-                    sink: Optional[torch.Tensor] = None) -> torch.Tensor:
+                    sink: Optional[torch.Tensor] = None, chunk: int = 0, keep_first: int = 0, cap: float = 0.0,
+                    value_heads: int = 0, out_scale: float = 1.0) -> torch.Tensor:
     """Softmax attention of this step's tokens over their sequences' cached rows (which already hold this step's keys).
 
     ``q1 [T, H, D1]`` (and ``q2 [T, H, D2]``) against key rows ``[G, D1 + D2]``: ``score = (q1·k[:D1] + q2·k[D1:]) · scale ·
@@ -224,25 +225,30 @@ def token_attention(out: torch.Tensor, q1: torch.Tensor, q2: Optional[torch.Tens
     ``window`` > 0: a query at position ``p`` sees positions ``p-window+1 … p``; 0: all up to ``p``.  ``gate [T, H]``
     (pre-activation, row-strided view): head ``h``'s result is multiplied by ``sigmoid(gate[t, h])``.  Views may be strided
     (last dim contiguous).  ``sink`` fp32 ``[H]``: the softmax denominator of head ``h`` also holds ``exp(sink[h])`` (a logit
-    without key or value, not scaled).  Writes ``out [T, H, Dv]``."""
+    without key or value, not scaled).  ``chunk`` > 0: a query at position ``p`` sees positions from ``p - p % chunk`` on;
+    ``keep_first``: the sequence's first tokens that stay visible however far back the window ends; ``cap`` > 0: ``score ← cap ·
+    tanh(score / cap)``; ``value_heads`` (0: ``G``): number of value heads, each shared by ``G / value_heads`` consecutive key heads;
+    ``out_scale`` multiplies the result.  Writes ``out [T, H, Dv]`` (the activation type, or fp32)."""
+    Gv = value_heads or G
     if _act_ok(q1):
         lib = _hip()
+        opts = (chunk, keep_first, cap, Gv, out_scale)
         rows = -1
         if TILE_ATTENTION and q1.dtype == torch.bfloat16 and meta.num_prefill_tiles > 0:
             # prefill chunks: 64-query tiles on the matrix cores; the per-token kernel keeps the decode rows in front
             if lib.sm_tile_attention(out, q1, q2, k_cache, v_cache, meta.block_tables, meta.seq_lens, meta.query_start_loc,
                                      meta.prefill_tile_seq, meta.prefill_tile_q0, meta.num_prefill_tiles,
-                                     meta.counts if meta.counts_on_device else None, G, Dv, scale, window, temp, r1, r2, gate, sink):
+                                     meta.counts if meta.counts_on_device else None, G, Dv, scale, window, temp, r1, r2, gate, sink, *opts):
                 rows = meta.num_decode
         T, H = q1.shape[0], q1.shape[1]
         todo = T if rows < 0 else rows                       # tokens the tile kernel left (all of them in a pure decode step)
         if (HEAD_DECODE and todo > 0 and q1.dtype == torch.bfloat16 and H // G >= 8 and meta.num_prefill_tiles == (0 if rows < 0 else meta.num_prefill_tiles)
                 and lib.sm_head_decode_attention(out, q1, q2, k_cache, v_cache, meta.block_tables, meta.positions, meta.token_seq,
-                                                 G, Dv, scale, window, temp, r1, r2, todo, gate, sink)):
+                                                 G, Dv, scale, window, temp, r1, r2, todo, gate, sink, *opts)):
             rows = 0                                         # done with the heads as matrix-core columns
         if rows != 0:
             lib.sm_token_attention(out, q1, q2, k_cache, v_cache, meta.block_tables, meta.positions, meta.token_seq,
-                                   G, Dv, scale, window, temp, r1, r2, rows, gate, sink)
+                                   G, Dv, scale, window, temp, r1, r2, rows, gate, sink, *opts)
         return out
     T, H, D1 = q1.shape
     rowk = k_cache.shape[-1]
@@ -259,11 +265,11 @@ def token_attention(out: torch.Tensor, q1: torch.Tensor, q2: Optional[torch.Tens
             continue
         pos = meta.positions[t0:t1].long()
         L = int(pos[-1]) + 1
-        lo = max(int(pos[0]) - window + 1, 0) if window > 0 else 0
+        lo = max(int(pos[0]) - window + 1, 0) if window > 0 and not keep_first else 0
         j = torch.arange(lo, L)
         slots = meta.block_tables[i, j // KV_BLOCK_SIZE].long() * KV_BLOCK_SIZE + j % KV_BLOCK_SIZE
         K = kflat[slots].float().view(-1, G, Dk)
-        V = (vflat[slots].float().view(-1, G, vflat.shape[-1] // G))[..., :Dv]
+        V = (vflat[slots].float().view(-1, Gv, vflat.shape[-1] // Gv))[..., :Dv].repeat_interleave(G // Gv, dim=1)
         q = q1[t0:t1].float() if q2 is None else torch.cat([q1[t0:t1].float(), q2[t0:t1].float()], dim=-1)
         rep = H // G
         Kh, Vh = K.repeat_interleave(rep, dim=1), V.repeat_interleave(rep, dim=1)      # [L', H, ·]
@@ -273,9 +279,13 @@ def token_attention(out: torch.Tensor, q1: torch.Tensor, q2: Optional[torch.Tens
         dist = (pos[:, None] - j[None, :])                                             # [n, L']
         if r1 is not None:
             s = s - r1.view(1, H, 1) * torch.log1p(r2.view(1, H, 1) * dist.clamp(min=0).float().unsqueeze(1))
+        if cap > 0.0:
+            s = cap * torch.tanh(s / cap)
         hidden = dist < 0
         if window > 0:
-            hidden = hidden | (dist >= window)
+            hidden = hidden | ((dist >= window) & (j >= keep_first)[None, :])
+        if chunk > 0:
+            hidden = hidden | (j[None, :] < (pos - pos % chunk)[:, None])
         s = s.masked_fill(hidden.unsqueeze(1), float("-inf"))
         if sink is not None:
             pw = torch.softmax(torch.cat([s, sink.view(1, H, 1).expand(t1 - t0, H, 1)], dim=-1), dim=-1)[..., :-1]
@@ -284,7 +294,7 @@ def token_attention(out: torch.Tensor, q1: torch.Tensor, q2: Optional[torch.Tens
         o = torch.einsum("nhl,lhd->nhd", pw, Vh)
         if gate is not None:
             o = o * torch.sigmoid(gate[t0:t1].float()).unsqueeze(2)
-        out[t0:t1] = o.to(out.dtype)
+        out[t0:t1] = (o * out_scale).to(out.dtype)
     return out
 
 
@@ -631,14 +641,17 @@ def retention_prep(qkvg: torch.Tensor, positions: torch.Tensor, inv_freq: Option
     return x
 
 
-def act_mul(x: torch.Tensor, kind: str) -> torch.Tensor:
-    """``act(x[:, :F]) · x[:, F:]`` of rows ``[T, 2F]``; ``kind``: ``"gelu_tanh"`` (``0.5 z (1 + tanh(√(2/π) (z + 0.044715 z³)))``)
-    or ``"silu"``."""
-    assert kind in ("gelu_tanh", "silu")
+def act_mul(x: torch.Tensor, kind: str, limit: float = 0.0) -> torch.Tensor:
+    """``act(x[:, :F]) · x[:, F:]`` of rows ``[T, 2F]``; ``kind``: ``"gelu_tanh"`` (``0.5 z (1 + tanh(√(2/π) (z + 0.044715 z³)))``),
+    ``"silu"``, or ``"clamped"``: ``g = min(x[:, :F], limit)``, ``u = clamp(x[:, F:], ±limit)``, ``g · sigmoid(1.702 g) · (u + 1)``."""
+    assert kind in ("gelu_tanh", "silu", "clamped") and (limit > 0.0) == (kind == "clamped")
     if _act_ok(x):
-        return _hip().hm_act_mul(x, kind == "silu")
+        return _hip().hm_act_mul(x, kind == "silu", limit)
     F = x.shape[1] // 2
     a, b = x[:, :F].float(), x[:, F:].float()
+    if kind == "clamped":
+        a, b = a.clamp(max=limit), b.clamp(-limit, limit)
+        return (a * torch.sigmoid(1.702 * a) * (b + 1.0)).to(x.dtype)
     a = torch.nn.functional.gelu(a, approximate="tanh") if kind == "gelu_tanh" else torch.nn.functional.silu(a)
     return (a * b).to(x.dtype)
 
@@ -698,14 +711,15 @@ def causal_conv(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor], 
     unit length, ``v / sqrt(Σ v² + 1e-6)``, the first ``scaled`` of them times ``scale``.  ``gates = (kind, g, rate, gate_bias)`` (``g`` a view
     with ``x``'s row stride; ``rate``, ``gate_bias`` fp32 ``[H]``) also returns two fp32 ``[T, H]`` tensors, the log decay and the input
     weight of every head for ``gated_scan``: ``"delta"``, ``g = [β | decay]`` columns — ``-rate · softplus(decay + gate_bias)`` and
-    ``sigmoid(β)``; ``"ssd"``, ``g`` = step sizes — ``-rate · dt`` and ``dt = softplus(g + gate_bias)``."""
+    ``sigmoid(β)``; ``"ssd"``, ``g`` = step sizes — ``-rate · dt`` and ``dt = softplus(g + gate_bias)``; ``"beta"``, ``g`` = write strengths
+    (``rate`` and ``gate_bias`` are not used but size it) — zeros (the decay comes from elsewhere) and ``sigmoid(g)``."""
     assert act in ("none", "silu")
     if _act_ok(x):
         kind, g, rate, gb = gates if gates is not None else ("", None, None, None)
         n, d, scaled, scale = unit if unit is not None else (0, 1, 0, 1.0)
         out, decay, weight = _hip().rm_causal_conv(x, w, bias, state, meta.positions, meta.token_seq, meta.query_start_loc, meta.state_slots,
                                                    meta.counts, meta.num_seqs, out_dtype == torch.bfloat16, act == "silu", n, d, scaled,
-                                                   scale, {"": 0, "delta": 1, "ssd": 2}[kind], g, rate, gb, meta.num_prefill_tiles > 0)
+                                                   scale, {"": 0, "delta": 1, "ssd": 2, "beta": 3}[kind], g, rate, gb, meta.num_prefill_tiles > 0)
         return (out, decay, weight) if gates is not None else out
     taps, C = w.shape
     xf = x.float()
@@ -738,6 +752,8 @@ def causal_conv(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor], 
     if kind == "delta":
         H = rate.numel()
         return out, -rate * torch.nn.functional.softplus(g[:, H:].float() + gb, threshold=1e9), torch.sigmoid(g[:, :H].float())
+    if kind == "beta":
+        return out, torch.zeros(g.shape[0], rate.numel()), torch.sigmoid(g[:, :rate.numel()].float())
     dt = torch.nn.functional.softplus(g.float() + gb, threshold=1e9)
     return out, -rate * dt, dt
 
@@ -971,3 +987,99 @@ def gated_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.T
         if normaliser:
             flat[:, D * Dv:] = S[:, :, Dv]
     return o[:, :, :Dv].reshape(T, H * Dv), (o[:, :, Dv] if normaliser else None)
+
+
+# ====================================================================================== post-norm layers, masked attention
+# Ops of stacks whose sublayers read the unnormed stream and add a norm of their output, of attention with per-head norms, chunk /
+# window masks, capped scores or two differential maps, and of the delta rule with a decay per key channel (``models/mixers.py``:
+# ``PostNormLayer``, ``MaskedAttention``, ``ChannelDelta``, ``ScaledPair``).  GPU kernels: ``csrc/kernels/postmix.hip``
+# (``torch.ops.dli.pm_*``) beside extensions of the kernels above.
+def embed_rows(ids: torch.Tensor, table: torch.Tensor, scale: float, out_dtype: torch.dtype):
+    """``x = scale · table[ids]`` in fp32, and the same rows in ``out_dtype`` (what the first sublayer reads)."""
+    if table.is_cuda:
+        x, h = _hip().pm_embed_rows(ids, table, scale)
+        return x, h
+    x = table[ids.long()].float() * scale
+    return x, x.to(out_dtype)
+
+
+def post_norm_add(x: torch.Tensor, y: torch.Tensor, w: torch.Tensor, eps: float, out_dtype: torch.dtype,
+                  w2: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """In place on the fp32 stream: ``x += y / sqrt(mean(y²) + eps) · (1 + w)``.  Returns the new ``x`` in ``out_dtype`` — with ``w2``
+    its norm ``x / sqrt(mean(x²) + eps) · (1 + w2)`` instead."""
+    if x.is_cuda:
+        return _hip().pm_post_norm_add(x, y, w, eps, w2, out_dtype == torch.bfloat16)
+    yf = y.float()
+    x.add_(yf * torch.rsqrt((yf * yf).mean(-1, keepdim=True) + eps) * (1.0 + w))
+    if w2 is None:
+        return x.to(out_dtype, copy=True)
+    return (x * torch.rsqrt((x * x).mean(-1, keepdim=True) + eps) * (1.0 + w2)).to(out_dtype)
+
+
+def head_norm_rope_cache(proj: torch.Tensor, qw: Optional[torch.Tensor], kw: Optional[torch.Tensor], eps: float, positions: torch.Tensor,
+                         inv_freq: Optional[torch.Tensor], rot_dims: int, slot_mapping: torch.Tensor, k_cache: torch.Tensor,
+                         v_cache: torch.Tensor, H: int, G: int, D: int, Dv: int, maps: int = 1) -> torch.Tensor:
+    """``proj [T, (H + G)·maps·D + G·Dv]`` (row-strided view) = query vectors head by head (``maps`` of them each), key vectors
+    likewise, values.  Every query / key vector is divided by its root mean square and multiplied by ``qw`` / ``kw`` (fp32 ``[D]``, or
+    None); then entries ``i`` and ``i + rot_dims/2`` are turned by ``position · inv_freq[i]``.  Keys and values go to the token-major
+    cache rows ``slot_mapping`` (< 0: skipped).  Returns the queries ``[T, maps·H, D]`` ordered (key head, map, head of its group): query
+    vector ``i`` belongs to key vector ``i // (H/G)`` of a cache row."""
+    if _act_ok(proj):
+        return _hip().pm_head_norm_rope_cache(proj, qw, kw, eps, positions, inv_freq if rot_dims else None, rot_dims, slot_mapping,
+                                              k_cache, v_cache, H, G, D, Dv, maps)
+    T = proj.shape[0]
+    nq, nk = H * maps * D, G * maps * D
+
+    def one(v, w):
+        v = v * torch.rsqrt((v * v).mean(-1, keepdim=True) + eps)
+        v = v if w is None else v * w
+        return _turn_half(v, positions[:T], inv_freq, 1.0, rot_dims) if rot_dims else v
+
+    q = one(proj[:, :nq].float().reshape(T, H * maps, D), qw).view(T, G, H // G, maps, D).transpose(2, 3)
+    k = one(proj[:, nq:nq + nk].float().reshape(T, G * maps, D), kw)
+    keep = slot_mapping[:T] >= 0
+    s = slot_mapping[:T][keep].long()
+    k_cache.view(-1, nk)[s] = k.reshape(T, nk)[keep].to(k_cache.dtype)
+    v_cache.view(-1, G * Dv)[s] = proj[:, nq + nk:nq + nk + G * Dv][keep].to(v_cache.dtype)
+    return q.reshape(T, maps * H, D).to(proj.dtype)
+
+
+def map_combine(o: torch.Tensor, lam: torch.Tensor, eps: float, scale: float, G: int, out: torch.Tensor, token_seq: Optional[torch.Tensor] = None):
+    """Two attention maps per head, ``o`` fp32 ``[T, 2H, Dv]`` ordered (key head, map, head of its group): ``d = o₁ - lam · o₂`` (``lam`` fp32
+    ``[1]``), ``out[t, h] = scale · d / sqrt(mean(d²) + eps)`` in head order (``out [T, H·Dv]``, a row-strided view; rows with a negative
+    ``token_seq`` become zeros on the GPU)."""
+    T, H2, Dv = o.shape
+    if o.is_cuda:
+        _hip().pm_map_combine(o, lam, eps, scale, G, out, token_seq)
+        return
+    p = o.view(T, G, 2, H2 // (2 * G), Dv)
+    d = p[:, :, 0] - lam * p[:, :, 1]
+    out.copy_((d * torch.rsqrt((d * d).mean(-1, keepdim=True) + eps) * scale).reshape(T, -1).to(out.dtype))
+
+
+def channel_delta_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, z: torch.Tensor, rate: torch.Tensor, bias: torch.Tensor,
+                       weight: torch.Tensor, state: torch.Tensor, meta, H: int, G: int, D: int, Dv: int) -> torch.Tensor:
+    """Gated delta rule with a decay per key channel.  ``q``, ``k`` ``[T, G·D]`` and ``v`` ``[T, H·Dv]`` fp32 (row-strided views; head ``h`` uses
+    q / k head ``h // (H/G)``); ``z [T, H·D]`` (row-strided view): ``g = exp(-rate[h] · softplus(z + bias))`` (``rate`` fp32 ``[H]``, ``bias``
+    ``[H·D]``); ``weight`` fp32 ``[T, H]``.  Per sequence and head, token by token in fp32, with ``S`` the sequence's ``state[slot, h]`` ``[D, Dv]``
+    (zero at position 0), written back after the step's last token: ``S ← g ⊙ S`` (rows); ``S ← S + k (weight · (v - Sᵀ k))ᵀ``;
+    ``o = Sᵀ q``.  Returns fp32 ``[T, H·Dv]``."""
+    if _act_ok(z):
+        tiles = meta.num_prefill_tiles if BLOCK_SCAN else 0
+        return _hip().pm_channel_delta_scan(q, k, v, z, rate, bias, weight, state, meta.positions, meta.query_start_loc, meta.state_slots,
+                                            meta.counts, meta.num_seqs, H, G, D, Dv, meta.prefill_tile_seq if tiles else None,
+                                            meta.prefill_tile_q0 if tiles else None, tiles)
+    T = q.shape[0]
+    qf, kf = (t.reshape(T, G, D).repeat_interleave(H // G, dim=1) for t in (q, k))
+    vf = v.reshape(T, H, Dv)
+    g = torch.exp(-rate.view(1, H, 1) * torch.nn.functional.softplus(z.float() + bias, threshold=1e9).view(T, H, D))
+    o = torch.zeros(T, H, Dv)
+    for _i, t0, t1, slot in _seq_rows(meta):
+        S = state[slot].clone() if int(meta.positions[t0]) > 0 else torch.zeros(H, D, Dv)
+        for t in range(t0, t1):
+            S = g[t].unsqueeze(2) * S
+            u = weight[t].unsqueeze(1) * (vf[t] - torch.einsum("hde,hd->he", S, kf[t]))
+            S = S + kf[t].unsqueeze(2) * u.unsqueeze(1)
+            o[t] = torch.einsum("hde,hd->he", S, qf[t])
+        state[slot] = S
+    return o.view(T, H * Dv)
