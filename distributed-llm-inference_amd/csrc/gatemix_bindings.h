@@ -103,3 +103,49 @@ std::tuple<Tensor, Tensor> gm_gated_scan(const Tensor& q, const Tensor& k, const
                             num_tiles > 0 ? ws.data_ptr<float>() : nullptr, cur_stream(q));
   return {out, nq};
 }
+
+// the delta rule with a decay per key channel (see ops/seqmix.py: channel_delta_scan) → o fp32 [T, H·Dv]
+Tensor gm_channel_scan(const Tensor& q, const Tensor& k, const Tensor& v, const Tensor& z, const Tensor& rate, const Tensor& bias,
+                       const Tensor& weight, Tensor state, const Tensor& positions, const Tensor& qsl, const Tensor& state_slots,
+                       const Tensor& counts, int64_t num_seqs, int64_t H, int64_t G, int64_t D, int64_t Dv,
+                       const c10::optional<Tensor>& tile_seq, const c10::optional<Tensor>& tile_q0, int64_t num_tiles) {
+  const int64_t T = q.size(0);
+  TORCH_CHECK(G >= 1 && H >= 1 && H % G == 0 && D >= 1 && Dv >= 1 && D <= dli::gm_step_max_dim(), "head sizes: H a multiple of G, D up to ",
+              dli::gm_step_max_dim());
+  check_act_like(q, false, "q");
+  check_act_like(k, false, "k");
+  check_act_like(v, false, "v");
+  const bool zb = act_bf16(z, "z");
+  check_rows(q, "q");
+  check_rows(k, "k");
+  check_rows(v, "v");
+  check_rows(z, "z");
+  TORCH_CHECK(q.size(1) == G * D && k.size(0) == T && k.size(1) == G * D && v.size(0) == T && v.size(1) == H * Dv && z.size(0) == T &&
+                  z.size(1) == H * D, "q / k must be [T, G·D], v [T, H·Dv], z [T, H·D]");
+  check_f32(rate, "rate", H);
+  check_f32(bias, "bias", H * D);
+  check_f32(weight, "weight", T * H);
+  check_f32(state, "state");
+  TORCH_CHECK(state.dim() >= 2 && state.numel() == state.size(0) * H * D * Dv, "state must hold [slots][H][D · Dv]");
+  check_step_meta(positions, qsl, state_slots, counts, T, num_seqs);
+  Tensor out = at::empty({T, H * Dv}, state.options());
+  const int* tsp = nullptr;
+  const int* tqp = nullptr;
+  Tensor ws;
+  if (num_tiles > 0 && tile_seq.has_value() && tile_q0.has_value() && D <= dli::gm_block_max_dim()) {
+    check_i32(*tile_seq, "tile_seq");
+    check_i32(*tile_q0, "tile_q0");
+    TORCH_CHECK(tile_seq->numel() >= num_tiles && tile_q0->numel() >= num_tiles, "tile lists shorter than num_tiles");
+    tsp = tile_seq->data_ptr<int>();
+    tqp = tile_q0->data_ptr<int>();
+    ws = at::empty({dli::gm_channel_ws_floats((int)T, (int)num_seqs, (int)H, (int)D)}, state.options());
+  } else {
+    num_tiles = 0;
+  }
+  dli::launch_gm_channel_scan(q.data_ptr<float>(), q.stride(0), k.data_ptr<float>(), k.stride(0), v.data_ptr<float>(), v.stride(0), z.data_ptr(),
+                              zb, z.stride(0), rate.data_ptr<float>(), bias.data_ptr<float>(), weight.data_ptr<float>(), state.data_ptr<float>(),
+                              positions.data_ptr<int>(), qsl.data_ptr<int>(), state_slots.data_ptr<int>(), counts.data_ptr<int>(), (int)num_seqs,
+                              (int)H, (int)G, (int)D, (int)Dv, out.data_ptr<float>(), tsp, tqp, (int)num_tiles,
+                              num_tiles > 0 ? ws.data_ptr<float>() : nullptr, cur_stream(q));
+  return out;
+}

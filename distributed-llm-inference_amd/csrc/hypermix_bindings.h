@@ -77,13 +77,14 @@ Tensor hm_retention_prep(const Tensor& qkvg, const Tensor& positions, const c10:
   return out;
 }
 
-Tensor hm_act_mul(const Tensor& x, bool silu) {
+// limit > 0: the clamped gated form
+Tensor hm_act_mul(const Tensor& x, bool silu, double limit) {
   const bool bf = act_bf16(x, "x");
   check_rows(x, "x");
   TORCH_CHECK(x.size(1) % 2 == 0, "rows must hold gate | up");
   const int64_t F = x.size(1) / 2;
   Tensor out = at::empty({x.size(0), F}, x.options());
-  dli::launch_hm_act_mul(x.data_ptr(), bf, x.stride(0), (int)x.size(0), (int)F, silu, out.data_ptr(), cur_stream(x));
+  dli::launch_hm_act_mul(x.data_ptr(), bf, x.stride(0), (int)x.size(0), (int)F, silu, (float)limit, out.data_ptr(), cur_stream(x));
   return out;
 }
 

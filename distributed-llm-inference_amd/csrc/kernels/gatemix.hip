@@ -1,7 +1,7 @@
 // Kernels of the stacks with one tanh norm per layer and gated matrix states (models/mixers.py: SingleNormLayer, DeltaRule,
 // MatrixMemory, StateSpace; ops/seqmix.py): the residual update fused with the tanh norm, the plain GELU of a feed-forward,
 // exponential gates with a running maximum, and the recurrence itself — S ← a S + k uᵀ, o = Sᵀ q with a decay a and a weight per
-// head and token, u = weight · v or, for the delta rule, weight · (v - Sᵀ k).  (The convolutions in front of it, rotation and
+// head and token — or a decay per key channel, acting on the rows of S — u = weight · v or, for the delta rule, weight · (v - Sᵀ k).  (The convolutions in front of it, rotation and
 // cache write of the attention beside it and the norm / gate behind it are extensions of recurmix.hip and seqmix.hip.)
 //
 // Arithmetic: the stream, norms, gates, decays, the state and every product with it are fp32 (prefill blocks on the fp32 matrix
@@ -11,6 +11,8 @@
 // Step metadata (int32, static device buffers): positions[T], query_start_loc[B+1], state_slots[B] (< 0: none), tile_seq / tile_q0
 // (64-token prefill tiles), counts[2] / counts[3] = number of valid tiles / batch rows.
 #include <algorithm>
+#include <type_traits>
+#include <utility>
 
 #include "common.h"
 #include "kernels.h"
@@ -222,15 +224,35 @@ __global__ __launch_bounds__(NTH) void max_gates_kernel(const A* __restrict__ g,
 // Token by token: one workgroup per (sequence, head, 64 state columns); wave v keeps rows v·DR … of its lane's column in registers,
 // the workgroup of the first columns also the normaliser.  Serves single tokens (and, with single_only = 0, whole chunks: sizes
 // the block path does not take).
-template <typename A, int DRMAX, bool DELTA>
+//
+// Channel decays (Z, the type of z, not void; delta rule): g[d] = exp(-rate[h] · softplus(z[t, h, d] + bias[h, d])) instead of exp(decay).
+template <typename Z> struct ChannelArgs {
+  const Z* z;
+  int64_t stride;
+  const float *rate, *bias;
+};
+template <> struct ChannelArgs<void> {};
+template <typename Z> __device__ __forceinline__ float channel_decay(float z, float rate);
+template <> __device__ __forceinline__ float channel_decay<float>(float z, float rate) {
+  return expf(-rate * (fmaxf(z, 0.f) + log1pf(expf(-fabsf(z)))));
+}
+// bf16 projections: the hardware's exp2 / log2, the series of log1p where 1 + e would lose digits
+template <> __device__ __forceinline__ float channel_decay<uint16_t>(float z, float rate) {
+  const float e = fast_exp2(-1.4426950408889634f * fabsf(z));
+  const float l = e < 0.0625f ? e * (1.f - e * (0.5f - e * (0.33333333f - e * (0.25f - e * 0.2f)))) : 0.6931471805599453f * __builtin_amdgcn_logf(1.f + e);
+  return fast_exp2(-1.4426950408889634f * rate * (fmaxf(z, 0.f) + l));
+}
+
+template <typename A, int DRMAX, bool DELTA, typename Z>
 __global__ __launch_bounds__(NT) void scan_step_kernel(const A* __restrict__ q, int64_t q_stride, const A* __restrict__ k, int64_t k_stride,
                                                        const A* __restrict__ v, int64_t v_stride, const float* __restrict__ decay,
                                                        const float* __restrict__ weight, float* __restrict__ state,
                                                        const int* __restrict__ positions, const int* __restrict__ qsl,
                                                        const int* __restrict__ state_slots, const int* __restrict__ counts, int H, int G,
                                                        int D, int Dv, float q_scale, float* __restrict__ out, float* __restrict__ nq,
-                                                       int single_only) {
-  __shared__ float qs[DRMAX * 4], ks[DRMAX * 4], red[4][64], red2[4][64], sred[NT / 64];
+                                                       int single_only, ChannelArgs<Z> ch) {
+  constexpr bool CHAN = !std::is_void_v<Z>;
+  __shared__ float qs[DRMAX * 4], ks[DRMAX * 4], gs[CHAN ? DRMAX * 4 : 1], red[4][64], red2[4][64], sred[NT / 64];
   const int h = blockIdx.x, seq = blockIdx.z;
   if (seq >= counts[3]) return;
   const int t0 = qsl[seq], t1 = qsl[seq + 1];
@@ -257,15 +279,16 @@ __global__ __launch_bounds__(NT) void scan_step_kernel(const A* __restrict__ q, 
     for (int d = threadIdx.x; d < D; d += NT) {
       qs[d] = ldf<A>(q + (int64_t)t * q_stride + g * D + d);
       ks[d] = ldf<A>(k + (int64_t)t * k_stride + g * D + d);
+      if constexpr (CHAN) gs[d] = channel_decay<Z>(ldf<Z>(ch.z + (int64_t)t * ch.stride + (int64_t)h * D + d) + ch.bias[(int64_t)h * D + d], ch.rate[h]);
     }
-    const float a = expf(decay[(int64_t)t * H + h]), wt = weight[(int64_t)t * H + h];
+    const float a = CHAN ? 1.f : expf(decay[(int64_t)t * H + h]), wt = weight[(int64_t)t * H + h];
     float ve = active ? ldf<A>(v + (int64_t)t * v_stride + (int64_t)h * Dv + e) : 0.f;
     __syncthreads();
     float seen = 0.f;
 #pragma unroll
     for (int i = 0; i < DRMAX; ++i)
       if (i < dn) {
-        S[i] *= a;
+        S[i] *= CHAN ? gs[d0 + i] : a;
         if (DELTA) seen += S[i] * ks[d0 + i];
       }
     if (DELTA) {
@@ -330,6 +353,30 @@ template <typename A> __device__ __forceinline__ f32x4 row4(const A* row, int d,
 #pragma unroll
   for (int j = 0; j < 4; ++j) r[j] = d + j < D ? ldf<A>(row + d + j) : 0.f;
   return r;
+}
+
+// one wave: column `lane` of (I + M)⁻¹ by forward substitution, rows of M [64][BS] (strictly lower part) broadcast from LDS
+__device__ __forceinline__ void unit_lower_inverse(const float* M, float* __restrict__ wi, int lane) {
+  float x[BT];
+#pragma unroll
+  for (int t = 0; t < BT; ++t) {
+    float a0 = t == lane ? 1.f : 0.f, a1 = 0.f, a2 = 0.f, a3 = 0.f;
+#pragma unroll
+    for (int s = 0; s < t; s += 4) {
+      const f32x4 m = *reinterpret_cast<const f32x4*>(M + t * BS + s);
+      a0 -= m[0] * x[s];
+      if (s + 1 < t) a1 -= m[1] * x[s + 1];
+      if (s + 2 < t) a2 -= m[2] * x[s + 2];
+      if (s + 3 < t) a3 -= m[3] * x[s + 3];
+    }
+    x[t] = (a0 + a1) + (a2 + a3);
+    wi[t * BT + lane] = x[t];
+  }
+}
+// sum over the four lane groups l>>4 (every lane gets it)
+__device__ __forceinline__ float group_sum(float v) {
+  v += __shfl_xor(v, 16, 64);
+  return v + __shfl_xor(v, 32, 64);
 }
 
 template <typename A, bool DELTA>
@@ -409,22 +456,181 @@ __global__ __launch_bounds__(NT) void scan_block_kernel(const A* __restrict__ q,
   if (!DELTA) return;
   __syncthreads();
   if (wave != 0) return;
-  // column `lane` of (I + M)⁻¹ by forward substitution, rows of M broadcast from LDS
-  float x[BT];
+  unit_lower_inverse(M, wi, lane);
+}
+
+// Channel decays.  With P_t[d] the log decays summed to token t inside the block, the same block form reads
+//   o_t = (q_t ⊙ e^{P_t}) S0 + Σ_{j ≤ t} (Σ_d q_t[d] k_j[d] e^{P_t[d] - P_j[d]}) u_j,  S = e^{P_end} ⊙ S0 + Σ_j (k_j ⊙ e^{P_end - P_j}) u_jᵀ,
+// and likewise with k_t for the system that u solves.  Every exponential here is a product of decays ≤ 1, never a quotient:
+// wave w holds rows 16w … of the block as A fragments (lane c = token, 4 channels); L = product from the sub-block's first token
+// through the lane's own, R = product from the next token to the sub-block's end, both prefix products over 16 lanes.  A sub-block
+// of rows meets an earlier sub-block of columns as (q ⊙ L) · (k ⊙ R ⊙ totals of the sub-blocks between)ᵀ on the fp32 matrix cores;
+// inside a sub-block, pairs at distance s use the running product of the s decays between them (lane rotations, no exponential).
+// Workspace per (block, head): A [64][64] | (I + M)⁻¹ [64][64] | weights [64] | e^{P_end} [DP] | q ⊙ e^{P} [64][DP] |
+// k ⊙ e^{P} [64][DP] | (k ⊙ e^{P_end - P})ᵀ [DP][64], DP = D rounded up to 16.
+__host__ __device__ constexpr int64_t channel_block_floats(int DP) { return 2 * BT * BT + BT + DP + 3 * (int64_t)BT * DP; }
+
+// value of the lane N below (ror: rotated within 16 lanes; shr / shl: `fill` where there is none)
+template <int N> __device__ __forceinline__ float row_ror(float v) {
+  if constexpr (N == 0) return v;
+  else return __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x120 + N, 0xf, 0xf, false));
+}
+template <int N> __device__ __forceinline__ float row_shr(float v, float fill) {
+  return __int_as_float(__builtin_amdgcn_update_dpp(__float_as_int(fill), __float_as_int(v), 0x110 + N, 0xf, 0xf, false));
+}
+template <int N> __device__ __forceinline__ float row_shl(float v, float fill) {
+  return __int_as_float(__builtin_amdgcn_update_dpp(__float_as_int(fill), __float_as_int(v), 0x100 + N, 0xf, 0xf, false));
+}
+
+// pairs (row c, column c - S) of a 16-token sub-block, S = 1 … 15: `e` holds the product of the S decays between them
+template <int S>
+__device__ __forceinline__ void near_pairs(const f32x4& q, const f32x4& k, const f32x4& g, f32x4& e, float* aq, float* ak) {
 #pragma unroll
-  for (int t = 0; t < BT; ++t) {
-    float a0 = t == lane ? 1.f : 0.f, a1 = 0.f, a2 = 0.f, a3 = 0.f;
-#pragma unroll
-    for (int s = 0; s < t; s += 4) {
-      const f32x4 m = *reinterpret_cast<const f32x4*>(M + t * BS + s);
-      a0 -= m[0] * x[s];
-      if (s + 1 < t) a1 -= m[1] * x[s + 1];
-      if (s + 2 < t) a2 -= m[2] * x[s + 2];
-      if (s + 3 < t) a3 -= m[3] * x[s + 3];
-    }
-    x[t] = (a0 + a1) + (a2 + a3);
-    wi[t * BT + lane] = x[t];
+  for (int j = 0; j < 4; ++j) {
+    e[j] *= row_ror<S - 1>(g[j]);
+    const float x = e[j] * row_ror<S>(k[j]);
+    aq[S] += q[j] * x;
+    ak[S] += k[j] * x;
   }
+}
+template <int... S>
+__device__ __forceinline__ void all_near_pairs(std::integer_sequence<int, S...>, const f32x4& q, const f32x4& k, const f32x4& g, float* aq,
+                                               float* ak) {
+  f32x4 e = {1.f, 1.f, 1.f, 1.f};
+  (near_pairs<S + 1>(q, k, g, e, aq, ak), ...);
+}
+
+template <typename Z>
+__global__ __launch_bounds__(NT) void channel_block_kernel(const float* __restrict__ q, int64_t q_stride, const float* __restrict__ k,
+                                                           int64_t k_stride, ChannelArgs<Z> ch, const float* __restrict__ weight,
+                                                           const int* __restrict__ qsl, const int* __restrict__ state_slots,
+                                                           const int* __restrict__ counts, const int* __restrict__ tile_seq,
+                                                           const int* __restrict__ tile_q0, int num_tiles, int H, int G, int D, int wide,
+                                                           float* __restrict__ ws) {
+  __shared__ float wt[BT];
+  __shared__ __align__(16) float M[BT * BS];
+  __shared__ __align__(16) float KR[2][BT][20], EM[2][4][16];
+  const int tile = blockIdx.x, h = blockIdx.y;
+  if (tile >= min(counts[2], num_tiles)) return;
+  const int seq = tile_seq[tile];
+  const int s0 = qsl[seq], s1 = qsl[seq + 1];
+  if (s1 - s0 < 2 || state_slots[seq] < 0) return;        // single tokens belong to the step kernel
+  const int t0 = s0 + tile_q0[tile];
+  const int n = min(BT, s1 - t0);
+  if (n <= 0) return;
+  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), g4 = lane >> 4, c = lane & 15;
+  const int g = h / (H / G), DP = (D + 15) & ~15;
+  float* wa = ws + ((int64_t)((t0 >> 6) + seq) * H + h) * channel_block_floats(DP);
+  float* wi = wa + BT * BT;
+  float* we = wi + BT * BT + BT;                          // e^{P_end}
+  float* wq = we + DP;
+  float* wk = wq + BT * DP;
+  float* wkt = wk + BT * DP;
+  if (wave == 0) wt[lane] = wi[BT * BT + lane] = lane < n ? weight[(int64_t)(t0 + lane) * H + h] : 0.f;
+  const int row = 16 * wave + c;
+  const bool live = row < n;
+  const int64_t tok = t0 + min(row, n - 1);               // rows past the block repeat its last token, with decay 1
+  const float* qr = q + tok * q_stride + g * D;
+  const float* kr = k + tok * k_stride + g * D;
+  const Z* zr = ch.z + tok * ch.stride + (int64_t)h * D;
+  const float* br = ch.bias + (int64_t)h * D;
+  const float rate = ch.rate[h];
+  f32x4 qk[3], kk[3];
+#pragma unroll
+  for (int s = 0; s < 3; ++s) qk[s] = kk[s] = f32x4{0.f, 0.f, 0.f, 0.f};
+  float aq[16], ak[16];
+#pragma unroll
+  for (int s = 0; s < 16; ++s) aq[s] = ak[s] = 0.f;
+  f32x4 qn = row4(qr, 4 * g4, D, wide), kn = row4(kr, 4 * g4, D, wide), zn = row4(zr, 4 * g4, D, wide), bn = row4(br, 4 * g4, D, wide);
+  for (int d0 = 0, it = 0; d0 < D; d0 += 16, ++it) {
+    const int d = d0 + 4 * g4, buf = it & 1;
+    const f32x4 qc = qn, kc = kn, zc = zn, bc = bn;
+    if (d0 + 16 < D) {                                    // the next channels are fetched while these are computed
+      qn = row4(qr, d + 16, D, wide);
+      kn = row4(kr, d + 16, D, wide);
+      zn = row4(zr, d + 16, D, wide);
+      bn = row4(br, d + 16, D, wide);
+    }
+    f32x4 gd, L, R, ql, kl, kR;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      gd[j] = live && d + j < D ? channel_decay<Z>(zc[j] + bc[j], rate) : 1.f;
+      float p = gd[j];
+      p *= row_shr<1>(p, 1.f);
+      p *= row_shr<2>(p, 1.f);
+      p *= row_shr<4>(p, 1.f);
+      p *= row_shr<8>(p, 1.f);
+      L[j] = p;
+      float r = row_shl<1>(gd[j], 1.f);
+      r *= row_shl<1>(r, 1.f);
+      r *= row_shl<2>(r, 1.f);
+      r *= row_shl<4>(r, 1.f);
+      r *= row_shl<8>(r, 1.f);
+      R[j] = r;
+      ql[j] = qc[j] * p;
+      kl[j] = kc[j] * p;
+      kR[j] = kc[j] * r;
+    }
+    *reinterpret_cast<f32x4*>(&KR[buf][row][4 * g4]) = kR;
+    if (c == 15) *reinterpret_cast<f32x4*>(&EM[buf][wave][4 * g4]) = L;
+    __syncthreads();                                      // (the other buffer's readers are past the barrier before this one)
+    f32x4 before = {1.f, 1.f, 1.f, 1.f}, behind = before;
+#pragma unroll
+    for (int b = 2; b >= 0; --b)
+      if (b < wave) {                                     // `before`: totals of the sub-blocks between b and this one
+        const f32x4 kb = *reinterpret_cast<const f32x4*>(&KR[buf][16 * b + c][4 * g4]);
+        const f32x4 f = {kb[0] * before[0], kb[1] * before[1], kb[2] * before[2], kb[3] * before[3]};
+        qk[b] = mfma_k16(ql, f, qk[b]);
+        kk[b] = mfma_k16(kl, f, kk[b]);
+        const f32x4 m = *reinterpret_cast<const f32x4*>(&EM[buf][b][4 * g4]);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) before[j] *= m[j];
+      }
+#pragma unroll
+    for (int b = 1; b < 4; ++b)
+      if (b > wave) {
+        const f32x4 m = *reinterpret_cast<const f32x4*>(&EM[buf][b][4 * g4]);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) behind[j] *= m[j];
+      }
+    f32x4 oq, ok;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      oq[j] = ql[j] * before[j];
+      ok[j] = kl[j] * before[j];
+      wkt[(int64_t)(d + j) * BT + row] = kR[j] * behind[j];
+      aq[0] += qc[j] * kc[j];
+    }
+    *reinterpret_cast<f32x4*>(wq + (int64_t)row * DP + d) = oq;
+    *reinterpret_cast<f32x4*>(wk + (int64_t)row * DP + d) = ok;
+    if (wave == 3 && c == 15)
+      *reinterpret_cast<f32x4*>(we + d) = f32x4{L[0] * before[0], L[1] * before[1], L[2] * before[2], L[3] * before[3]};
+    all_near_pairs(std::make_integer_sequence<int, 15>{}, qc, kc, gd, aq, ak);
+  }
+  // off-diagonal tiles
+#pragma unroll
+  for (int b = 0; b < 3; ++b)
+    if (b < wave) {
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int i = 16 * wave + 4 * g4 + r, col = 16 * b + c;
+        wa[i * BT + col] = qk[b][r];
+        M[i * BS + col] = wt[i] * kk[b][r];
+      }
+    }
+  // the diagonal tile: lane c's entry at distance s; the lanes that wrapped around hold nothing and clear the upper triangle
+  const float wr = wt[row];
+#pragma unroll
+  for (int s = 0; s < 16; ++s) {
+    const float x = group_sum(aq[s]), y = group_sum(ak[s]);
+    if (g4 == (s & 3)) {
+      const int col = 16 * wave + ((c - s) & 15);
+      wa[row * BT + col] = c >= s ? x : 0.f;
+      M[row * BS + col] = s > 0 && c >= s ? wr * y : 0.f;
+    }
+  }
+  __syncthreads();
+  if (wave == 0) unit_lower_inverse(M, wi, lane);
 }
 
 // fragments as they come from memory (converted where they are used, so that a fetch ahead does not wait for its data)
@@ -457,13 +663,8 @@ __device__ __forceinline__ void lds_barrier() {
   __builtin_amdgcn_s_barrier();
   asm volatile("" ::: "memory");
 }
-// sum over the four lane groups l>>4 (every lane gets it)
-__device__ __forceinline__ float group_sum(float v) {
-  v += __shfl_xor(v, 16, 64);
-  return v + __shfl_xor(v, 32, 64);
-}
-
-template <typename A, bool DELTA, int DTMAX, int CT>
+// CHAN (delta rule, A = float): q, k and kᵀ come from the workspace with their channel decays in them (channel_block_kernel).
+template <typename A, bool DELTA, int DTMAX, int CT, bool CHAN>
 __global__ __launch_bounds__(NT) void scan_walk_kernel(const A* __restrict__ q, int64_t q_stride, const A* __restrict__ k, int64_t k_stride,
                                                        const A* __restrict__ v, int64_t v_stride, float* __restrict__ state,
                                                        const int* __restrict__ positions, const int* __restrict__ qsl,
@@ -484,7 +685,7 @@ __global__ __launch_bounds__(NT) void scan_walk_kernel(const A* __restrict__ q, 
   float* St = sh;                                         // [16·CT columns][DS]: the state at the block's start
   float* Rt = St + 16 * CT * DS;                          // [columns][BS]: right-hand sides of the delta rule
   float* Ut = Rt + (DELTA ? 16 * CT * BS : 0);            // [columns][BS]: u
-  float* Us = Ut + 16 * CT * BS;                          // [columns][BS]: exp(P_end - P) u
+  float* Us = CHAN ? Ut : Ut + 16 * CT * BS;              // [columns][BS]: exp(P_end - P) u
   const int e0 = blockIdx.y * 16 * CT;
   const bool norm = !DELTA && nq != nullptr && blockIdx.y == 0;
   float* head = state + ((int64_t)slot * H + h) * D * (Dv + (nq != nullptr ? 1 : 0));
@@ -495,9 +696,22 @@ __global__ __launch_bounds__(NT) void scan_walk_kernel(const A* __restrict__ q, 
   R4 qf[DTMAX], kf[DELTA ? DTMAX : 1], kt[DW][4];
   A vf[CT][4];
   f32x4 ia[DELTA ? 4 : 1], aa[4], ep, er, wt;
+  f32x4 pe4[CHAN ? DW : 1];                               // decay of this wave's state rows over the block
   float pend = 0.f, wl = 0.f, el = 0.f, epc = 0.f;
-  auto base_of = [&](int b) { return ws + ((int64_t)(((s0 + BT * b) >> 6) + seq) * H + h) * block_floats<DELTA>(); };
+  const int DP = DT * 16;
+  const int64_t bf = CHAN ? channel_block_floats(DP) : block_floats<DELTA>();
+  auto base_of = [&](int b) { return ws + ((int64_t)(((s0 + BT * b) >> 6) + seq) * H + h) * bf; };
   auto fetch_rows = [&](int b) {                          // q (and k) rows 16·wave + c; rows past the chunk repeat its last token
+    if constexpr (CHAN) {
+      const float* wq = base_of(b) + 2 * BT * BT + BT + DP + (int64_t)(16 * wave + c) * DP + 4 * g4;
+#pragma unroll
+      for (int i = 0; i < DTMAX; ++i)
+        if (i < DT) {
+          qf[i] = ld4<float>(wq + 16 * i);
+          kf[i] = ld4<float>(wq + (int64_t)BT * DP + 16 * i);
+        }
+      return;
+    }
     const int64_t tr = s0 + min(BT * b + 16 * wave + c, n - 1);
     const A* qr = q + tr * q_stride + g * D;
     const A* kr = k + tr * k_stride + g * D;
@@ -518,6 +732,14 @@ __global__ __launch_bounds__(NT) void scan_walk_kernel(const A* __restrict__ q, 
     }
   };
   auto fetch_vectors = [&](int b) {
+    if constexpr (CHAN) {
+      const float* wv = base_of(b) + 2 * BT * BT;
+      wt = ld4<float>(wv + 16 * wave + 4 * g4);
+#pragma unroll
+      for (int i = 0; i < DW; ++i)
+        if (wave + 4 * i < DT) pe4[i] = ld4<float>(wv + BT + 16 * (wave + 4 * i) + 4 * g4);
+      return;
+    }
     const float* wv = base_of(b) + (DELTA ? 2 : 1) * BT * BT;
     ep = ld4<float>(wv + 16 * wave + 4 * g4);
     er = ld4<float>(wv + BT + 16 * wave + 4 * g4);
@@ -542,6 +764,16 @@ __global__ __launch_bounds__(NT) void scan_walk_kernel(const A* __restrict__ q, 
       if (s <= wave) aa[s] = ld4<float>(wa + (16 * wave + c) * BT + 16 * s + 4 * g4);
   };
   auto fetch_columns = [&](int b) {                       // kᵀ of this wave's state row tiles
+    if constexpr (CHAN) {
+      const float* wkt = base_of(b) + 2 * BT * BT + BT + DP + 2 * (int64_t)BT * DP + (int64_t)c * BT + 4 * g4;
+#pragma unroll
+      for (int i = 0; i < DW; ++i)
+        if (wave + 4 * i < DT) {
+#pragma unroll
+          for (int s = 0; s < 4; ++s) kt[i][s] = ld4<float>(wkt + (int64_t)16 * (wave + 4 * i) * BT + 16 * s);
+        }
+      return;
+    }
 #pragma unroll
     for (int i = 0; i < DW; ++i)
       if (wave + 4 * i < DT) {
@@ -612,9 +844,10 @@ __global__ __launch_bounds__(NT) void scan_walk_kernel(const A* __restrict__ q, 
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         float x = ldf<A>(&vf[ct][r]);
-        if (DELTA) x -= ep[r] * ks[ct][r];
+        if (CHAN) x -= ks[ct][r];
+        else if (DELTA) x -= ep[r] * ks[ct][r];
         u[ct][r] = 16 * wave + 4 * g4 + r < nn ? wt[r] * x : 0.f;
-        o[ct][r] *= ep[r] * q_scale;
+        if (!CHAN) o[ct][r] *= ep[r] * q_scale;
       }
     }
     if (more) fetch_values(b + 1);
@@ -638,7 +871,7 @@ __global__ __launch_bounds__(NT) void scan_walk_kernel(const A* __restrict__ q, 
     for (int ct = 0; ct < CT; ++ct) {
       float* p = Ut + (16 * ct + c) * BS + 16 * wave + 4 * g4;
       *reinterpret_cast<f32x4*>(p) = u[ct];
-      *reinterpret_cast<f32x4*>(p + (Us - Ut)) = f32x4{u[ct][0] * er[0], u[ct][1] * er[1], u[ct][2] * er[2], u[ct][3] * er[3]};
+      if (!CHAN) *reinterpret_cast<f32x4*>(p + (Us - Ut)) = f32x4{u[ct][0] * er[0], u[ct][1] * er[1], u[ct][2] * er[2], u[ct][3] * er[3]};
     }
     lds_barrier();
     float rs = 0.f;
@@ -658,6 +891,14 @@ __global__ __launch_bounds__(NT) void scan_walk_kernel(const A* __restrict__ q, 
       if (g4 == 0 && 16 * wave + c < nn) nq[(int64_t)(t0 + 16 * wave + c) * H + h] = x;
     }
     const float pe = pend;
+    if (CHAN)                                             // (before the next block's decays arrive)
+#pragma unroll
+      for (int i = 0; i < DW; ++i)
+        if (wave + 4 * i < DT)
+#pragma unroll
+          for (int ct = 0; ct < CT; ++ct)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) S[i][ct][r] *= pe4[CHAN ? i : 0][r];
     if (more) {
       fetch_scores(b + 1);
       fetch_vectors(b + 1);
@@ -680,7 +921,8 @@ __global__ __launch_bounds__(NT) void scan_walk_kernel(const A* __restrict__ q, 
 #pragma unroll
         for (int ct = 0; ct < CT; ++ct)
 #pragma unroll
-          for (int r = 0; r < 4; ++r) S[i][ct][r] *= pe;
+          for (int r = 0; r < 4; ++r)
+            if (!CHAN) S[i][ct][r] *= pe;
 #pragma unroll
         for (int s = 0; s < 4; ++s) {
           f32x4 ka = Raw<A>::cvt(kt[i][s]);
@@ -785,9 +1027,9 @@ static void gated_scan(const A* q, int64_t q_stride, const A* k, int64_t k_strid
                        const int* tile_seq, const int* tile_q0, int num_tiles, float* ws, hipStream_t stream) {
   const bool blocks = num_tiles > 0 && ws != nullptr && D <= GM_BLOCK_MAX_D;
 #define GM_STEP(DR)                                                                                                                   \
-  hipLaunchKernelGGL((scan_step_kernel<A, DR, DELTA>), dim3(H, (Dv + 63) / 64, seqs), dim3(NT), 0, stream, q, q_stride, k, k_stride, \
+  hipLaunchKernelGGL((scan_step_kernel<A, DR, DELTA, void>), dim3(H, (Dv + 63) / 64, seqs), dim3(NT), 0, stream, q, q_stride, k, k_stride, \
                      v, v_stride, decay, weight, state, positions, qsl, state_slots, counts, H, G, D, Dv, q_scale, out, nq,           \
-                     blocks ? 1 : 0)
+                     blocks ? 1 : 0, ChannelArgs<void>{})
   const int dr = (D + 3) / 4;
   if (dr <= 8) GM_STEP(8);
   else if (dr <= 16) GM_STEP(16);
@@ -804,7 +1046,7 @@ static void gated_scan(const A* q, int64_t q_stride, const A* k, int64_t k_strid
   const size_t lds = (size_t)16 * ct * (DS + (DELTA ? 3 : 2) * BS) * sizeof(float);
   const dim3 grid(H, (Dv + 16 * ct - 1) / (16 * ct), seqs);
 #define GM_WALK(DT, CTV)                                                                                                               \
-  hipLaunchKernelGGL((scan_walk_kernel<A, DELTA, DT, CTV>), grid, dim3(NT), lds, stream, q, q_stride, k, k_stride, v, v_stride, state,  \
+  hipLaunchKernelGGL((scan_walk_kernel<A, DELTA, DT, CTV, false>), grid, dim3(NT), lds, stream, q, q_stride, k, k_stride, v, v_stride, state,  \
                      positions, qsl, state_slots, counts, H, G, D, Dv, wide, q_scale, ws, out, nq)
 #define GM_WALK_D(DT)          \
   do {                         \
@@ -832,6 +1074,53 @@ void launch_gm_gated_scan(const void* q, int64_t q_stride, const void* k, int64_
   if (delta) GM_SCAN(true);
   else GM_SCAN(false);
 #undef GM_SCAN
+}
+
+int64_t gm_channel_ws_floats(int rows, int seqs, int H, int D) {
+  return (int64_t)((rows >> 6) + seqs + 1) * H * channel_block_floats((D + 15) & ~15);
+}
+
+void launch_gm_channel_scan(const float* q, int64_t q_stride, const float* k, int64_t k_stride, const float* v, int64_t v_stride,
+                            const void* z, bool z_bf16, int64_t z_stride, const float* rate, const float* bias, const float* weight,
+                            float* state, const int* positions, const int* qsl, const int* state_slots, const int* counts, int seqs,
+                            int H, int G, int D, int Dv, float* out, const int* tile_seq, const int* tile_q0, int num_tiles, float* ws,
+                            hipStream_t stream) {
+  if (seqs == 0) return;
+  const bool blocks = num_tiles > 0 && ws != nullptr && D <= GM_BLOCK_MAX_D;
+#define GM_STEP(DR)                                                                                                                    \
+  GM_BF16(z_bf16, Z, hipLaunchKernelGGL((scan_step_kernel<float, DR, true, Z>), dim3(H, (Dv + 63) / 64, seqs), dim3(NT), 0, stream, q, q_stride, \
+                                        k, k_stride, v, v_stride, (const float*)nullptr, weight, state, positions, qsl, state_slots,   \
+                                        counts, H, G, D, Dv, 1.f, out, (float*)nullptr, blocks ? 1 : 0,                                \
+                                        (ChannelArgs<Z>{(const Z*)z, z_stride, rate, bias})))
+  const int dr = (D + 3) / 4;
+  if (dr <= 8) GM_STEP(8);
+  else if (dr <= 16) GM_STEP(16);
+  else if (dr <= 32) GM_STEP(32);
+  else if (dr <= 64) GM_STEP(64);
+  else GM_STEP(128);
+#undef GM_STEP
+  if (!blocks) return;
+  const int wide = D % 4 == 0 && q_stride % 4 == 0 && k_stride % 4 == 0 && z_stride % 4 == 0 && al16(q) && al16(k) && al16(z) && al16(bias);
+  GM_BF16(z_bf16, Z, hipLaunchKernelGGL(channel_block_kernel<Z>, dim3(num_tiles, H), dim3(NT), 0, stream, q, q_stride, k, k_stride,
+                                        (ChannelArgs<Z>{(const Z*)z, z_stride, rate, bias}), weight, qsl, state_slots, counts, tile_seq,
+                                        tile_q0, num_tiles, H, G, D, wide, ws));
+  const int ct = H * ((Dv + 31) / 32) >= 128 ? 2 : 1;   // 32 state columns per workgroup where that still leaves enough of them
+  const int DS = ((D + 15) / 16) * 16 + 4;
+  const size_t lds = (size_t)16 * ct * (DS + 2 * BS) * sizeof(float);
+  const dim3 grid(H, (Dv + 16 * ct - 1) / (16 * ct), seqs);
+#define GM_WALK(DT, CTV)                                                                                                                \
+  hipLaunchKernelGGL((scan_walk_kernel<float, true, DT, CTV, true>), grid, dim3(NT), lds, stream, q, q_stride, k, k_stride, v, v_stride, state, \
+                     positions, qsl, state_slots, counts, H, G, D, Dv, wide, 1.f, ws, out, (float*)nullptr)
+#define GM_WALK_D(DT)          \
+  do {                         \
+    if (ct == 2) GM_WALK(DT, 2); \
+    else GM_WALK(DT, 1);       \
+  } while (0)
+  if (D <= 64) GM_WALK_D(4);
+  else if (D <= 128) GM_WALK_D(8);
+  else GM_WALK_D(16);
+#undef GM_WALK_D
+#undef GM_WALK
 }
 
 }  // namespace dli

@@ -274,7 +274,7 @@ __global__ __launch_bounds__(NT) void retention_prep_kernel(const A* __restrict_
 // out[r, f] = act(x[r, f]) · x[r, F + f]; act: tanh-form GELU, or silu.  V entries per thread and trip.
 template <typename A, int V>
 __global__ __launch_bounds__(NT) void act_mul_kernel(const A* __restrict__ x, int64_t x_stride, int F, int64_t n, int silu,
-                                                     A* __restrict__ out) {
+                                                     float limit, A* __restrict__ out) {
   for (int64_t i = ((int64_t)blockIdx.x * NT + threadIdx.x) * V; i < n; i += (int64_t)gridDim.x * NT * V) {
     const int64_t r = i / F;
     const int f = (int)(i - r * F);
@@ -284,6 +284,10 @@ __global__ __launch_bounds__(NT) void act_mul_kernel(const A* __restrict__ x, in
 #pragma unroll
     for (int j = 0; j < V; ++j) {
       const float zz = z.v[j];
+      if (limit > 0.f) {                                  // clamped form
+        o.v[j] = gated_act(zz, u.v[j], limit);
+        continue;
+      }
       const float a = silu ? zz / (1.f + expf(-zz)) : 0.5f * zz * (1.f + tanhf(0.7978845608028654f * (zz + 0.044715f * zz * zz * zz)));
       o.v[j] = a * u.v[j];
     }
@@ -454,7 +458,7 @@ void launch_hm_retention_prep(const void* qkvg, bool bf16, int64_t row_stride, c
                                         positions, freq, rot_dims, H, D, Dv, k_scale, out));
 }
 
-void launch_hm_act_mul(const void* x, bool bf16, int64_t x_stride, int rows, int F, bool silu, void* out, hipStream_t stream) {
+void launch_hm_act_mul(const void* x, bool bf16, int64_t x_stride, int rows, int F, bool silu, float limit, void* out, hipStream_t stream) {
   const int64_t n = (int64_t)rows * F;
   if (n == 0) return;
   const bool wide = F % 4 == 0 && x_stride % 4 == 0 && al16(x) && al16(out);
@@ -462,10 +466,10 @@ void launch_hm_act_mul(const void* x, bool bf16, int64_t x_stride, int rows, int
   const int blocks = (int)std::min<int64_t>((items + NT - 1) / NT, 16384);
   if (wide)
     HM_BF16(bf16, A, hipLaunchKernelGGL((act_mul_kernel<A, 4>), dim3(blocks), dim3(NT), 0, stream, (const A*)x, x_stride, F, n,
-                                        silu ? 1 : 0, (A*)out));
+                                        silu ? 1 : 0, limit, (A*)out));
   else
     HM_BF16(bf16, A, hipLaunchKernelGGL((act_mul_kernel<A, 1>), dim3(blocks), dim3(NT), 0, stream, (const A*)x, x_stride, F, n,
-                                        silu ? 1 : 0, (A*)out));
+                                        silu ? 1 : 0, limit, (A*)out));
 }
 
 void launch_hm_softmax_route(const void* h, bool bf16, int64_t h_stride, const float* router, const float* bias, int E, int K, int rows,

@@ -87,26 +87,37 @@ void launch_sm_qk_norm_cache(void* qkv, bool bf16, int64_t row_stride, const flo
 void launch_sm_latent_prep(void* q, bool bf16, int64_t q_stride, const void* dkv, int64_t dkv_stride, const float* cw, float eps,
                            const int* positions, const double* inv_freq, int rot_dims, const int* slot_mapping, void* cache,
                            int rows, int H, int D, int R, int C, hipStream_t stream);
+// options of the token-major attention kernels
+struct AttnOpts {
+  int chunk = 0;                  // keys from the query's own stretch of `chunk` positions only (0: off)
+  int keep = 0;                   // first tokens visible behind the window
+  float cap = 0.f;                // score ← cap · tanh(score / cap) (0: off)
+  int vshare = 1;                 // consecutive key heads per value head
+  float out_scale = 1.f;
+  float* out_f32 = nullptr;       // results here in fp32 (the strides of `out`)
+  const float* lam = nullptr;     // tile kernel: differential maps (out = out_scale · d / rms(d), d = map 1 - lam · map 2)
+  float eps = 0.f;
+};
 void launch_sm_token_attention(void* out, int64_t o_ts, int64_t o_hs, const void* q1, int64_t q1_ts, int64_t q1_hs, int D1,
                                const void* q2, int64_t q2_ts, int64_t q2_hs, int D2, const void* kc, int rowk, const void* vc,
                                int rowv, int vhead, int Dv, const int* block_tables, int max_blocks, const int* positions,
                                const int* token_seq, int rows, int H, int G, float scale, int window, const float* temp,
                                const float* r1, const float* r2, bool bf16, int nsplit, float* part, const void* gate, int64_t g_ts, const float* sink,
-                               hipStream_t stream);
+                               AttnOpts opt, hipStream_t stream);
 int sm_token_attention_splits(int rows, int H, int G);
 bool launch_sm_head_decode_attention(void* out, int64_t o_ts, int64_t o_hs, const void* q1, int64_t q1_ts, int64_t q1_hs, int D1,
                                      const void* q2, int64_t q2_ts, int64_t q2_hs, int D2, const void* kc, int rowk, const void* vc,
                                      int rowv, int vhead, int Dv, const int* block_tables, int max_blocks, const int* positions,
                                      const int* token_seq, int rows, int H, int G, float scale, int window, const float* temp,
                                      const float* r1, const float* r2, int nsplit, float* part, const void* gate, int64_t g_ts, const float* sink,
-                                     hipStream_t stream);
+                                     AttnOpts opt, hipStream_t stream);
 int sm_head_decode_splits(int rows, int H, int G);
 bool launch_sm_tile_attention(void* out, int64_t o_ts, int64_t o_hs, const void* q1, int64_t q1_ts, int64_t q1_hs, int D1,
                               const void* q2, int64_t q2_ts, int64_t q2_hs, int D2, const void* kc, int rowk, const void* vc,
                               int rowv, int vhead, int Dv, const int* block_tables, int max_blocks, const int* seq_lens,
                               const int* qsl, const int* tile_seq, const int* tile_q0, int num_tiles, const int* counts, int H,
                               int G, float scale, int window, const float* temp, const float* r1, const float* r2,
-                              const void* gate, int64_t g_ts, const float* sink, hipStream_t stream);
+                              const void* gate, int64_t g_ts, const float* sink, AttnOpts opt, hipStream_t stream);
 void launch_sm_lightning_scan(const void* qkvg, bool bf16, int64_t row_stride, float* state, const int* positions, const int* qsl,
                               const int* state_slots, const int* counts, int seqs, int H, int D, int Dv, const float* decay,
                               float* out, int64_t out_part, const int* tile_seq, const int* tile_q0, int num_tiles, float* ws,
@@ -188,7 +199,7 @@ void launch_hm_causal_conv_add(const float* h, const float* w, int taps, float* 
                                bool out_bf16, hipStream_t stream);
 void launch_hm_retention_prep(const void* qkvg, bool bf16, int64_t row_stride, const int* positions, const double* freq, int rot_dims,
                               int rows, int H, int D, int Dv, float k_scale, float* out, hipStream_t stream);
-void launch_hm_act_mul(const void* x, bool bf16, int64_t x_stride, int rows, int F, bool silu, void* out, hipStream_t stream);
+void launch_hm_act_mul(const void* x, bool bf16, int64_t x_stride, int rows, int F, bool silu, float limit, void* out, hipStream_t stream);
 void launch_hm_softmax_route(const void* h, bool bf16, int64_t h_stride, const float* router, const float* bias, int E, int K, int rows,
                              int W, int* ids, float* wts, bool all, hipStream_t stream);
 // gated linear recurrences and gated latent attention (recurmix.hip)
@@ -237,5 +248,23 @@ void launch_gm_gated_scan(const void* q, int64_t q_stride, const void* k, int64_
                           const int* state_slots, const int* counts, int seqs, int H, int G, int D, int Dv, bool delta, float q_scale,
                           bool normaliser, float* out, float* nq, const int* tile_seq, const int* tile_q0, int num_tiles, float* ws,
                           hipStream_t stream);
+
+int64_t gm_channel_ws_floats(int rows, int seqs, int H, int D);
+void launch_gm_channel_scan(const float* q, int64_t q_stride, const float* k, int64_t k_stride, const float* v, int64_t v_stride,
+                            const void* z, bool z_bf16, int64_t z_stride, const float* rate, const float* bias, const float* weight,
+                            float* state, const int* positions, const int* qsl, const int* state_slots, const int* counts, int seqs,
+                            int H, int G, int D, int Dv, float* out, const int* tile_seq, const int* tile_q0, int num_tiles, float* ws,
+                            hipStream_t stream);
+
+// post-norm layers, per-head norms, differential maps (postmix.hip)
+void launch_pm_embed_rows(const int* ids, const void* table, bool bf16, int vocab, float scale, int rows, int W, float* x, void* h,
+                          hipStream_t stream);
+void launch_pm_post_norm_add(float* x, const void* y, bool bf16, const float* w, float eps, const float* w2, int rows, int W, void* out,
+                             bool out_bf16, hipStream_t stream);
+void launch_pm_head_norm_rope_cache(const void* proj, bool bf16, int64_t p_stride, const float* qw, const float* kw, float eps,
+                                    const int* positions, const double* freq, int rot_dims, const int* slot_mapping, void* k_cache,
+                                    void* v_cache, int rows, int H, int G, int D, int Dv, int maps, void* q, hipStream_t stream);
+void launch_pm_map_combine(const float* o, const float* lam, float eps, float scale, int rows, int H, int G, int Dv, const int* token_seq,
+                           void* out, bool out_bf16, int64_t out_stride, hipStream_t stream);
 
 }  // namespace dli

@@ -181,6 +181,11 @@ __global__ __launch_bounds__(NT) void causal_conv_kernel(const A* __restrict__ x
   if (gate.kind != 0 && blockIdx.y == gridDim.y - 1) {
     const A* gr = gate.g + t * x_stride;
     for (int h = threadIdx.x; h < gate.H; h += NT) {
+      if (gate.kind == 3) {                                       // write strengths only
+        gate.decay[t * gate.H + h] = 0.f;
+        gate.weight[t * gate.H + h] = 1.f / (1.f + expf(-ldf<A>(gr + h)));
+        continue;
+      }
       const float z = ldf<A>(gr + (gate.kind == 1 ? gate.H + h : h)) + gate.bias[h];
       const float sp = fmaxf(z, 0.f) + log1pf(expf(-fabsf(z)));  // softplus
       gate.decay[t * gate.H + h] = -gate.rate[h] * sp;

@@ -569,6 +569,15 @@ template <> __device__ __forceinline__ void load_vals<uint16_t, 2>(const uint16_
 template <> __device__ __forceinline__ void load_vals<uint16_t, 4>(const uint16_t* p, bool w, float* d) { load_vals_bf16<4>(p, w, d); }
 template <> __device__ __forceinline__ void load_vals<uint16_t, 8>(const uint16_t* p, bool w, float* d) { load_vals_bf16<8>(p, w, d); }
 
+// first position a query at position p sees (besides kept first tokens)
+__device__ __forceinline__ int first_visible(int p, int window, int chunk) {
+  return window > 0 ? max(p - window + 1, 0) : (chunk > 0 ? p - p % chunk : 0);
+}
+template <typename A> __device__ __forceinline__ void store_out(A* out, const AttnOpts& opt, int64_t i, float v) {
+  if (opt.out_f32 != nullptr) opt.out_f32[i] = v;
+  else stf<A>(out + i, v);
+}
+
 // One workgroup per (token, group of HG query heads that read the same key / value head): a key row and a value row are
 // loaded once for the HG heads.  Every wave takes chunks of 64 consecutive keys: a lane per key for the scores (the HG
 // queries broadcast from LDS, the key row in 16-byte pieces), then lanes over the value columns for P·V — lane owns the
@@ -583,7 +592,7 @@ __global__ __launch_bounds__(NT) void token_attention_kernel(
     const A* __restrict__ vc, int rowv, int vhead, int Dv, const int* __restrict__ block_tables, int max_blocks,
     const int* __restrict__ positions, const int* __restrict__ token_seq, int H, int G, float scale, int window,
     const float* __restrict__ temp, const float* __restrict__ r1, const float* __restrict__ r2, int nsplit,
-    float* __restrict__ part, const A* __restrict__ gate, int64_t g_ts, const float* __restrict__ sink) {
+    float* __restrict__ part, const A* __restrict__ gate, int64_t g_ts, const float* __restrict__ sink, AttnOpts opt) {
   extern __shared__ float sh[];          // q [HG][Dk] | acc [4 waves][HG][Dv] | m [4][HG] | l [4][HG]
   constexpr int NW = NT / 64;
   const int64_t t = blockIdx.x;
@@ -593,8 +602,10 @@ __global__ __launch_bounds__(NT) void token_attention_kernel(
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int Dk = D1 + D2;
   const int p = positions[t];
-  const int lo = window > 0 ? max(p - window + 1, 0) : 0;
-  const int g = h0 / (H / G);
+  const int lo = first_visible(p, window, opt.chunk);
+  const int kept = min(opt.keep, lo);    // first tokens in front of the window: visible positions are 0 … kept-1, lo … p
+  const int visible = kept + p - lo + 1;
+  const int g = h0 / (H / G), gv = g / opt.vshare;
   float* qs = sh;
   float* accs = sh + HG * Dk;
   float* ms = accs + NW * HG * Dv;
@@ -630,13 +641,13 @@ __global__ __launch_bounds__(NT) void token_attention_kernel(
 
   // gridDim.z = nsplit workgroups share a long key range: each takes a contiguous run of 64-key chunks and leaves
   // (max, sum, unnormalised output) in `part`; token_attention_merge_kernel combines them
-  const int nchunks = (p - lo + 64) >> 6;
+  const int nchunks = (visible + 63) >> 6;
   const int per_split = (nchunks + nsplit - 1) / nsplit;
   const int c_begin = blockIdx.z * per_split, c_end = min(c_begin + per_split, nchunks);
   for (int ci = c_begin + wave; ci < c_end; ci += NW) {
-    const int base = lo + ci * 64;
-    const int j = base + lane;
-    const bool valid = j <= p;
+    const int idx = ci * 64 + lane;
+    const bool valid = idx < visible;
+    const int j = idx < kept ? idx : lo + idx - kept;
     int slot = 0;
     float s[HG];
 #pragma unroll
@@ -684,6 +695,7 @@ __global__ __launch_bounds__(NT) void token_attention_kernel(
     for (int hh = 0; hh < HG; ++hh) {
       float sv = -INFINITY;
       if (valid) sv = pen ? s[hh] - r1h[hh] * log1pf(r2h[hh] * (float)(p - j)) : s[hh];
+      if (opt.cap > 0.f && valid) sv = opt.cap * tanhf(sv / opt.cap);
       const float mn = fmaxf(m[hh], wave_max(sv));
       const float corr = expf(m[hh] - mn);             // first chunk: exp(-inf) = 0
       pl[hh] = valid ? expf(sv - mn) : 0.f;
@@ -692,7 +704,7 @@ __global__ __launch_bounds__(NT) void token_attention_kernel(
 #pragma unroll
       for (int v = 0; v < VPL; ++v) acc[hh][v] *= corr;
     }
-    const int nvalid = min(p - base + 1, 64);
+    const int nvalid = min(visible - ci * 64, 64);
     if (e0 < Dv) {
       int jj = 0;
       if (vwide) {
@@ -702,7 +714,7 @@ __global__ __launch_bounds__(NT) void token_attention_kernel(
 #pragma unroll
           for (int u = 0; u < UB; ++u) {
             const int sj = __builtin_amdgcn_readlane(slot, jj + u);
-            load_vals<A, VPL>(vc + (int64_t)sj * rowv + g * vhead + e0, true, vv[u]);
+            load_vals<A, VPL>(vc + (int64_t)sj * rowv + gv * vhead + e0, true, vv[u]);
           }
 #pragma unroll
           for (int u = 0; u < UB; ++u)
@@ -717,7 +729,7 @@ __global__ __launch_bounds__(NT) void token_attention_kernel(
       for (; jj < nvalid; ++jj) {
         const int sj = __builtin_amdgcn_readlane(slot, jj);
         float vv[VPL];
-        const A* vr = vc + (int64_t)sj * rowv + g * vhead + e0;
+        const A* vr = vc + (int64_t)sj * rowv + gv * vhead + e0;
         if (vwide) {
           load_vals<A, VPL>(vr, true, vv);
         } else {
@@ -759,7 +771,7 @@ __global__ __launch_bounds__(NT) void token_attention_kernel(
     if (nsplit == 1) {
       const float gm = gate != nullptr ? 1.f / (1.f + expf(-ldf<A>(gate + t * g_ts + h0 + hh))) : 1.f;
       if (sink != nullptr) L += expf(sink[h0 + hh] - M);            // a logit without key or value in the denominator
-      stf<A>(out + t * o_ts + (h0 + hh) * o_hs + e, o / L * gm);
+      store_out(out, opt, t * o_ts + (h0 + hh) * o_hs + e, o / L * gm * opt.out_scale);
     } else {
       float* pr = part + ((t * H + (h0 + hh)) * nsplit + blockIdx.z) * (int64_t)(Dv + 2);
       pr[2 + e] = o;
@@ -776,7 +788,8 @@ template <typename A>
 __global__ __launch_bounds__(128) void token_attention_merge_kernel(A* __restrict__ out, int64_t o_ts, int64_t o_hs,
                                                                     const float* __restrict__ part,
                                                                     const int* __restrict__ token_seq, int H, int Dv,
-                                                                    int nsplit, const A* __restrict__ gate, int64_t g_ts, const float* __restrict__ sink) {
+                                                                    int nsplit, const A* __restrict__ gate, int64_t g_ts, const float* __restrict__ sink,
+                                                                    AttnOpts opt) {
   const int64_t t = blockIdx.x;
   const int h = blockIdx.y;
   if (token_seq[t] < 0) return;
@@ -792,13 +805,13 @@ __global__ __launch_bounds__(128) void token_attention_merge_kernel(A* __restric
     if (z < nsplit) L += f[z] * pr[z * (Dv + 2) + 1];
   }
   if (sink != nullptr) L += expf(sink[h] - M);
-  const float rl = (gate != nullptr ? 1.f / (1.f + expf(-ldf<A>(gate + t * g_ts + h))) : 1.f) / L;
+  const float rl = (gate != nullptr ? 1.f / (1.f + expf(-ldf<A>(gate + t * g_ts + h))) : 1.f) / L * opt.out_scale;
   for (int e = threadIdx.x; e < Dv; e += 128) {
     float o = 0.f;
 #pragma unroll
     for (int z = 0; z < 16; ++z)
       if (z < nsplit) o += f[z] * pr[z * (Dv + 2) + 2 + e];
-    stf<A>(out + t * o_ts + h * o_hs + e, o * rl);
+    store_out(out, opt, t * o_ts + h * o_hs + e, o * rl);
   }
 }
 
@@ -811,7 +824,9 @@ __global__ __launch_bounds__(128) void token_attention_merge_kernel(A* __restric
 // remainder (two MFMAs: P enters the product with 16 mantissa bits, not 8).  The lane's eight Sᵀ values (two 16-key
 // tiles) are, in register order, the B fragment of the P·V k-step when the staged V columns sit in the slot order
 // slot(t) = ((t & 15) >> 2)·8 + (t >> 4)·4 + (t & 3).  KSMAX / MTMAX: compile-time bounds of ceil(Dk / 32) and Dv / 16.
-template <int KSMAX, int MTMAX, int HW>
+// DIFF (HW = 2): the two halves of the workgroup are the two maps of one head — each with a key slice of its own, values shared;
+// map 2's result goes through LDS and map 1's waves write scale · d / rms(d), d = a1 - lam · a2.
+template <int KSMAX, int MTMAX, int HW, bool DIFF>
 __global__ __launch_bounds__(NT * HW) void tile_attention_kernel(
     uint16_t* __restrict__ out, int64_t o_ts, int64_t o_hs, const uint16_t* __restrict__ q1, int64_t q1_ts, int64_t q1_hs, int D1,
     const uint16_t* __restrict__ q2, int64_t q2_ts, int64_t q2_hs, int D2, const uint16_t* __restrict__ kc, int rowk,
@@ -819,7 +834,7 @@ __global__ __launch_bounds__(NT * HW) void tile_attention_kernel(
     const int* __restrict__ seq_lens, const int* __restrict__ qsl, const int* __restrict__ tile_seq,
     const int* __restrict__ tile_q0, int num_tiles, const int* __restrict__ counts, int H, int G, float scale, int window,
     const float* __restrict__ temp, const float* __restrict__ r1, const float* __restrict__ r2,
-    const uint16_t* __restrict__ gate, int64_t g_ts, const float* __restrict__ sink) {
+    const uint16_t* __restrict__ gate, int64_t g_ts, const float* __restrict__ sink, AttnOpts opt) {
   extern __shared__ __align__(16) uint16_t tl[];
   const int ntiles = counts != nullptr ? min(counts[2], num_tiles) : num_tiles;
   // the host walks causal tiles longest-first from the END of the list
@@ -828,7 +843,9 @@ __global__ __launch_bounds__(NT * HW) void tile_attention_kernel(
   // HW heads of one key / value group per workgroup (4 waves each): the staged page serves all of them
   constexpr int TNT = NT * HW;
   const int wave_all = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
-  const int h = blockIdx.y * HW + (wave_all >> 2);
+  const int map = DIFF ? wave_all >> 2 : 0, per = H / G;
+  // DIFF: blockIdx.y counts (value head, head of its group); query heads are ordered (value head, map, head of its group)
+  const int h = DIFF ? ((int)blockIdx.y / per * 2 + map) * per + (int)blockIdx.y % per : (int)blockIdx.y * HW + (wave_all >> 2);
   const int seq = tile_seq[tile], q0 = tile_q0[tile];
   const int t_begin = qsl[seq];
   const int n_chunk = qsl[seq + 1] - t_begin;
@@ -841,12 +858,12 @@ __global__ __launch_bounds__(NT * HW) void tile_attention_kernel(
   const int KS = (Dk + 31) >> 5, MT = Dv >> 4;
   const int KST = KS * 32 + 8;                            // LDS row strides (elements): +16 bytes against bank conflicts
   constexpr int VST = 40;
-  uint16_t* Ks = tl;
-  uint16_t* Vt = tl + 32 * KST;
-  const int g = h / (H / G);
+  uint16_t* Ks = tl;                                      // [DIFF ? 2 maps : 1][32][KST]
+  uint16_t* Vt = tl + (DIFF ? 64 : 32) * KST;
+  const int g = h / per, gv = g / opt.vshare, g0 = g - map;    // g0: key head of the first staged slice
 
   // zero the K padding columns once (Dk not a multiple of 32): they are never staged over
-  for (int i = threadIdx.x; i < 32 * (KS * 32 - Dk); i += TNT) {
+  for (int i = threadIdx.x; i < (DIFF ? 64 : 32) * (KS * 32 - Dk); i += TNT) {
     const int row = i / (KS * 32 - Dk), col = Dk + i % (KS * 32 - Dk);
     Ks[row * KST + col] = 0;
   }
@@ -868,12 +885,17 @@ __global__ __launch_bounds__(NT * HW) void tile_attention_kernel(
   // scores are kept in the log2 domain: s·log2(e) − r1·log2(1 + r2·distance), weights 2^(s − max) — one v_exp_f32 and one
   // v_log_f32 per score (this kernel is bound by the per-score vector arithmetic, not by the matrix cores; its results are
   // rounded to bf16 anyway: the fp32 model never takes this path)
-  const float qmul = scale * (temp != nullptr ? temp[h] : 1.f) * 1.4426950408889634f;
+  // soft cap: cap · tanh(s / cap) = cap · (1 - 2 / (2^(2 log2(e) s / cap) + 1))
+  const bool capped = opt.cap > 0.f;
+  const float capl = opt.cap * 1.4426950408889634f;
+  const float qmul = scale * (temp != nullptr ? temp[h] : 1.f) * 1.4426950408889634f * (capped ? 2.f / opt.cap : 1.f);
   const float r1h = r1 != nullptr ? r1[h] : 0.f, r2h = r1 != nullptr ? r2[h] : 0.f;
   const bool pen = r1h != 0.f;
   const int pq = p0 + q0 + qi;                            // this lane's query position
   const int p_first = p0 + q0, p_last = p0 + q0 + nq - 1;
-  const int kb_lo = (window > 0 ? max(p_first - window + 1, 0) : 0) >> 5, kb_hi = p_last >> 5;
+  const int kb_lo = first_visible(p_first, window, opt.chunk) >> 5, kb_hi = p_last >> 5;
+  const int lo_q = first_visible(pq, window, opt.chunk), lo_last = first_visible(p_last, window, opt.chunk);
+  const int kept_pages = min((opt.keep + 31) >> 5, kb_lo);    // pages of kept first tokens in front of the window's
   const int* bt = block_tables + (int64_t)seq * max_blocks;
 
   float m = -INFINITY, l = 0.f;
@@ -883,19 +905,21 @@ __global__ __launch_bounds__(NT * HW) void tile_attention_kernel(
 
   const int kchunks = Dk >> 3, vchunks = Dv >> 3;
   const bool vfromk = vc == kc && rowv == rowk && vhead == Dk;     // latent attention: one row is key and value
-  for (int kb = kb_lo; kb <= kb_hi; ++kb) {
+  const uint16_t* Km = Ks + map * 32 * KST;
+  for (int it = kb_lo - kept_pages; it <= kb_hi; ++it) {
+    const int kb = it < kb_lo ? it - (kb_lo - kept_pages) : it;
     __syncthreads();                                      // everyone is done with the previous page
     const int64_t page_row = (int64_t)bt[kb] * kBlockTokens;
-    for (int i = threadIdx.x; i < 32 * kchunks; i += TNT) {
-      const int row = i / kchunks, ch = i - row * kchunks;
-      *reinterpret_cast<bf16x8*>(Ks + row * KST + 8 * ch) =
-          *reinterpret_cast<const bf16x8*>(kc + (page_row + row) * rowk + g * Dk + 8 * ch);
+    for (int i = threadIdx.x; i < (DIFF ? 64 : 32) * kchunks; i += TNT) {
+      const int srow = i / kchunks, ch = i - srow * kchunks, row = srow & 31;
+      *reinterpret_cast<bf16x8*>(Ks + srow * KST + 8 * ch) =
+          *reinterpret_cast<const bf16x8*>(kc + (page_row + row) * rowk + (DIFF ? g0 + (srow >> 5) : g) * Dk + 8 * ch);
     }
     if (vfromk) __syncthreads();                          // values = leading columns of the key rows just staged
     for (int i = threadIdx.x; i < 32 * vchunks; i += TNT) {
       const int row = i & 31, ch = i >> 5;
       const bf16x8 v = vfromk ? *reinterpret_cast<const bf16x8*>(Ks + row * KST + 8 * ch)
-                              : *reinterpret_cast<const bf16x8*>(vc + (page_row + row) * rowv + g * vhead + 8 * ch);
+                              : *reinterpret_cast<const bf16x8*>(vc + (page_row + row) * rowv + gv * vhead + 8 * ch);
       const int slot = ((row & 15) >> 2) * 8 + (row >> 4) * 4 + (row & 3);
 #pragma unroll
       for (int j = 0; j < 8; ++j) Vt[(8 * ch + j) * VST + slot] = (uint16_t)v[j];
@@ -906,8 +930,8 @@ __global__ __launch_bounds__(NT * HW) void tile_attention_kernel(
 #pragma unroll
     for (int s = 0; s < KSMAX; ++s) {
       if (s < KS) {
-        const bf16x8 ka = *reinterpret_cast<const bf16x8*>(Ks + c * KST + 32 * s + 8 * g4);
-        const bf16x8 kb2 = *reinterpret_cast<const bf16x8*>(Ks + (16 + c) * KST + 32 * s + 8 * g4);
+        const bf16x8 ka = *reinterpret_cast<const bf16x8*>(Km + c * KST + 32 * s + 8 * g4);
+        const bf16x8 kb2 = *reinterpret_cast<const bf16x8*>(Km + (16 + c) * KST + 32 * s + 8 * g4);
         sa = mfma16(ka, qf[s], sa);
         sb = mfma16(kb2, qf[s], sb);
       }
@@ -915,14 +939,15 @@ __global__ __launch_bounds__(NT * HW) void tile_attention_kernel(
     float sv[8];
     float mx = -INFINITY;
     // a page every query of the tile sees whole (the common case far from the diagonal) needs no per-score masks
-    const bool whole = nq == 64 && 32 * kb + 31 <= p_first && (window <= 0 || 32 * kb > p_last - window);
+    const bool whole = nq == 64 && 32 * kb + 31 <= p_first && (32 * kb >= lo_last || 32 * kb + 31 < opt.keep);
 #pragma unroll
     for (int r = 0; r < 8; ++r) {
       const int j = 32 * kb + (r < 4 ? 4 * g4 + r : 16 + 4 * g4 + (r - 4));
       float v = (r < 4 ? sa[r] : sb[r - 4]) * qmul;
       if (pen) v -= r1h * __builtin_amdgcn_logf(1.f + r2h * (float)max(pq - j, 0));
+      if (capped) v = capl - 2.f * capl * fast_rcp(fast_exp2(v) + 1.f);
       if (!whole) {
-        const bool ok = qvalid && j <= pq && (window <= 0 || j > pq - window);
+        const bool ok = qvalid && j <= pq && (j >= lo_q || j < opt.keep);
         v = ok ? v : -INFINITY;
       }
       sv[r] = v;
@@ -958,17 +983,49 @@ __global__ __launch_bounds__(NT * HW) void tile_attention_kernel(
   }
   l += __shfl_xor(l, 16, 64);
   l += __shfl_xor(l, 32, 64);
+  if constexpr (DIFF) {
+    float* X = reinterpret_cast<float*>(tl) + wave * MT * 256 + lane;      // [wave][value tile · 4 + r][lane]
+    __syncthreads();                                      // the last page's readers are done
+    if (map == 1) {
+      const float rl = opt.lam[0] / l;
+#pragma unroll
+      for (int i = 0; i < MTMAX; ++i)
+        if (i < MT)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) X[(4 * i + r) * 64] = acc[i][r] * rl;
+    }
+    __syncthreads();
+    if (map == 1) return;
+    const float rl = 1.f / l;
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < MTMAX; ++i)
+      if (i < MT)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          acc[i][r] = acc[i][r] * rl - X[(4 * i + r) * 64];
+          ss += acc[i][r] * acc[i][r];
+        }
+    ss += __shfl_xor(ss, 16, 64);
+    ss += __shfl_xor(ss, 32, 64);
+    if (!qvalid) return;
+    const float inv = opt.out_scale / sqrtf(ss / (float)Dv + opt.eps);
+    uint16_t* orow = out + tq * o_ts + (int64_t)blockIdx.y * o_hs;
+#pragma unroll
+    for (int i = 0; i < MTMAX; ++i)
+      if (i < MT) st4<uint16_t>(orow + 16 * i + 4 * g4, f32x4{acc[i][0] * inv, acc[i][1] * inv, acc[i][2] * inv, acc[i][3] * inv});
+    return;
+  }
   if (!qvalid) return;
   if (sink != nullptr) l += fast_exp2(sink[h] * 1.4426950408889634f - m);
-  const float rl = (gate != nullptr ? 1.f / (1.f + expf(-bf2f(gate[tq * g_ts + h]))) : 1.f) / l;
-  uint16_t* orow = out + tq * o_ts + h * o_hs;
+  const float rl = (gate != nullptr ? 1.f / (1.f + expf(-bf2f(gate[tq * g_ts + h]))) : 1.f) / l * opt.out_scale;
+  const int64_t o0 = tq * o_ts + h * o_hs;
 #pragma unroll
   for (int i = 0; i < MTMAX; ++i) {
     if (i < MT) {
-      bf16x4 o;
-#pragma unroll
-      for (int r = 0; r < 4; ++r) o[r] = (short)f2bf(acc[i][r] * rl);
-      *reinterpret_cast<bf16x4*>(orow + 16 * i + 4 * g4) = o;
+      const f32x4 o = {acc[i][0] * rl, acc[i][1] * rl, acc[i][2] * rl, acc[i][3] * rl};
+      if (opt.out_f32 != nullptr) st4<float>(opt.out_f32 + o0 + 16 * i + 4 * g4, o);
+      else st4<uint16_t>(out + o0 + 16 * i + 4 * g4, o);
     }
   }
 }
@@ -987,13 +1044,13 @@ __global__ __launch_bounds__(NT) void head_decode_attention_kernel(
     const uint16_t* __restrict__ vc, int rowv, int vhead, int Dv, const int* __restrict__ block_tables, int max_blocks,
     const int* __restrict__ positions, const int* __restrict__ token_seq, int H, int G, int groups, float scale, int window,
     const float* __restrict__ temp, const float* __restrict__ r1, const float* __restrict__ r2, int nsplit,
-    float* __restrict__ part, const uint16_t* __restrict__ gate, int64_t g_ts, const float* __restrict__ sink) {
+    float* __restrict__ part, const uint16_t* __restrict__ gate, int64_t g_ts, const float* __restrict__ sink, AttnOpts opt) {
   extern __shared__ __align__(16) uint16_t tl[];
   const int64_t t = blockIdx.x;
   const int seq = token_seq[t];
   if (seq < 0) return;
   const int per = H / G;
-  const int g = blockIdx.y / groups, grp = blockIdx.y - g * groups;
+  const int g = blockIdx.y / groups, grp = blockIdx.y - g * groups, gv = g / opt.vshare;
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int lane = threadIdx.x & 63, g4 = lane >> 4, c = lane & 15;
   const bool hvalid = 16 * grp + c < per;
@@ -1019,14 +1076,18 @@ __global__ __launch_bounds__(NT) void head_decode_attention_kernel(
                  : *reinterpret_cast<const bf16x8*>(q2 + t * q2_ts + h * q2_hs + (d - D1));
     qf[s] = v;
   }
-  const float qmul = scale * (temp != nullptr ? temp[h] : 1.f) * 1.4426950408889634f;     // log2 domain, as in the tile kernel
+  // log2 domain and soft cap as in the tile kernel
+  const bool capped = opt.cap > 0.f;
+  const float capl = opt.cap * 1.4426950408889634f;
+  const float qmul = scale * (temp != nullptr ? temp[h] : 1.f) * 1.4426950408889634f * (capped ? 2.f / opt.cap : 1.f);
   const float r1h = r1 != nullptr ? r1[h] : 0.f, r2h = r1 != nullptr ? r2[h] : 0.f;
   const bool pen = r1 != nullptr;
   const int p = positions[t];
-  const int lo = window > 0 ? max(p - window + 1, 0) : 0;
+  const int lo = first_visible(p, window, opt.chunk);
   const int kb_lo = lo >> 5, kb_hi = p >> 5;
-  const int per_split = (kb_hi - kb_lo + nsplit) / nsplit;
-  const int kb_begin = kb_lo + blockIdx.z * per_split, kb_end = min(kb_begin + per_split - 1, kb_hi);
+  const int kept_pages = min((opt.keep + 31) >> 5, kb_lo), it_lo = kb_lo - kept_pages;     // kept first tokens in front of the window
+  const int per_split = (kb_hi - it_lo + nsplit) / nsplit;
+  const int it_begin = it_lo + blockIdx.z * per_split, it_end = min(it_begin + per_split - 1, kb_hi);
   const int* bt = block_tables + (int64_t)seq * max_blocks;
 
   float m = -INFINITY, l = 0.f;
@@ -1035,7 +1096,8 @@ __global__ __launch_bounds__(NT) void head_decode_attention_kernel(
   for (int i = 0; i < MTQ; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
   const int kchunks = Dk >> 3, vchunks = Dv >> 3;
   const bool vfromk = vc == kc && rowv == rowk && vhead == Dk;     // latent attention: one row is key and value
-  for (int kb = kb_begin; kb <= kb_end; ++kb) {
+  for (int it = it_begin; it <= it_end; ++it) {
+    const int kb = it < kb_lo ? it - it_lo : it;
     __syncthreads();
     const int64_t page_row = (int64_t)bt[kb] * kBlockTokens;
     for (int i = threadIdx.x; i < 32 * kchunks; i += NT) {
@@ -1047,7 +1109,7 @@ __global__ __launch_bounds__(NT) void head_decode_attention_kernel(
     for (int i = threadIdx.x; i < 32 * vchunks; i += NT) {
       const int row = i & 31, ch = i >> 5;
       const bf16x8 v = vfromk ? *reinterpret_cast<const bf16x8*>(Ks + row * KST + 8 * ch)
-                              : *reinterpret_cast<const bf16x8*>(vc + (page_row + row) * rowv + g * vhead + 8 * ch);
+                              : *reinterpret_cast<const bf16x8*>(vc + (page_row + row) * rowv + gv * vhead + 8 * ch);
       const int slot = ((row & 15) >> 2) * 8 + (row >> 4) * 4 + (row & 3);
 #pragma unroll
       for (int j = 0; j < 8; ++j) Vt[(8 * ch + j) * VST + slot] = (uint16_t)v[j];
@@ -1070,7 +1132,8 @@ __global__ __launch_bounds__(NT) void head_decode_attention_kernel(
       const int j = 32 * kb + (r < 4 ? 4 * g4 + r : 16 + 4 * g4 + (r - 4));
       float v = (r < 4 ? sa[r] : sb[r - 4]) * qmul;
       if (pen) v -= r1h * __builtin_amdgcn_logf(1.f + r2h * (float)max(p - j, 0));
-      v = (j >= lo && j <= p) ? v : -INFINITY;
+      if (capped) v = capl - 2.f * capl * fast_rcp(fast_exp2(v) + 1.f);
+      v = (j <= p && (j >= lo || j < opt.keep)) ? v : -INFINITY;
       sv[r] = v;
       mx = fmaxf(mx, v);
     }
@@ -1108,16 +1171,15 @@ __global__ __launch_bounds__(NT) void head_decode_attention_kernel(
   if (!hvalid) return;
   if (nsplit == 1) {
     if (sink != nullptr) l += fast_exp2(sink[h] * 1.4426950408889634f - m);
-    const float rl = (gate != nullptr ? 1.f / (1.f + expf(-bf2f(gate[t * g_ts + h]))) : 1.f) / l;
-    uint16_t* orow = out + t * o_ts + h * o_hs;
+    const float rl = (gate != nullptr ? 1.f / (1.f + expf(-bf2f(gate[t * g_ts + h]))) : 1.f) / l * opt.out_scale;
+    const int64_t o0 = t * o_ts + h * o_hs;
 #pragma unroll
     for (int ii = 0; ii < MTQ; ++ii) {
       const int i = wave * MTW + ii;
       if (ii < MTW && i < MT) {
-        bf16x4 o;
-#pragma unroll
-        for (int r = 0; r < 4; ++r) o[r] = (short)f2bf(acc[ii][r] * rl);
-        *reinterpret_cast<bf16x4*>(orow + 16 * i + 4 * g4) = o;
+        const f32x4 o = {acc[ii][0] * rl, acc[ii][1] * rl, acc[ii][2] * rl, acc[ii][3] * rl};
+        if (opt.out_f32 != nullptr) st4<float>(opt.out_f32 + o0 + 16 * i + 4 * g4, o);
+        else st4<uint16_t>(out + o0 + 16 * i + 4 * g4, o);
       }
     }
   } else {
@@ -1385,11 +1447,12 @@ static void token_attention_hg(int hg, dim3 grid, size_t lds, hipStream_t stream
                                int64_t q1_ts, int64_t q1_hs, int D1, const A* q2, int64_t q2_ts, int64_t q2_hs, int D2, const A* kc,
                                int rowk, const A* vc, int rowv, int vhead, int Dv, const int* bt, int max_blocks, const int* pos,
                                const int* tseq, int H, int G, float scale, int window, const float* temp, const float* r1,
-                               const float* r2, int nsplit, float* part, const A* gate, int64_t g_ts, const float* __restrict__ sink) {
+                               const float* r2, int nsplit, float* part, const A* gate, int64_t g_ts, const float* __restrict__ sink,
+                               AttnOpts opt) {
 #define SM_ATT(HGV)                                                                                                              \
   hipLaunchKernelGGL((token_attention_kernel<A, VPL, HGV>), grid, dim3(NT), lds, stream, out, o_ts, o_hs, q1, q1_ts, q1_hs, D1,  \
                      q2, q2_ts, q2_hs, D2, kc, rowk, vc, rowv, vhead, Dv, bt, max_blocks, pos, tseq, H, G, scale, window, temp,  \
-                     r1, r2, nsplit, part, gate, g_ts, sink)
+                     r1, r2, nsplit, part, gate, g_ts, sink, opt)
   if (hg == 1) SM_ATT(1);
   else if (hg == 2) SM_ATT(2);
   else SM_ATT(4);
@@ -1401,15 +1464,18 @@ void launch_sm_token_attention(void* out, int64_t o_ts, int64_t o_hs, const void
                                int rowv, int vhead, int Dv, const int* block_tables, int max_blocks, const int* positions,
                                const int* token_seq, int rows, int H, int G, float scale, int window, const float* temp,
                                const float* r1, const float* r2, bool bf16, int nsplit, float* part, const void* gate, int64_t g_ts, const float* sink,
-                               hipStream_t stream) {
+                               AttnOpts opt, hipStream_t stream) {
   if (rows == 0) return;
   if (Dv > 512) {
     // wider values than a lane's 8 columns × 64 lanes: slabs of 512 columns, each a launch of its own (scores recomputed)
-    for (int e = 0; e < Dv; e += 512)
+    const AttnOpts o0 = opt;
+    for (int e = 0; e < Dv; e += 512) {
+      if (o0.out_f32 != nullptr) opt.out_f32 = o0.out_f32 + e;
       launch_sm_token_attention(bf16 ? (void*)((uint16_t*)out + e) : (void*)((float*)out + e), o_ts, o_hs, q1, q1_ts, q1_hs, D1, q2,
                                 q2_ts, q2_hs, D2, kc, rowk, bf16 ? (const void*)((const uint16_t*)vc + e) : (const void*)((const float*)vc + e),
                                 rowv, vhead, std::min(512, Dv - e), block_tables, max_blocks, positions, token_seq, rows, H, G, scale,
-                                window, temp, r1, r2, bf16, 1, nullptr, gate, g_ts, sink, stream);
+                                window, temp, r1, r2, bf16, 1, nullptr, gate, g_ts, sink, opt, stream);
+    }
     return;
   }
   // heads per workgroup: as many of the heads sharing a key / value head as divide their number and fit the LDS budget
@@ -1424,7 +1490,7 @@ void launch_sm_token_attention(void* out, int64_t o_ts, int64_t o_hs, const void
   SM_DISPATCH_BF16(bf16, A, (token_attention_hg<A, VPLV>(hg, grid, lds, stream, (A*)out, o_ts, o_hs, (const A*)q1, q1_ts, q1_hs, \
                                                          D1, (const A*)q2, q2_ts, q2_hs, D2, (const A*)kc, rowk, (const A*)vc,   \
                                                          rowv, vhead, Dv, block_tables, max_blocks, positions, token_seq, H, G,  \
-                                                         scale, window, temp, r1, r2, nsplit, part, (const A*)gate, g_ts, sink)))
+                                                         scale, window, temp, r1, r2, nsplit, part, (const A*)gate, g_ts, sink, opt)))
   if (nv <= 1) SM_ATT_V(1);
   else if (nv <= 2) SM_ATT_V(2);
   else if (nv <= 4) SM_ATT_V(4);
@@ -1432,7 +1498,7 @@ void launch_sm_token_attention(void* out, int64_t o_ts, int64_t o_hs, const void
 #undef SM_ATT_V
   if (nsplit > 1)
     SM_DISPATCH_BF16(bf16, A, hipLaunchKernelGGL(token_attention_merge_kernel<A>, dim3(rows, H), dim3(128), 0, stream, (A*)out, o_ts,
-                                                 o_hs, (const float*)part, token_seq, H, Dv, nsplit, (const A*)gate, g_ts, sink));
+                                                 o_hs, (const float*)part, token_seq, H, Dv, nsplit, (const A*)gate, g_ts, sink, opt));
 }
 
 // workgroups of a per-token attention launch over `rows` tokens: long key ranges are cut so that about 1024 exist
@@ -1450,36 +1516,43 @@ bool launch_sm_tile_attention(void* out, int64_t o_ts, int64_t o_hs, const void*
                               int rowv, int vhead, int Dv, const int* block_tables, int max_blocks, const int* seq_lens,
                               const int* qsl, const int* tile_seq, const int* tile_q0, int num_tiles, const int* counts, int H,
                               int G, float scale, int window, const float* temp, const float* r1, const float* r2,
-                              const void* gate, int64_t g_ts, const float* sink, hipStream_t stream) {
+                              const void* gate, int64_t g_ts, const float* sink, AttnOpts opt, hipStream_t stream) {
   const int Dk = D1 + D2, KS = (Dk + 31) / 32, MT = Dv / 16;
+  const bool diff = opt.lam != nullptr;                   // H query vectors = two maps of H / 2 heads, G key vectors likewise
   auto al = [](const void* p, int64_t a) { return p == nullptr || reinterpret_cast<uintptr_t>(p) % a == 0; };
   const bool ok = D1 % 8 == 0 && D2 % 8 == 0 && Dv % 16 == 0 && KS <= 18 && MT <= 32 && rowk % 8 == 0 && rowv % 8 == 0 &&
                   vhead % 8 == 0 && q1_ts % 8 == 0 && q1_hs % 8 == 0 && q2_ts % 8 == 0 && q2_hs % 8 == 0 && o_ts % 4 == 0 &&
-                  o_hs % 4 == 0 && al(out, 8) && al(q1, 16) && al(q2, 16) && al(kc, 16) && al(vc, 16);
-  if (!ok) return false;
+                  o_hs % 4 == 0 && al(out, 8) && al(opt.out_f32, 16) && al(q1, 16) && al(q2, 16) && al(kc, 16) && al(vc, 16);
+  if (!ok || (diff && (KS > 8 || MT > 16))) return false;
   if (num_tiles == 0) return true;
-  const size_t lds = (size_t)(32 * (KS * 32 + 8) + Dv * 40) * sizeof(uint16_t);
-  // two heads of a key / value group per workgroup (8 waves) where the group has an even number of heads
-  const int hw = (H / G) % 2 == 0 ? 2 : 1;
+  size_t lds = (size_t)((diff ? 64 : 32) * (KS * 32 + 8) + Dv * 40) * sizeof(uint16_t);
+  if (diff) lds = std::max(lds, (size_t)64 * Dv * sizeof(float));
+  // two heads of a key / value group (or the two maps of a head) per workgroup (8 waves) where the group has an even number of heads
+  const int hw = diff || (H / G) % 2 == 0 ? 2 : 1;
   const dim3 grid(num_tiles, H / hw);
-#define SM_TILE_HW(KSM, MTM, HWV)                                                                                                \
+#define SM_TILE_HW(KSM, MTM, HWV, DIFF)                                                                                                \
   do {                                                                                                                           \
     static bool big = false;                                                                                                     \
     if (lds > 48 * 1024 && !big) {                                                                                               \
-      (void)hipFuncSetAttribute(reinterpret_cast<const void*>(&tile_attention_kernel<KSM, MTM, HWV>),                            \
+      (void)hipFuncSetAttribute(reinterpret_cast<const void*>(&tile_attention_kernel<KSM, MTM, HWV, DIFF>),                      \
                                 hipFuncAttributeMaxDynamicSharedMemorySize, 100 * 1024);                                         \
       big = true;                                                                                                                \
     }                                                                                                                            \
-    hipLaunchKernelGGL((tile_attention_kernel<KSM, MTM, HWV>), grid, dim3(NT * HWV), lds, stream, (uint16_t*)out, o_ts, o_hs,    \
+    hipLaunchKernelGGL((tile_attention_kernel<KSM, MTM, HWV, DIFF>), grid, dim3(NT * HWV), lds, stream, (uint16_t*)out, o_ts, o_hs,    \
                        (const uint16_t*)q1, q1_ts, q1_hs, D1, (const uint16_t*)q2, q2_ts, q2_hs, D2, (const uint16_t*)kc, rowk,  \
                        (const uint16_t*)vc, rowv, vhead, Dv, block_tables, max_blocks, seq_lens, qsl, tile_seq, tile_q0,        \
-                       num_tiles, counts, H, G, scale, window, temp, r1, r2, (const uint16_t*)gate, g_ts, sink);                       \
+                       num_tiles, counts, H, G, scale, window, temp, r1, r2, (const uint16_t*)gate, g_ts, sink, opt);                       \
   } while (0)
 #define SM_TILE(KSM, MTM)              \
   do {                                 \
-    if (hw == 2) SM_TILE_HW(KSM, MTM, 2); \
-    else SM_TILE_HW(KSM, MTM, 1);      \
+    if (hw == 2) SM_TILE_HW(KSM, MTM, 2, false); \
+    else SM_TILE_HW(KSM, MTM, 1, false);      \
   } while (0)
+  if (diff) {
+    if (KS <= 4 && MT <= 8) SM_TILE_HW(4, 8, 2, true);
+    else SM_TILE_HW(8, 16, 2, true);
+    return true;
+  }
   if (KS <= 4 && MT <= 8) SM_TILE(4, 8);
   else if (KS <= 8 && MT <= 16) SM_TILE(8, 16);
   else SM_TILE(18, 32);
@@ -1494,12 +1567,12 @@ bool launch_sm_head_decode_attention(void* out, int64_t o_ts, int64_t o_hs, cons
                                      int rowv, int vhead, int Dv, const int* block_tables, int max_blocks, const int* positions,
                                      const int* token_seq, int rows, int H, int G, float scale, int window, const float* temp,
                                      const float* r1, const float* r2, int nsplit, float* part, const void* gate, int64_t g_ts, const float* sink,
-                                     hipStream_t stream) {
+                                     AttnOpts opt, hipStream_t stream) {
   const int Dk = D1 + D2, KS = (Dk + 31) / 32, MT = Dv / 16, per = H / G;
   auto al = [](const void* p, int64_t a) { return p == nullptr || reinterpret_cast<uintptr_t>(p) % a == 0; };
   const bool ok = per >= 8 && D1 % 8 == 0 && D2 % 8 == 0 && Dv % 16 == 0 && KS <= 18 && MT <= 32 && rowk % 8 == 0 && rowv % 8 == 0 &&
                   vhead % 8 == 0 && q1_ts % 8 == 0 && q1_hs % 8 == 0 && q2_ts % 8 == 0 && q2_hs % 8 == 0 && o_ts % 4 == 0 &&
-                  o_hs % 4 == 0 && al(out, 8) && al(q1, 16) && al(q2, 16) && al(kc, 16) && al(vc, 16);
+                  o_hs % 4 == 0 && al(out, 8) && al(opt.out_f32, 16) && al(q1, 16) && al(q2, 16) && al(kc, 16) && al(vc, 16);
   if (!ok) return false;
   if (rows == 0) return true;
   const size_t lds = (size_t)(32 * (KS * 32 + 8) + Dv * 40) * sizeof(uint16_t);
@@ -1516,7 +1589,7 @@ bool launch_sm_head_decode_attention(void* out, int64_t o_ts, int64_t o_hs, cons
     hipLaunchKernelGGL((head_decode_attention_kernel<KSM, MTQV>), grid, dim3(NT), lds, stream, (uint16_t*)out, o_ts, o_hs,       \
                        (const uint16_t*)q1, q1_ts, q1_hs, D1, (const uint16_t*)q2, q2_ts, q2_hs, D2, (const uint16_t*)kc, rowk,  \
                        (const uint16_t*)vc, rowv, vhead, Dv, block_tables, max_blocks, positions, token_seq, H, G, groups, scale,\
-                       window, temp, r1, r2, nsplit, part, (const uint16_t*)gate, g_ts, sink);                                         \
+                       window, temp, r1, r2, nsplit, part, (const uint16_t*)gate, g_ts, sink, opt);                                         \
   } while (0)
   if (KS <= 4 && MT <= 8) SM_HD(4, 2);
   else if (KS <= 8 && MT <= 16) SM_HD(8, 4);
@@ -1524,7 +1597,7 @@ bool launch_sm_head_decode_attention(void* out, int64_t o_ts, int64_t o_hs, cons
 #undef SM_HD
   if (nsplit > 1)
     hipLaunchKernelGGL(token_attention_merge_kernel<uint16_t>, dim3(rows, H), dim3(128), 0, stream, (uint16_t*)out, o_ts, o_hs,
-                       (const float*)part, token_seq, H, Dv, nsplit, (const uint16_t*)gate, g_ts, sink);
+                       (const float*)part, token_seq, H, Dv, nsplit, (const uint16_t*)gate, g_ts, sink, opt);
   return true;
 }
 

@@ -37,7 +37,7 @@ std::tuple<Tensor, Tensor, Tensor> rm_causal_conv(const Tensor& x, const Tensor&
   const float *rp = nullptr, *gbp = nullptr;
   Tensor decay, weight;
   if (gate_kind != 0) {
-    TORCH_CHECK((gate_kind == 1 || gate_kind == 2) && gate.has_value() && rate.has_value() && gate_bias.has_value(), "gates need columns, rates and biases");
+    TORCH_CHECK(gate_kind >= 1 && gate_kind <= 3 && gate.has_value() && rate.has_value() && gate_bias.has_value(), "gates need columns, rates and biases");
     H = rate->numel();
     check_f32(*rate, "rate", H);
     check_f32(*gate_bias, "gate_bias", H);

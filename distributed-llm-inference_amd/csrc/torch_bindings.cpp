@@ -584,6 +584,7 @@ void ar_all_gather(int64_t st, const Tensor& inp, Tensor out) {
 #include "hypermix_bindings.h"
 #include "recurmix_bindings.h"
 #include "gatemix_bindings.h"
+#include "postmix_bindings.h"
 
 }  // namespace
 
@@ -602,16 +603,17 @@ TORCH_LIBRARY(dli, m) {
   m.def("sm_latent_prep(Tensor(a!) q, Tensor dkv, Tensor cw, float eps, Tensor positions, Tensor inv_freq, int rot_dims, "
         "Tensor slot_mapping, Tensor(b!) cache, int H, int D, int R, int C) -> ()", &sm_latent_prep);
   m.def("sm_token_attention(Tensor(a!) out, Tensor q1, Tensor? q2, Tensor k_cache, Tensor? v_cache, Tensor block_tables, "
-        "Tensor positions, Tensor token_seq, int G, int Dv, float scale, int window, Tensor? temp, Tensor? r1, Tensor? r2, int rows=-1, "
-        "Tensor? gate=None, Tensor? sink=None) -> ()",
+        "Tensor positions, Tensor token_seq, int G, int Dv, float scale, int window, Tensor? temp, Tensor? r1, Tensor? r2, int rows, "
+        "Tensor? gate, Tensor? sink, int chunk, int keep, float cap, int Gv, float out_scale) -> ()",
         &sm_token_attention);
   m.def("sm_head_decode_attention(Tensor(a!) out, Tensor q1, Tensor? q2, Tensor k_cache, Tensor? v_cache, Tensor block_tables, "
         "Tensor positions, Tensor token_seq, int G, int Dv, float scale, int window, Tensor? temp, Tensor? r1, Tensor? r2, int rows, "
-        "Tensor? gate=None, Tensor? sink=None) -> bool",
+        "Tensor? gate, Tensor? sink, int chunk, int keep, float cap, int Gv, float out_scale) -> bool",
         &sm_head_decode_attention);
   m.def("sm_tile_attention(Tensor(a!) out, Tensor q1, Tensor? q2, Tensor k_cache, Tensor? v_cache, Tensor block_tables, Tensor seq_lens, "
         "Tensor qsl, Tensor tile_seq, Tensor tile_q0, int num_tiles, Tensor? counts, int G, int Dv, float scale, int window, "
-        "Tensor? temp, Tensor? r1, Tensor? r2, Tensor? gate=None, Tensor? sink=None) -> bool", &sm_tile_attention);
+        "Tensor? temp, Tensor? r1, Tensor? r2, Tensor? gate, Tensor? sink, int chunk, int keep, float cap, int Gv, float out_scale, "
+        "Tensor? lam=None, float eps=0.0) -> bool", &sm_tile_attention);
   m.def("sm_lightning_scan(Tensor qkvg, Tensor(a!) state, Tensor positions, Tensor qsl, Tensor state_slots, Tensor counts, "
         "int num_seqs, int H, int D, int Dv, Tensor decay, Tensor? tile_seq=None, Tensor? tile_q0=None, int num_tiles=0, "
         "bool plain_act=False) -> Tensor", &sm_lightning_scan);
@@ -638,7 +640,7 @@ TORCH_LIBRARY(dli, m) {
         "Tensor counts, int num_seqs, bool out_bf16) -> Tensor", &hm_causal_conv_add);
   m.def("hm_retention_prep(Tensor qkvg, Tensor positions, Tensor? freq, int rot_dims, int H, int D, int Dv, float k_scale) -> Tensor",
         &hm_retention_prep);
-  m.def("hm_act_mul(Tensor x, bool silu) -> Tensor", &hm_act_mul);
+  m.def("hm_act_mul(Tensor x, bool silu, float limit=0.0) -> Tensor", &hm_act_mul);
   m.def("hm_softmax_route(Tensor h, Tensor router, Tensor? bias, int K, bool all=False) -> (Tensor, Tensor)", &hm_softmax_route);
   m.def("rm_causal_conv(Tensor x, Tensor w, Tensor? bias, Tensor(a!) state, Tensor positions, Tensor token_seq, Tensor qsl, "
         "Tensor state_slots, Tensor counts, int num_seqs, bool out_bf16, bool silu, int unit_n, int unit_d, int unit_scaled, "
@@ -664,6 +666,15 @@ TORCH_LIBRARY(dli, m) {
   m.def("gm_gated_scan(Tensor q, Tensor k, Tensor v, Tensor decay, Tensor weight, Tensor(a!) state, Tensor positions, Tensor qsl, "
         "Tensor state_slots, Tensor counts, int num_seqs, int H, int G, int D, int Dv, bool delta, float q_scale, bool normaliser, "
         "Tensor? tile_seq, Tensor? tile_q0, int num_tiles) -> (Tensor, Tensor)", &gm_gated_scan);
+  m.def("gm_channel_scan(Tensor q, Tensor k, Tensor v, Tensor z, Tensor rate, Tensor bias, Tensor weight, Tensor(a!) state, "
+        "Tensor positions, Tensor qsl, Tensor state_slots, Tensor counts, int num_seqs, int H, int G, int D, int Dv, Tensor? tile_seq, "
+        "Tensor? tile_q0, int num_tiles) -> Tensor", &gm_channel_scan);
+  m.def("pm_embed_rows(Tensor ids, Tensor table, float scale) -> (Tensor, Tensor)", &pm_embed_rows);
+  m.def("pm_post_norm_add(Tensor(a!) x, Tensor y, Tensor w, float eps, Tensor? w2, bool out_bf16) -> Tensor", &pm_post_norm_add);
+  m.def("pm_head_norm_rope_cache(Tensor proj, Tensor? qw, Tensor? kw, float eps, Tensor positions, Tensor? freq, int rot_dims, "
+        "Tensor slot_mapping, Tensor(a!) k_cache, Tensor(b!) v_cache, int H, int G, int D, int Dv, int maps) -> Tensor",
+        &pm_head_norm_rope_cache);
+  m.def("pm_map_combine(Tensor o, Tensor lam, float eps, float scale, int G, Tensor(a!) out, Tensor? token_seq) -> ()", &pm_map_combine);
   m.def("dm_relu2_rows(Tensor x) -> Tensor", &dm_relu2_rows);
   m.def("dm_set_grouped_experts(bool on) -> ()", &dm_set_grouped_experts);
   m.def("dm_gated_combine(Tensor(a!) x, float mult, Tensor p0, Tensor p1, float s0, float s1, Tensor g1, Tensor b1, Tensor? ff, "

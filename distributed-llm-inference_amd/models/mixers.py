@@ -744,7 +744,7 @@ class MaskedAttention(nn.Module):
         self.s, self.eps, self.out_scale = spec, eps, out_scale
         H, G, D, Dv, M = spec.heads, spec.kv_heads, spec.dim, spec.vdim, spec.maps
         assert M in (1, 2) and H % G == 0 and spec.rot_dims % 2 == 0 and spec.rot_dims <= D
-        assert M == 1 or not (spec.sink or spec.score_cap), "differential maps have plain softmaxes"
+        assert M == 1 or not (spec.sink or spec.score_cap or spec.chunk or spec.keep_first), "differential maps have plain window softmaxes"
         self.in_cols, self.out_cols = (H + G) * M * D + G * Dv, H * Dv
         self.q_norm, self.k_norm = (_param((D,), ctx, device), _param((D,), ctx, device)) if spec.qk_weight else (None, None)
         self.sink = _param((H,), ctx, device) if spec.sink else None
@@ -775,7 +775,6 @@ class MaskedAttention(nn.Module):
     def forward(self, proj, out, meta, cache: LayerCache):
         s = self.s
         H, G, D, Dv, M = s.heads, s.kv_heads, s.dim, s.vdim, s.maps
-        T = proj.shape[0]
         if M == 2 and self._lam is None:
             a = self.lam.data
             self._lam = torch.exp((a[0] * a[1]).sum()) - torch.exp((a[2] * a[3]).sum()).reshape(1) + s.map_diff
@@ -787,10 +786,7 @@ class MaskedAttention(nn.Module):
                                    sink=self.sink.data if self.sink is not None else None, chunk=s.chunk, keep_first=s.keep_first,
                                    cap=s.score_cap, out_scale=self.out_scale)
             return
-        o = torch.empty(T, 2 * H, Dv, dtype=torch.float32, device=out.device)
-        seqmix.token_attention(o, q, None, cache.k, cache.v, meta, 2 * G, Dv, s.scale, s.window, chunk=s.chunk, keep_first=s.keep_first,
-                               value_heads=G)
-        seqmix.map_combine(o, self._lam, self.eps, (1.0 - s.map_diff) * self.out_scale, G, out, meta.token_seq)
+        seqmix.map_attention(out, q, cache.k, cache.v, meta, G, Dv, s.scale, s.window, self._lam, self.eps, (1.0 - s.map_diff) * self.out_scale)
 
 
 class ChannelDelta(nn.Module):

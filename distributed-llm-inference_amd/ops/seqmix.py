@@ -211,6 +211,18 @@ def latent_prep(q: torch.Tensor, dkv: torch.Tensor, cw: torch.Tensor, eps: float
 
 
 # ------------------------------------------------------------------------------------ attention over token-major pages
+def _attend_rows(lib, out, q1, q2, k_cache, v_cache, meta, rows, args, opts) -> None:
+    """The first ``rows`` tokens (< 0: all of them, no tile kernel ran) on the kernels that take one token per workgroup."""
+    T, H = q1.shape[0], q1.shape[1]
+    todo = T if rows < 0 else rows                           # tokens the tile kernel left (all of them in a pure decode step)
+    if (HEAD_DECODE and todo > 0 and q1.dtype == torch.bfloat16 and H // args[0] >= 8 and (rows >= 0 or meta.num_prefill_tiles == 0)
+            and lib.sm_head_decode_attention(out, q1, q2, k_cache, v_cache, meta.block_tables, meta.positions, meta.token_seq, *args, todo,
+                                             *opts)):
+        rows = 0                                             # done with the heads as matrix-core columns
+    if rows != 0:
+        lib.sm_token_attention(out, q1, q2, k_cache, v_cache, meta.block_tables, meta.positions, meta.token_seq, *args, rows, *opts)
+
+
 def token_attention(out: torch.Tensor, q1: torch.Tensor, q2: Optional[torch.Tensor], k_cache: torch.Tensor,
                     v_cache: Optional[torch.Tensor], meta, G: int, Dv: int, scale: float, window: int = 0,
                     temp: Optional[torch.Tensor] = None, r1: Optional[torch.Tensor] = None,
@@ -240,15 +252,7 @@ def token_attention(out: torch.Tensor, q1: torch.Tensor, q2: Optional[torch.Tens
                                      meta.prefill_tile_seq, meta.prefill_tile_q0, meta.num_prefill_tiles,
                                      meta.counts if meta.counts_on_device else None, G, Dv, scale, window, temp, r1, r2, gate, sink, *opts):
                 rows = meta.num_decode
-        T, H = q1.shape[0], q1.shape[1]
-        todo = T if rows < 0 else rows                       # tokens the tile kernel left (all of them in a pure decode step)
-        if (HEAD_DECODE and todo > 0 and q1.dtype == torch.bfloat16 and H // G >= 8 and meta.num_prefill_tiles == (0 if rows < 0 else meta.num_prefill_tiles)
-                and lib.sm_head_decode_attention(out, q1, q2, k_cache, v_cache, meta.block_tables, meta.positions, meta.token_seq,
-                                                 G, Dv, scale, window, temp, r1, r2, todo, gate, sink, *opts)):
-            rows = 0                                         # done with the heads as matrix-core columns
-        if rows != 0:
-            lib.sm_token_attention(out, q1, q2, k_cache, v_cache, meta.block_tables, meta.positions, meta.token_seq,
-                                   G, Dv, scale, window, temp, r1, r2, rows, gate, sink, *opts)
+        _attend_rows(lib, out, q1, q2, k_cache, v_cache, meta, rows, (G, Dv, scale, window, temp, r1, r2), (gate, sink, *opts))
         return out
     T, H, D1 = q1.shape
     rowk = k_cache.shape[-1]
@@ -993,7 +997,7 @@ def gated_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.T
 # Ops of stacks whose sublayers read the unnormed stream and add a norm of their output, of attention with per-head norms, chunk /
 # window masks, capped scores or two differential maps, and of the delta rule with a decay per key channel (``models/mixers.py``:
 # ``PostNormLayer``, ``MaskedAttention``, ``ChannelDelta``, ``ScaledPair``).  GPU kernels: ``csrc/kernels/postmix.hip``
-# (``torch.ops.dli.pm_*``) beside extensions of the kernels above.
+# (``torch.ops.dli.pm_*``), the recurrence's in ``csrc/kernels/gatemix.hip``, beside extensions of the kernels above.
 def embed_rows(ids: torch.Tensor, table: torch.Tensor, scale: float, out_dtype: torch.dtype):
     """``x = scale · table[ids]`` in fp32, and the same rows in ``out_dtype`` (what the first sublayer reads)."""
     if table.is_cuda:
@@ -1044,6 +1048,32 @@ def head_norm_rope_cache(proj: torch.Tensor, qw: Optional[torch.Tensor], kw: Opt
     return q.reshape(T, maps * H, D).to(proj.dtype)
 
 
+def map_attention(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, meta, G: int, Dv: int, scale: float,
+                  window: int, lam: torch.Tensor, eps: float, out_scale: float) -> None:
+    """Differential attention: two softmax maps per head over the same values (``token_attention``; ``q [T, 2H, D]`` ordered (key head, map,
+    head of its group), key rows ``[G, 2, D]``), combined by ``map_combine`` into ``out [T, H·Dv]``.  Prefill tiles do both maps and the
+    combination in one kernel."""
+    T, H2, _D = q.shape
+    rows = T
+    if _act_ok(q):
+        lib = _hip()
+        args, opts = (2 * G, Dv, scale, window, None, None, None), (None, None, 0, 0, 0.0, G)
+        if TILE_ATTENTION and q.dtype == torch.bfloat16 and meta.num_prefill_tiles > 0:
+            if lib.sm_tile_attention(out.unflatten(1, (H2 // 2, Dv)), q, None, k_cache, v_cache, meta.block_tables, meta.seq_lens,
+                                     meta.query_start_loc, meta.prefill_tile_seq, meta.prefill_tile_q0, meta.num_prefill_tiles,
+                                     meta.counts if meta.counts_on_device else None, *args, *opts, out_scale, lam, eps):
+                rows = meta.num_decode
+        if rows == 0:
+            return
+        o = torch.empty(rows, H2, Dv, dtype=torch.float32, device=out.device)
+        _attend_rows(lib, o, q[:rows], None, k_cache, v_cache, meta, rows if rows < T else -1, args, (*opts, 1.0))
+        map_combine(o, lam, eps, out_scale, G, out[:rows], meta.token_seq)
+        return
+    o = torch.empty(T, H2, Dv)
+    token_attention(o, q, None, k_cache, v_cache, meta, 2 * G, Dv, scale, window, value_heads=G)
+    map_combine(o, lam, eps, out_scale, G, out)
+
+
 def map_combine(o: torch.Tensor, lam: torch.Tensor, eps: float, scale: float, G: int, out: torch.Tensor, token_seq: Optional[torch.Tensor] = None):
     """Two attention maps per head, ``o`` fp32 ``[T, 2H, Dv]`` ordered (key head, map, head of its group): ``d = o₁ - lam · o₂`` (``lam`` fp32
     ``[1]``), ``out[t, h] = scale · d / sqrt(mean(d²) + eps)`` in head order (``out [T, H·Dv]``, a row-strided view; rows with a negative
@@ -1066,9 +1096,9 @@ def channel_delta_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, z: tor
     ``o = Sᵀ q``.  Returns fp32 ``[T, H·Dv]``."""
     if _act_ok(z):
         tiles = meta.num_prefill_tiles if BLOCK_SCAN else 0
-        return _hip().pm_channel_delta_scan(q, k, v, z, rate, bias, weight, state, meta.positions, meta.query_start_loc, meta.state_slots,
-                                            meta.counts, meta.num_seqs, H, G, D, Dv, meta.prefill_tile_seq if tiles else None,
-                                            meta.prefill_tile_q0 if tiles else None, tiles)
+        return _hip().gm_channel_scan(q, k, v, z, rate, bias, weight, state, meta.positions, meta.query_start_loc, meta.state_slots,
+                                      meta.counts, meta.num_seqs, H, G, D, Dv, meta.prefill_tile_seq if tiles else None,
+                                      meta.prefill_tile_q0 if tiles else None, tiles)
     T = q.shape[0]
     qf, kf = (t.reshape(T, G, D).repeat_interleave(H // G, dim=1) for t in (q, k))
     vf = v.reshape(T, H, Dv)
