@@ -263,7 +263,7 @@ def random_weights(cfg, seed=0, ranks=(6, 10)):
             H, G, D, Dv = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
             W.update({p + "q": mat(H * 2 * D, Wd), p + "k": mat(G * 2 * D, Wd), p + "v": mat(G * Dv, Wd), p + "q.norm": vec(D, 1.3, 0.3),
                       p + "k.norm": vec(D, 1.3, 0.3), p + "o": mat(Wd, H * Dv)})
-            W.update({p + s: vec(D, 0.0, 0.7 * D ** -0.25) for s in ("lq1", "lk1", "lq2", "lk2")})
+            W.update({p + s: vec(D, 0.0, 0.55 * D ** -0.25) for s in ("lq1", "lk1", "lq2", "lk2")})
         else:
             a, b = m["left"], m["right"]
             H, G, D, Dv = a["heads"], a["kv_heads"], a["dim"], a["vdim"]
