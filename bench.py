@@ -14,6 +14,8 @@
                                                       # side benchmark: Sevelorn stacks beside their closest families
     python bench.py --mixers --models rodelix-lightning,sinilorn-recurrence,rodelix-latent_attention,sinilorn-latent,mixtral,sinilorn
                                                       # side benchmark: Sinilorn stacks beside their closest families
+    python bench.py --mixers --models rodelix-attention,mozalix-chunk,mozalix-diff,nefarax-delta,mozalix-delta,mozalix-pair,llama,mozalix
+                                                     # side benchmark: Mozalix stacks beside their closest families
     python bench.py --mixers --models rodelix-lightning,nefarax-delta,nefarax-mlstm,rodelix-attention,nefarax-pair,nefarax
                                                       # side benchmark: Nefarax stacks beside their closest families
 

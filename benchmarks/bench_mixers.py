@@ -39,6 +39,14 @@ tanh norm per layer, mixer and plain tanh-GELU feed-forward of 1.5× the Llama F
 ``nefarax-mlstm`` = mLSTM (heads of 128 × 128) — both beside ``rodelix-lightning``, the framework's other ``[128, 128]`` state per head;
 ``nefarax-pair`` = convolved attention beside a Mamba-2 recurrence (inner width twice the model width in heads of 64, state 128) —
 beside ``rodelix-attention`` (attention) and ``rodelix-lightning`` (recurrence); ``nefarax`` = one layer of each.
+
+``--models rodelix-attention,mozalix-chunk,mozalix-diff,nefarax-delta,mozalix-delta,mozalix-pair,llama,mozalix`` compares the Mozalix
+stacks (post-norm layers on the unnormed stream, a clamped gated feed-forward with biases of the Llama FFN width) with their closest
+families: ``mozalix-chunk`` = attention in chunks of 1024 with a sink and ``mozalix-diff`` = differential attention over a window of 1024
+(two maps of 64 per head of 128) — both beside ``rodelix-attention`` (window 1024); ``mozalix-pair`` = soft-capped window attention
+(1024, four kept tokens) beside the delta rule with channel decays (half as many q / k heads as value heads, heads of 128 × 128,
+four taps, both low ranks 128) — beside ``rodelix-attention`` and ``nefarax-delta``; ``mozalix-delta`` = the same with the attention half cut to
+one head of 16 over a window of 32, for the recurrence alone; ``mozalix`` = one layer of chunk, diff and pair.
 """
 from __future__ import annotations
 
@@ -129,8 +137,24 @@ def nefarax_raw(width, heads, kv, ffn, kinds):
             "layers": [mk[k] for k in kinds]}
 
 
+def mozalix_raw(width, heads, kv, ffn, kinds):
+    ff = {"kind": "dense", "ff": ffn, "limit": 7.0}
+    att = {"heads": heads, "kv_heads": kv, "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "mask": {"size": 1024}}
+    left = dict(att, softcap=30.0, mask={"size": 1024, "keep_first": 4})
+    little = {"heads": 1, "kv_heads": 1, "dim": 16, "vdim": 16, "scale": 0.25, "softcap": 30.0, "mask": {"size": 32, "keep_first": 0}}
+    right = {"heads": heads, "kv_heads": heads // 2, "dim": 128, "vdim": 128, "conv": 4, "lora": 128, "gate_lora": 128}
+    mk = {
+        "chunk": {"type": "attention", "mlp": ff, "mixer": dict(att, rot={"base": 500000.0, "dims": 64})},
+        "diff": {"type": "attention_2", "mlp": ff, "mixer": dict(att, dim=64, scale=0.125, diff=0.5, rot={"base": 500000.0, "dims": 64})},
+        "pair": {"type": "parallel", "mlp": ff, "mixer": {"left_scale": 0.7, "right_scale": 0.7, "left": left, "right": right}},
+        "delta": {"type": "parallel", "mlp": ff, "mixer": {"left_scale": 0.7, "right_scale": 0.7, "left": little, "right": right}},
+    }
+    return {"architecture": "Mozalix", "vocab": 32000, "width": width, "embedding": {"scale": 1.0}, "norm": {"eps": 1e-5},
+            "layers": [mk[k] for k in kinds]}
+
+
 def model_configs(size):
-    from dli_amd.config import ModelConfig, nefarax_config, rodelix_config, sevelorn_config, sinilorn_config, vibunex_config
+    from dli_amd.config import ModelConfig, mozalix_config, nefarax_config, rodelix_config, sevelorn_config, sinilorn_config, vibunex_config
     s = SIZES[size]
     out = {"llama": ModelConfig(name=f"llama-{size}", arch="llama", vocab_size=32000, hidden_size=s["width"],
                                 intermediate_size=s["ffn"], num_layers=LAYERS, num_heads=s["heads"], num_kv_heads=s["kv"],
@@ -148,6 +172,9 @@ def model_configs(size):
     for name, kinds in (("nefarax", ("delta", "mlstm", "pair")), ("nefarax-delta", ("delta",) * LAYERS), ("nefarax-mlstm", ("mlstm",) * LAYERS),
                         ("nefarax-pair", ("pair",) * LAYERS)):
         out[name] = nefarax_config(nefarax_raw(s["width"], s["heads"], s["kv"], s["ffn"], kinds), name=f"{name}-{size}")
+    for name, kinds in (("mozalix", ("chunk", "diff", "pair")), ("mozalix-chunk", ("chunk",) * LAYERS), ("mozalix-diff", ("diff",) * LAYERS),
+                        ("mozalix-pair", ("pair",) * LAYERS), ("mozalix-delta", ("delta",) * LAYERS)):
+        out[name] = mozalix_config(mozalix_raw(s["width"], s["heads"], s["kv"], s["ffn"], kinds), name=f"{name}-{size}")
     kinds = ("attention", "lightning", "latent_attention")
     out["rodelix"] = rodelix_config(rodelix_raw(s["width"], s["heads"], s["kv"], s["ffn"], kinds), name=f"rodelix-{size}")
     for k in kinds:
