@@ -89,6 +89,13 @@ __device__ __forceinline__ float wave_max(float v) {
   return v;
 }
 
+// workgroup barrier for data exchanged through LDS only: fetches from memory stay in flight
+__device__ __forceinline__ void lds_barrier() {
+  asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+  __builtin_amdgcn_s_barrier();
+  asm volatile("" ::: "memory");
+}
+
 // Block-wide sum for blockDim.x = NT (multiple of 64).  `red` is NT/64 floats of LDS.
 template <int NT>
 __device__ __forceinline__ float block_sum(float v, float* red) {

@@ -657,12 +657,6 @@ template <typename A> __device__ __forceinline__ typename Raw<A>::v4 raw4(const 
   for (int j = 0; j < 4; ++j) r[j] = d + j < D ? row[d + j] : A(0);
   return r;
 }
-// workgroup barrier for data exchanged through LDS only: fetches from memory stay in flight
-__device__ __forceinline__ void lds_barrier() {
-  asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
-  __builtin_amdgcn_s_barrier();
-  asm volatile("" ::: "memory");
-}
 // CHAN (delta rule, A = float): q, k and kᵀ come from the workspace with their channel decays in them (channel_block_kernel).
 template <typename A, bool DELTA, int DTMAX, int CT, bool CHAN>
 __global__ __launch_bounds__(NT) void scan_walk_kernel(const A* __restrict__ q, int64_t q_stride, const A* __restrict__ k, int64_t k_stride,

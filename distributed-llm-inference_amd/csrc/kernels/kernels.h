@@ -95,7 +95,7 @@ struct AttnOpts {
   int vshare = 1;                 // consecutive key heads per value head
   float out_scale = 1.f;
   float* out_f32 = nullptr;       // results here in fp32 (the strides of `out`)
-  const float* lam = nullptr;     // tile kernel: differential maps (out = out_scale · d / rms(d), d = map 1 - lam · map 2)
+  const float* lam = nullptr;     // differential maps: out = out_scale · d / rms(d), d = map 1 - lam · map 2 (per-token kernels: through `part`)
   float eps = 0.f;
 };
 void launch_sm_token_attention(void* out, int64_t o_ts, int64_t o_hs, const void* q1, int64_t q1_ts, int64_t q1_hs, int D1,

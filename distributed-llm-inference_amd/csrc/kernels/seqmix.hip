@@ -598,7 +598,11 @@ __global__ __launch_bounds__(NT) void token_attention_kernel(
   const int64_t t = blockIdx.x;
   const int h0 = blockIdx.y * HG;        // first head of the group (all HG heads share one key / value head)
   const int seq = token_seq[t];
-  if (seq < 0) return;
+  if (seq < 0) {                         // padding row: zeros (from the merge kernel where there is one)
+    if (part == nullptr)
+      for (int i = threadIdx.x; i < HG * Dv; i += NT) store_out(out, opt, t * o_ts + (h0 + i / Dv) * o_hs + i % Dv, 0.f);
+    return;
+  }
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int Dk = D1 + D2;
   const int p = positions[t];
@@ -768,7 +772,7 @@ __global__ __launch_bounds__(NT) void token_attention_kernel(
       L += f * ls[w * HG + hh];
       o += f * accs[(w * HG + hh) * Dv + e];
     }
-    if (nsplit == 1) {
+    if (part == nullptr) {
       const float gm = gate != nullptr ? 1.f / (1.f + expf(-ldf<A>(gate + t * g_ts + h0 + hh))) : 1.f;
       if (sink != nullptr) L += expf(sink[h0 + hh] - M);            // a logit without key or value in the denominator
       store_out(out, opt, t * o_ts + (h0 + hh) * o_hs + e, o / L * gm * opt.out_scale);
@@ -792,7 +796,10 @@ __global__ __launch_bounds__(128) void token_attention_merge_kernel(A* __restric
                                                                     AttnOpts opt) {
   const int64_t t = blockIdx.x;
   const int h = blockIdx.y;
-  if (token_seq[t] < 0) return;
+  if (token_seq[t] < 0) {
+    for (int e = threadIdx.x; e < Dv; e += 128) store_out(out, opt, t * o_ts + h * o_hs + e, 0.f);
+    return;
+  }
   const float* pr = part + (t * H + h) * nsplit * (int64_t)(Dv + 2);
   float M = -INFINITY;
   for (int z = 0; z < nsplit; ++z) M = fmaxf(M, pr[z * (Dv + 2)]);
@@ -815,6 +822,56 @@ __global__ __launch_bounds__(128) void token_attention_merge_kernel(A* __restric
   }
 }
 
+// The same for differential maps: part [T][2H][nsplit][2 + Dv], query vectors ordered (value head, map, head of its group); out [T][H][Dv] =
+// out_scale · d / rms(d), d = map 1 - lam · map 2.
+template <typename A>
+__global__ __launch_bounds__(128) void map_merge_kernel(A* __restrict__ out, int64_t o_ts, int64_t o_hs, const float* __restrict__ part,
+                                                        const int* __restrict__ token_seq, int per, int Dv, int nsplit, AttnOpts opt) {
+  __shared__ float red[2];
+  const int64_t t = blockIdx.x;
+  const int head = blockIdx.y, H2 = 2 * gridDim.y;
+  A* o = out + t * o_ts + head * o_hs;
+  if (token_seq[t] < 0) {
+    for (int e = threadIdx.x; e < Dv; e += 128) stf<A>(o + e, 0.f);
+    return;
+  }
+  const int64_t ps = Dv + 2;
+  const float* pr[2];
+  float f[2][16];
+#pragma unroll
+  for (int m = 0; m < 2; ++m) {
+    pr[m] = part + (t * H2 + (head / per * 2 + m) * per + head % per) * nsplit * ps;
+    float M = -INFINITY, L = 0.f;
+    for (int z = 0; z < nsplit; ++z) M = fmaxf(M, pr[m][z * ps]);
+#pragma unroll
+    for (int z = 0; z < 16; ++z) {
+      const float mz = z < nsplit ? pr[m][z * ps] : -INFINITY;
+      f[m][z] = mz == -INFINITY ? 0.f : expf(mz - M);
+      if (z < nsplit) L += f[m][z] * pr[m][z * ps + 1];
+    }
+    const float r = (m == 0 ? 1.f : -opt.lam[0]) / L;
+#pragma unroll
+    for (int z = 0; z < 16; ++z) f[m][z] *= r;
+  }
+  auto value = [&](int e) {
+    float d = 0.f;
+#pragma unroll
+    for (int z = 0; z < 16; ++z)
+      if (z < nsplit) d += f[0][z] * pr[0][z * ps + 2 + e] + f[1][z] * pr[1][z * ps + 2 + e];
+    return d;
+  };
+  float d[4], ss = 0.f;                                   // Dv ≤ 512
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    d[i] = threadIdx.x + 128 * i < Dv ? value(threadIdx.x + 128 * i) : 0.f;
+    ss += d[i] * d[i];
+  }
+  const float inv = opt.out_scale / sqrtf(block_sum<128>(ss, red) / (float)Dv + opt.eps);
+#pragma unroll
+  for (int i = 0; i < 4; ++i)
+    if (threadIdx.x + 128 * i < Dv) stf<A>(o + threadIdx.x + 128 * i, d[i] * inv);
+}
+
 // ------------------------------------------------------------------------------------------------ attention, prefill tiles
 // bf16 only.  One workgroup per (64-query tile of one sequence's chunk, query head); a wave owns 16 queries.  Per 32-key
 // page: the page's key rows (this head's slice) and its value rows, transposed, are staged in LDS once for the four
@@ -824,10 +881,11 @@ __global__ __launch_bounds__(128) void token_attention_merge_kernel(A* __restric
 // remainder (two MFMAs: P enters the product with 16 mantissa bits, not 8).  The lane's eight Sᵀ values (two 16-key
 // tiles) are, in register order, the B fragment of the P·V k-step when the staged V columns sit in the slot order
 // slot(t) = ((t & 15) >> 2)·8 + (t >> 4)·4 + (t & 3).  KSMAX / MTMAX: compile-time bounds of ceil(Dk / 32) and Dv / 16.
-// DIFF (HW = 2): the two halves of the workgroup are the two maps of one head — each with a key slice of its own, values shared;
-// map 2's result goes through LDS and map 1's waves write scale · d / rms(d), d = a1 - lam · a2.
+// DIFF: every two groups of four waves are the two maps of one head — each with a key slice of its own, values shared; map 2's result
+// goes through LDS and map 1's waves write scale · d / rms(d), d = a1 - lam · a2.
+// Up to 256-wide keys (KSMAX ≤ 8) the next page is fetched into registers while this one is computed; the barriers wait for LDS only.
 template <int KSMAX, int MTMAX, int HW, bool DIFF>
-__global__ __launch_bounds__(NT * HW) void tile_attention_kernel(
+__global__ __launch_bounds__(NT * HW, KSMAX <= 4 ? 4 : (KSMAX <= 8 ? 2 : 1)) void tile_attention_kernel(
     uint16_t* __restrict__ out, int64_t o_ts, int64_t o_hs, const uint16_t* __restrict__ q1, int64_t q1_ts, int64_t q1_hs, int D1,
     const uint16_t* __restrict__ q2, int64_t q2_ts, int64_t q2_hs, int D2, const uint16_t* __restrict__ kc, int rowk,
     const uint16_t* __restrict__ vc, int rowv, int vhead, int Dv, const int* __restrict__ block_tables, int max_blocks,
@@ -843,9 +901,12 @@ __global__ __launch_bounds__(NT * HW) void tile_attention_kernel(
   // HW heads of one key / value group per workgroup (4 waves each): the staged page serves all of them
   constexpr int TNT = NT * HW;
   const int wave_all = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
-  const int map = DIFF ? wave_all >> 2 : 0, per = H / G;
-  // DIFF: blockIdx.y counts (value head, head of its group); query heads are ordered (value head, map, head of its group)
-  const int h = DIFF ? ((int)blockIdx.y / per * 2 + map) * per + (int)blockIdx.y % per : (int)blockIdx.y * HW + (wave_all >> 2);
+  constexpr int KROWS = DIFF ? 64 : 32;                   // staged key rows per page
+  constexpr bool PREF = KSMAX <= 8;
+  const int map = DIFF ? (wave_all >> 2) & 1 : 0, per = H / G;
+  // DIFF: `head` counts (value head, head of its group); query heads are ordered (value head, map, head of its group)
+  const int head = DIFF ? (int)blockIdx.y * (HW / 2) + (wave_all >> 3) : (int)blockIdx.y * HW + (wave_all >> 2);
+  const int h = DIFF ? (head / per * 2 + map) * per + head % per : head;
   const int seq = tile_seq[tile], q0 = tile_q0[tile];
   const int t_begin = qsl[seq];
   const int n_chunk = qsl[seq + 1] - t_begin;
@@ -857,13 +918,13 @@ __global__ __launch_bounds__(NT * HW) void tile_attention_kernel(
   const int Dk = D1 + D2;
   const int KS = (Dk + 31) >> 5, MT = Dv >> 4;
   const int KST = KS * 32 + 8;                            // LDS row strides (elements): +16 bytes against bank conflicts
-  constexpr int VST = 40;
+  constexpr int VST = 36;                                 // 18 dwords: 8-byte writes of eight 4-row groups × 8 columns hit all banks
   uint16_t* Ks = tl;                                      // [DIFF ? 2 maps : 1][32][KST]
-  uint16_t* Vt = tl + (DIFF ? 64 : 32) * KST;
+  uint16_t* Vt = tl + KROWS * KST;
   const int g = h / per, gv = g / opt.vshare, g0 = g - map;    // g0: key head of the first staged slice
 
   // zero the K padding columns once (Dk not a multiple of 32): they are never staged over
-  for (int i = threadIdx.x; i < (DIFF ? 64 : 32) * (KS * 32 - Dk); i += TNT) {
+  for (int i = threadIdx.x; i < KROWS * (KS * 32 - Dk); i += TNT) {
     const int row = i / (KS * 32 - Dk), col = Dk + i % (KS * 32 - Dk);
     Ks[row * KST + col] = 0;
   }
@@ -906,25 +967,73 @@ __global__ __launch_bounds__(NT * HW) void tile_attention_kernel(
   const int kchunks = Dk >> 3, vchunks = Dv >> 3;
   const bool vfromk = vc == kc && rowv == rowk && vhead == Dk;     // latent attention: one row is key and value
   const uint16_t* Km = Ks + map * 32 * KST;
+  // staging: keys in 16-byte pieces of a row; values in groups of 4 rows × 8 columns, whose slots are neighbours in Vt
+  auto page_of = [&](int it) { return (int64_t)bt[it < kb_lo ? it - (kb_lo - kept_pages) : it] * kBlockTokens; };
+  auto put_values = [&](int i, bf16x8 v0, bf16x8 v1, bf16x8 v2, bf16x8 v3) {
+    const int rg = i & 7;
+    uint16_t* dst = Vt + (i >> 3) * 8 * VST + (rg & 3) * 8 + (rg >> 2) * 4;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) *reinterpret_cast<bf16x4*>(dst + j * VST) = bf16x4{v0[j], v1[j], v2[j], v3[j]};
+  };
+  constexpr int NKP = PREF ? (KROWS * KSMAX * 4 + TNT - 1) / TNT : 1, NVP = PREF ? (16 * MTMAX + TNT - 1) / TNT : 1;
+  bf16x8 kr[NKP], vr[NVP][4];
+  int kg[NKP], kl[NKP];
+  if constexpr (PREF) {
+#pragma unroll
+    for (int u = 0; u < NKP; ++u) {
+      const int i = threadIdx.x + u * TNT, srow = i / kchunks, ch = i - srow * kchunks;
+      kl[u] = i < KROWS * kchunks ? srow * KST + 8 * ch : -1;
+      kg[u] = (srow & 31) * rowk + (DIFF ? g0 + (srow >> 5) : g) * Dk + 8 * ch;
+    }
+  }
+  auto fetch = [&](int64_t page_row) {
+#pragma unroll
+    for (int u = 0; u < NKP; ++u)
+      if (kl[u] >= 0) kr[u] = *reinterpret_cast<const bf16x8*>(kc + page_row * rowk + kg[u]);
+#pragma unroll
+    for (int u = 0; u < NVP; ++u) {
+      const int i = threadIdx.x + u * TNT;
+      if (i < 8 * vchunks) {
+        const uint16_t* p = vc + (page_row + 4 * (i & 7)) * rowv + gv * vhead + 8 * (i >> 3);
+#pragma unroll
+        for (int r = 0; r < 4; ++r) vr[u][r] = *reinterpret_cast<const bf16x8*>(p + (int64_t)r * rowv);
+      }
+    }
+  };
+  if constexpr (PREF) fetch(page_of(kb_lo - kept_pages));
   for (int it = kb_lo - kept_pages; it <= kb_hi; ++it) {
     const int kb = it < kb_lo ? it - (kb_lo - kept_pages) : it;
-    __syncthreads();                                      // everyone is done with the previous page
-    const int64_t page_row = (int64_t)bt[kb] * kBlockTokens;
-    for (int i = threadIdx.x; i < (DIFF ? 64 : 32) * kchunks; i += TNT) {
-      const int srow = i / kchunks, ch = i - srow * kchunks, row = srow & 31;
-      *reinterpret_cast<bf16x8*>(Ks + srow * KST + 8 * ch) =
-          *reinterpret_cast<const bf16x8*>(kc + (page_row + row) * rowk + (DIFF ? g0 + (srow >> 5) : g) * Dk + 8 * ch);
-    }
-    if (vfromk) __syncthreads();                          // values = leading columns of the key rows just staged
-    for (int i = threadIdx.x; i < 32 * vchunks; i += TNT) {
-      const int row = i & 31, ch = i >> 5;
-      const bf16x8 v = vfromk ? *reinterpret_cast<const bf16x8*>(Ks + row * KST + 8 * ch)
-                              : *reinterpret_cast<const bf16x8*>(vc + (page_row + row) * rowv + gv * vhead + 8 * ch);
-      const int slot = ((row & 15) >> 2) * 8 + (row >> 4) * 4 + (row & 3);
+    if constexpr (PREF) {
+      lds_barrier();                                      // everyone is done with the previous page
 #pragma unroll
-      for (int j = 0; j < 8; ++j) Vt[(8 * ch + j) * VST + slot] = (uint16_t)v[j];
+      for (int u = 0; u < NKP; ++u)
+        if (kl[u] >= 0) *reinterpret_cast<bf16x8*>(Ks + kl[u]) = kr[u];
+#pragma unroll
+      for (int u = 0; u < NVP; ++u) {
+        const int i = threadIdx.x + u * TNT;
+        if (i < 8 * vchunks) put_values(i, vr[u][0], vr[u][1], vr[u][2], vr[u][3]);
+      }
+      if (it < kb_hi) fetch(page_of(it + 1));
+      lds_barrier();
+    } else {
+      __syncthreads();                                    // everyone is done with the previous page
+      const int64_t page_row = page_of(it);
+      for (int i = threadIdx.x; i < KROWS * kchunks; i += TNT) {
+        const int srow = i / kchunks, ch = i - srow * kchunks;
+        *reinterpret_cast<bf16x8*>(Ks + srow * KST + 8 * ch) =
+            *reinterpret_cast<const bf16x8*>(kc + (page_row + (srow & 31)) * rowk + (DIFF ? g0 + (srow >> 5) : g) * Dk + 8 * ch);
+      }
+      if (vfromk) __syncthreads();                        // values = leading columns of the key rows just staged
+      for (int i = threadIdx.x; i < 32 * vchunks; i += TNT) {
+        const int row = i & 31, ch = i >> 5;
+        const bf16x8 v = vfromk ? *reinterpret_cast<const bf16x8*>(Ks + row * KST + 8 * ch)
+                                : *reinterpret_cast<const bf16x8*>(vc + (page_row + row) * rowv + gv * vhead + 8 * ch);
+        const int slot = ((row & 15) >> 2) * 8 + (row >> 4) * 4 + (row & 3);
+#pragma unroll
+        for (int j = 0; j < 8; ++j) Vt[(8 * ch + j) * VST + slot] = (uint16_t)v[j];
+      }
+      __syncthreads();
     }
-    __syncthreads();
 
     f32x4 sa = {0.f, 0.f, 0.f, 0.f}, sb = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
@@ -973,7 +1082,8 @@ __global__ __launch_bounds__(NT * HW) void tile_attention_kernel(
 #pragma unroll
     for (int i = 0; i < MTMAX; ++i) {
       if (i < MT) {
-        const bf16x8 vf = *reinterpret_cast<const bf16x8*>(Vt + (16 * i + c) * VST + 8 * g4);
+        const bf16x4* vp = reinterpret_cast<const bf16x4*>(Vt + (16 * i + c) * VST + 8 * g4);
+        const bf16x8 vf = __builtin_shufflevector(vp[0], vp[1], 0, 1, 2, 3, 4, 5, 6, 7);
         f32x4 a = acc[i];
         a[0] *= corr; a[1] *= corr; a[2] *= corr; a[3] *= corr;
         a = mfma16(vf, ph, a);
@@ -984,7 +1094,7 @@ __global__ __launch_bounds__(NT * HW) void tile_attention_kernel(
   l += __shfl_xor(l, 16, 64);
   l += __shfl_xor(l, 32, 64);
   if constexpr (DIFF) {
-    float* X = reinterpret_cast<float*>(tl) + wave * MT * 256 + lane;      // [wave][value tile · 4 + r][lane]
+    float* X = reinterpret_cast<float*>(tl) + ((wave_all >> 3) * 4 + wave) * MT * 256 + lane;      // [head][wave][value tile · 4 + r][lane]
     __syncthreads();                                      // the last page's readers are done
     if (map == 1) {
       const float rl = opt.lam[0] / l;
@@ -997,23 +1107,29 @@ __global__ __launch_bounds__(NT * HW) void tile_attention_kernel(
     __syncthreads();
     if (map == 1) return;
     const float rl = 1.f / l;
-    float ss = 0.f;
+    float ss = 0.f;                                       // (the differences are formed twice: kept, they would cost a wave of occupancy)
 #pragma unroll
     for (int i = 0; i < MTMAX; ++i)
-      if (i < MT)
+      if (i < MT) {
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          acc[i][r] = acc[i][r] * rl - X[(4 * i + r) * 64];
-          ss += acc[i][r] * acc[i][r];
+          const float d = acc[i][r] * rl - X[(4 * i + r) * 64];
+          ss += d * d;
         }
+      }
     ss += __shfl_xor(ss, 16, 64);
     ss += __shfl_xor(ss, 32, 64);
     if (!qvalid) return;
     const float inv = opt.out_scale / sqrtf(ss / (float)Dv + opt.eps);
-    uint16_t* orow = out + tq * o_ts + (int64_t)blockIdx.y * o_hs;
+    uint16_t* orow = out + tq * o_ts + (int64_t)head * o_hs;
 #pragma unroll
     for (int i = 0; i < MTMAX; ++i)
-      if (i < MT) st4<uint16_t>(orow + 16 * i + 4 * g4, f32x4{acc[i][0] * inv, acc[i][1] * inv, acc[i][2] * inv, acc[i][3] * inv});
+      if (i < MT) {
+        f32x4 d;
+#pragma unroll
+        for (int r = 0; r < 4; ++r) d[r] = (acc[i][r] * rl - X[(4 * i + r) * 64]) * inv;
+        st4<uint16_t>(orow + 16 * i + 4 * g4, d);
+      }
     return;
   }
   if (!qvalid) return;
@@ -1047,9 +1163,13 @@ __global__ __launch_bounds__(NT) void head_decode_attention_kernel(
     float* __restrict__ part, const uint16_t* __restrict__ gate, int64_t g_ts, const float* __restrict__ sink, AttnOpts opt) {
   extern __shared__ __align__(16) uint16_t tl[];
   const int64_t t = blockIdx.x;
-  const int seq = token_seq[t];
-  if (seq < 0) return;
-  const int per = H / G;
+  const int seq = token_seq[t], per = H / G;
+  if (seq < 0) {                                          // padding row: zeros (from the merge kernel where there is one)
+    const int hb = blockIdx.y / groups * per + 16 * (blockIdx.y % groups), n = min(16, per - 16 * (int)(blockIdx.y % groups)) * Dv;
+    if (part == nullptr)
+      for (int i = threadIdx.x; i < n; i += NT) store_out(out, opt, t * o_ts + (hb + i / Dv) * o_hs + i % Dv, 0.f);
+    return;
+  }
   const int g = blockIdx.y / groups, grp = blockIdx.y - g * groups, gv = g / opt.vshare;
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int lane = threadIdx.x & 63, g4 = lane >> 4, c = lane & 15;
@@ -1169,7 +1289,7 @@ __global__ __launch_bounds__(NT) void head_decode_attention_kernel(
   l += __shfl_xor(l, 16, 64);
   l += __shfl_xor(l, 32, 64);
   if (!hvalid) return;
-  if (nsplit == 1) {
+  if (part == nullptr) {
     if (sink != nullptr) l += fast_exp2(sink[h] * 1.4426950408889634f - m);
     const float rl = (gate != nullptr ? 1.f / (1.f + expf(-bf2f(gate[t * g_ts + h]))) : 1.f) / l * opt.out_scale;
     const int64_t o0 = t * o_ts + h * o_hs;
@@ -1496,7 +1616,10 @@ void launch_sm_token_attention(void* out, int64_t o_ts, int64_t o_hs, const void
   else if (nv <= 4) SM_ATT_V(4);
   else SM_ATT_V(8);
 #undef SM_ATT_V
-  if (nsplit > 1)
+  if (opt.lam != nullptr)
+    SM_DISPATCH_BF16(bf16, A, hipLaunchKernelGGL(map_merge_kernel<A>, dim3(rows, H / 2), dim3(128), 0, stream, (A*)out, o_ts, o_hs,
+                                                 (const float*)part, token_seq, per, Dv, nsplit, opt));
+  else if (nsplit > 1)
     SM_DISPATCH_BF16(bf16, A, hipLaunchKernelGGL(token_attention_merge_kernel<A>, dim3(rows, H), dim3(128), 0, stream, (A*)out, o_ts,
                                                  o_hs, (const float*)part, token_seq, H, Dv, nsplit, (const A*)gate, g_ts, sink, opt));
 }
@@ -1525,10 +1648,12 @@ bool launch_sm_tile_attention(void* out, int64_t o_ts, int64_t o_hs, const void*
                   o_hs % 4 == 0 && al(out, 8) && al(opt.out_f32, 16) && al(q1, 16) && al(q2, 16) && al(kc, 16) && al(vc, 16);
   if (!ok || (diff && (KS > 8 || MT > 16))) return false;
   if (num_tiles == 0) return true;
-  size_t lds = (size_t)((diff ? 64 : 32) * (KS * 32 + 8) + Dv * 40) * sizeof(uint16_t);
-  if (diff) lds = std::max(lds, (size_t)64 * Dv * sizeof(float));
-  // two heads of a key / value group (or the two maps of a head) per workgroup (8 waves) where the group has an even number of heads
-  const int hw = diff || (H / G) % 2 == 0 ? 2 : 1;
+  size_t lds = (size_t)((diff ? 64 : 32) * (KS * 32 + 8) + Dv * 36) * sizeof(uint16_t);
+  // two heads of a key / value group per workgroup (8 waves) where the group has an even number of heads; with two maps 16 waves
+  // for two heads
+  const bool even = (H / G) % 2 == 0;
+  const int hw = diff ? (even && KS <= 4 && MT <= 8 ? 4 : 2) : (even ? 2 : 1);
+  if (diff) lds = std::max(lds, (size_t)hw / 2 * 64 * Dv * sizeof(float));
   const dim3 grid(num_tiles, H / hw);
 #define SM_TILE_HW(KSM, MTM, HWV, DIFF)                                                                                                \
   do {                                                                                                                           \
@@ -1549,7 +1674,8 @@ bool launch_sm_tile_attention(void* out, int64_t o_ts, int64_t o_hs, const void*
     else SM_TILE_HW(KSM, MTM, 1, false);      \
   } while (0)
   if (diff) {
-    if (KS <= 4 && MT <= 8) SM_TILE_HW(4, 8, 2, true);
+    if (hw == 4) SM_TILE_HW(4, 8, 4, true);
+    else if (KS <= 4 && MT <= 8) SM_TILE_HW(4, 8, 2, true);
     else SM_TILE_HW(8, 16, 2, true);
     return true;
   }
@@ -1595,7 +1721,10 @@ bool launch_sm_head_decode_attention(void* out, int64_t o_ts, int64_t o_hs, cons
   else if (KS <= 8 && MT <= 16) SM_HD(8, 4);
   else SM_HD(18, 8);
 #undef SM_HD
-  if (nsplit > 1)
+  if (opt.lam != nullptr)
+    hipLaunchKernelGGL(map_merge_kernel<uint16_t>, dim3(rows, H / 2), dim3(128), 0, stream, (uint16_t*)out, o_ts, o_hs, (const float*)part,
+                       token_seq, per, Dv, nsplit, opt);
+  else if (nsplit > 1)
     hipLaunchKernelGGL(token_attention_merge_kernel<uint16_t>, dim3(rows, H), dim3(128), 0, stream, (uint16_t*)out, o_ts, o_hs,
                        (const float*)part, token_seq, H, Dv, nsplit, (const uint16_t*)gate, g_ts, sink, opt);
   return true;

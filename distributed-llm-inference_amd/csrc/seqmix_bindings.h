@@ -220,7 +220,7 @@ const void* head_gate(const c10::optional<Tensor>& gate, const Tensor& q1, int64
 
 // masks, soft cap, value sharing and result type of an attention launch (ops/seqmix.py: token_attention)
 dli::AttnOpts attn_opts(const Tensor& out, const Tensor& q1, int64_t G, int64_t window, int64_t chunk, int64_t keep, double cap, int64_t Gv,
-                        bool values, double out_scale) {
+                        bool values, double out_scale, const c10::optional<Tensor>& lam, double eps) {
   TORCH_CHECK(window >= 0 && chunk >= 0 && keep >= 0 && cap >= 0.0, "window, chunk, kept tokens and cap cannot be negative");
   TORCH_CHECK(!(window > 0 && chunk > 0) && (keep == 0 || window > 0), "a chunk excludes a window, kept tokens come with one");
   TORCH_CHECK(Gv > 0 && G % Gv == 0 && (values || Gv == G), "value heads must divide the key heads");
@@ -230,6 +230,11 @@ dli::AttnOpts attn_opts(const Tensor& out, const Tensor& q1, int64_t G, int64_t 
   o.cap = (float)cap;
   o.vshare = (int)(G / Gv);
   o.out_scale = (float)out_scale;
+  if (lam.has_value()) {
+    TORCH_CHECK(q1.size(1) == 2 * out.size(1) && G % 2 == 0 && Gv == G / 2 && out.scalar_type() == q1.scalar_type(), "two maps: pairs of query / key heads");
+    o.lam = opt_f32(lam, "lam", 1);
+    o.eps = (float)eps;
+  }
   o.out_f32 = out.scalar_type() == at::kFloat && q1.scalar_type() != at::kFloat ? out.data_ptr<float>() : nullptr;
   return o;
 }
@@ -239,7 +244,7 @@ void sm_token_attention(Tensor out, const Tensor& q1, const c10::optional<Tensor
                         const Tensor& token_seq, int64_t G, int64_t Dv, double scale, int64_t window, const c10::optional<Tensor>& temp,
                         const c10::optional<Tensor>& r1, const c10::optional<Tensor>& r2, int64_t rows,
                         const c10::optional<Tensor>& gate, const c10::optional<Tensor>& sink, int64_t chunk, int64_t keep, double cap,
-                        int64_t Gv, double out_scale) {
+                        int64_t Gv, double out_scale, const c10::optional<Tensor>& lam, double eps) {
   const bool bf = act_bf16(q1, "q1");
   TORCH_CHECK(q1.dim() == 3 && q1.stride(2) == 1, "q1 must be [T, H, D1] with a contiguous last dim");
   TORCH_CHECK(rows < 0 || rows <= q1.size(0), "rows past the batch");
@@ -265,28 +270,29 @@ void sm_token_attention(Tensor out, const Tensor& q1, const c10::optional<Tensor
   }
   TORCH_CHECK(Dv > 0 && Dv <= 8192, "value size must be in 1..8192");
   TORCH_CHECK(out.is_cuda() && (out.scalar_type() == q1.scalar_type() || out.scalar_type() == at::kFloat) && out.dim() == 3 && out.stride(2) == 1 && out.size(0) == T &&
-                  out.size(1) == H && out.size(2) == Dv, "out must be [T, H, Dv]");
+                  out.size(1) == (lam.has_value() ? H / 2 : H) && out.size(2) == Dv, "out must be [T, H, Dv] (two maps: [T, H / 2, Dv])");
   check_i32(block_tables, "block_tables");
   check_i32(positions, "positions");
   check_i32(token_seq, "token_seq");
   TORCH_CHECK(block_tables.dim() == 2 && positions.numel() >= T && token_seq.numel() >= T, "step metadata shorter than the batch");
   TORCH_CHECK(r1.has_value() == r2.has_value(), "r1 and r2 come together");
   TORCH_CHECK((Dk + 4 * std::min<int64_t>(Dv, 512) + 8) * 4 <= kSmMaxLds, "head sizes exceed the kernel's LDS budget");
-  dli::AttnOpts opt = attn_opts(out, q1, G, window, chunk, keep, cap, Gv, v_cache.has_value(), out_scale);
+  dli::AttnOpts opt = attn_opts(out, q1, G, window, chunk, keep, cap, Gv, v_cache.has_value(), out_scale, lam, eps);
+  if (lam.has_value()) TORCH_CHECK(!gate.has_value() && !sink.has_value() && Dv <= 512, "two maps: plain softmaxes, values up to 512");
   int64_t g_ts = 0;
   const void* gp = head_gate(gate, q1, T, H, &g_ts);
   // few rows (decode steps): long key ranges are cut over several workgroups, partial results in `part`
   const int64_t n_rows = rows < 0 ? T : rows;
   const int nsplit = Dv > 512 ? 1 : dli::sm_token_attention_splits((int)n_rows, (int)H, (int)G);
   Tensor part;
-  if (nsplit > 1) part = at::empty({n_rows, H, nsplit, Dv + 2}, q1.options().dtype(at::kFloat));
+  if (nsplit > 1 || lam.has_value()) part = at::empty({n_rows, H, nsplit, Dv + 2}, q1.options().dtype(at::kFloat));
   dli::launch_sm_token_attention(out.data_ptr(), out.stride(0), out.stride(1), q1.data_ptr(), q1.stride(0), q1.stride(1), (int)D1,
                                  q2.has_value() ? q2->data_ptr() : nullptr, q2.has_value() ? q2->stride(0) : 0,
                                  q2.has_value() ? q2->stride(1) : 0, (int)D2, k_cache.data_ptr(), (int)(G * Dk), vc.data_ptr(),
                                  (int)vc.size(2), (int)vhead, (int)Dv, block_tables.data_ptr<int>(), (int)block_tables.size(1),
                                  positions.data_ptr<int>(), token_seq.data_ptr<int>(), (int)n_rows, (int)H, (int)G, (float)scale,
                                  (int)window, opt_f32(temp, "temp", H), opt_f32(r1, "r1", H), opt_f32(r2, "r2", H), bf, nsplit,
-                                 nsplit > 1 ? part.data_ptr<float>() : nullptr, gp, g_ts, opt_f32(sink, "sink", H), opt, cur_stream(q1));
+                                 part.defined() ? part.data_ptr<float>() : nullptr, gp, g_ts, opt_f32(sink, "sink", H), opt, cur_stream(q1));
 }
 
 // Decode rows (the first `rows` tokens) of a mixer whose heads share key / value heads in groups of 8 or more, heads as the
@@ -296,7 +302,7 @@ bool sm_head_decode_attention(Tensor out, const Tensor& q1, const c10::optional<
                               const Tensor& token_seq, int64_t G, int64_t Dv, double scale, int64_t window,
                               const c10::optional<Tensor>& temp, const c10::optional<Tensor>& r1, const c10::optional<Tensor>& r2,
                               int64_t rows, const c10::optional<Tensor>& gate, const c10::optional<Tensor>& sink, int64_t chunk, int64_t keep, double cap,
-                        int64_t Gv, double out_scale) {
+                        int64_t Gv, double out_scale, const c10::optional<Tensor>& lam, double eps) {
   TORCH_CHECK(q1.is_cuda() && q1.scalar_type() == at::kBFloat16 && q1.dim() == 3 && q1.stride(2) == 1, "q1 must be bfloat16 [T, H, D1]");
   const int64_t T = q1.size(0), H = q1.size(1), D1 = q1.size(2);
   TORCH_CHECK(rows >= 0 && rows <= T, "rows past the batch");
@@ -320,25 +326,26 @@ bool sm_head_decode_attention(Tensor out, const Tensor& q1, const c10::optional<
     TORCH_CHECK(Dv <= Dk, "values read from the key rows cannot be wider than a key");
   }
   TORCH_CHECK(out.is_cuda() && (out.scalar_type() == at::kBFloat16 || out.scalar_type() == at::kFloat) && out.dim() == 3 && out.stride(2) == 1 && out.size(0) == T &&
-                  out.size(1) == H && out.size(2) == Dv, "out must be [T, H, Dv]");
+                  out.size(1) == (lam.has_value() ? H / 2 : H) && out.size(2) == Dv, "out must be [T, H, Dv] (two maps: [T, H / 2, Dv])");
   check_i32(block_tables, "block_tables");
   check_i32(positions, "positions");
   check_i32(token_seq, "token_seq");
   TORCH_CHECK(block_tables.dim() == 2 && positions.numel() >= T && token_seq.numel() >= T, "step metadata shorter than the batch");
   TORCH_CHECK(r1.has_value() == r2.has_value(), "r1 and r2 come together");
-  dli::AttnOpts opt = attn_opts(out, q1, G, window, chunk, keep, cap, Gv, v_cache.has_value(), out_scale);
+  dli::AttnOpts opt = attn_opts(out, q1, G, window, chunk, keep, cap, Gv, v_cache.has_value(), out_scale, lam, eps);
+  if (lam.has_value()) TORCH_CHECK(!gate.has_value() && !sink.has_value() && Dv <= 512, "two maps: plain softmaxes, values up to 512");
   int64_t g_ts = 0;
   const void* gp = head_gate(gate, q1, T, H, &g_ts);
   const int nsplit = dli::sm_head_decode_splits((int)rows, (int)H, (int)G);
   Tensor part;
-  if (nsplit > 1) part = at::empty({std::max<int64_t>(rows, 1), H, nsplit, Dv + 2}, q1.options().dtype(at::kFloat));
+  if (nsplit > 1 || lam.has_value()) part = at::empty({std::max<int64_t>(rows, 1), H, nsplit, Dv + 2}, q1.options().dtype(at::kFloat));
   return dli::launch_sm_head_decode_attention(out.data_ptr(), out.stride(0), out.stride(1), q1.data_ptr(), q1.stride(0), q1.stride(1),
                                               (int)D1, q2.has_value() ? q2->data_ptr() : nullptr, q2.has_value() ? q2->stride(0) : 0,
                                               q2.has_value() ? q2->stride(1) : 0, (int)D2, k_cache.data_ptr(), (int)(G * Dk),
                                               vc.data_ptr(), (int)vc.size(2), (int)vhead, (int)Dv, block_tables.data_ptr<int>(),
                                               (int)block_tables.size(1), positions.data_ptr<int>(), token_seq.data_ptr<int>(), (int)rows,
                                               (int)H, (int)G, (float)scale, (int)window, opt_f32(temp, "temp", H), opt_f32(r1, "r1", H),
-                                              opt_f32(r2, "r2", H), nsplit, nsplit > 1 ? part.data_ptr<float>() : nullptr, gp, g_ts, opt_f32(sink, "sink", H), opt,
+                                              opt_f32(r2, "r2", H), nsplit, part.defined() ? part.data_ptr<float>() : nullptr, gp, g_ts, opt_f32(sink, "sink", H), opt,
                                               cur_stream(q1));
 }
 
@@ -373,8 +380,6 @@ bool sm_tile_attention(Tensor out, const Tensor& q1, const c10::optional<Tensor>
   }
   TORCH_CHECK(out.is_cuda() && (out.scalar_type() == at::kBFloat16 || out.scalar_type() == at::kFloat) && out.dim() == 3 && out.stride(2) == 1 && out.size(0) == T &&
                   out.size(1) == (lam.has_value() ? H / 2 : H) && out.size(2) == Dv, "out must be [T, H, Dv] (two maps: [T, H / 2, Dv])");
-  if (lam.has_value()) TORCH_CHECK(H == 2 * out.size(1) && G % 2 == 0 && Gv == G / 2 && out.scalar_type() == at::kBFloat16 && !gate.has_value() &&
-                                       !sink.has_value() && !r1.has_value(), "two maps: pairs of plain bfloat16 query / key heads");
   check_i32(block_tables, "block_tables");
   check_i32(seq_lens, "seq_lens");
   check_i32(qsl, "query_start_loc");
@@ -389,9 +394,8 @@ bool sm_tile_attention(Tensor out, const Tensor& q1, const c10::optional<Tensor>
     cnt = counts->data_ptr<int>();
   }
   TORCH_CHECK(r1.has_value() == r2.has_value(), "r1 and r2 come together");
-  dli::AttnOpts opt = attn_opts(out, q1, G, window, chunk, keep, cap, Gv, v_cache.has_value(), out_scale);
-  opt.lam = opt_f32(lam, "lam", 1);
-  opt.eps = (float)eps;
+  dli::AttnOpts opt = attn_opts(out, q1, G, window, chunk, keep, cap, Gv, v_cache.has_value(), out_scale, lam, eps);
+  if (lam.has_value()) TORCH_CHECK(!gate.has_value() && !sink.has_value() && Dv <= 512, "two maps: plain softmaxes, values up to 512");
   int64_t g_ts = 0;
   const void* gp = head_gate(gate, q1, T, H, &g_ts);
   return dli::launch_sm_tile_attention(out.data_ptr(), out.stride(0), out.stride(1), q1.data_ptr(), q1.stride(0), q1.stride(1), (int)D1,

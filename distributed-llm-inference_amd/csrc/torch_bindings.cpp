@@ -604,11 +604,13 @@ TORCH_LIBRARY(dli, m) {
         "Tensor slot_mapping, Tensor(b!) cache, int H, int D, int R, int C) -> ()", &sm_latent_prep);
   m.def("sm_token_attention(Tensor(a!) out, Tensor q1, Tensor? q2, Tensor k_cache, Tensor? v_cache, Tensor block_tables, "
         "Tensor positions, Tensor token_seq, int G, int Dv, float scale, int window, Tensor? temp, Tensor? r1, Tensor? r2, int rows, "
-        "Tensor? gate, Tensor? sink, int chunk, int keep, float cap, int Gv, float out_scale) -> ()",
+        "Tensor? gate, Tensor? sink, int chunk, int keep, float cap, int Gv, float out_scale, "
+        "Tensor? lam=None, float eps=0.0) -> ()",
         &sm_token_attention);
   m.def("sm_head_decode_attention(Tensor(a!) out, Tensor q1, Tensor? q2, Tensor k_cache, Tensor? v_cache, Tensor block_tables, "
         "Tensor positions, Tensor token_seq, int G, int Dv, float scale, int window, Tensor? temp, Tensor? r1, Tensor? r2, int rows, "
-        "Tensor? gate, Tensor? sink, int chunk, int keep, float cap, int Gv, float out_scale) -> bool",
+        "Tensor? gate, Tensor? sink, int chunk, int keep, float cap, int Gv, float out_scale, "
+        "Tensor? lam=None, float eps=0.0) -> bool",
         &sm_head_decode_attention);
   m.def("sm_tile_attention(Tensor(a!) out, Tensor q1, Tensor? q2, Tensor k_cache, Tensor? v_cache, Tensor block_tables, Tensor seq_lens, "
         "Tensor qsl, Tensor tile_seq, Tensor tile_q0, int num_tiles, Tensor? counts, int G, int Dv, float scale, int window, "

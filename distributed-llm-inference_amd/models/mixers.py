@@ -1196,7 +1196,10 @@ class PostNormLayer(nn.Module):
         """``x``: fp32 stream ``[T, W]``, updated in place; ``h``: the same in the model dtype.  Returns the new ``x`` in the model dtype, or
         its norm with the weight ``final_norm`` (the stack's last layer)."""
         proj = ops.linear(h, self.inp.data)
-        acts = torch.zeros(h.shape[0], self.mixer.out_cols, dtype=h.dtype, device=h.device)      # padding rows of a captured step stay zero
+        # padding rows of a captured step are zeros: the kernels of pure decode steps write them, prefill tiles leave them out
+        acts = torch.empty(h.shape[0], self.mixer.out_cols, dtype=h.dtype, device=h.device)
+        if meta.num_prefill_tiles and meta.counts_on_device:
+            acts.zero_()
         self.mixer(proj[:, :self.mixer.in_cols], acts, meta, cache)
         h = seqmix.post_norm_add(x, ops.linear(acts, self.out.data), self.norm1.data, self.eps, self.dtype,
                                  final_norm if self.ff is None else None)

@@ -1054,20 +1054,23 @@ def map_attention(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v_c
     head of its group), key rows ``[G, 2, D]``), combined by ``map_combine`` into ``out [T, H·Dv]``.  Prefill tiles do both maps and the
     combination in one kernel."""
     T, H2, _D = q.shape
-    rows = T
     if _act_ok(q):
         lib = _hip()
+        out3 = out.unflatten(1, (H2 // 2, Dv))
         args, opts = (2 * G, Dv, scale, window, None, None, None), (None, None, 0, 0, 0.0, G)
+        rows = -1
         if TILE_ATTENTION and q.dtype == torch.bfloat16 and meta.num_prefill_tiles > 0:
-            if lib.sm_tile_attention(out.unflatten(1, (H2 // 2, Dv)), q, None, k_cache, v_cache, meta.block_tables, meta.seq_lens,
-                                     meta.query_start_loc, meta.prefill_tile_seq, meta.prefill_tile_q0, meta.num_prefill_tiles,
+            if lib.sm_tile_attention(out3, q, None, k_cache, v_cache, meta.block_tables, meta.seq_lens, meta.query_start_loc,
+                                     meta.prefill_tile_seq, meta.prefill_tile_q0, meta.num_prefill_tiles,
                                      meta.counts if meta.counts_on_device else None, *args, *opts, out_scale, lam, eps):
                 rows = meta.num_decode
-        if rows == 0:
-            return
-        o = torch.empty(rows, H2, Dv, dtype=torch.float32, device=out.device)
-        _attend_rows(lib, o, q[:rows], None, k_cache, v_cache, meta, rows if rows < T else -1, args, (*opts, 1.0))
-        map_combine(o, lam, eps, out_scale, G, out[:rows], meta.token_seq)
+        if Dv <= 512:
+            _attend_rows(lib, out3, q, None, k_cache, v_cache, meta, rows, args, (*opts, out_scale, lam, eps))
+        elif rows != 0:                                      # wider values run in slabs: both maps in fp32, then their difference
+            o = torch.empty(T, H2, Dv, dtype=torch.float32, device=out.device)
+            _attend_rows(lib, o, q, None, k_cache, v_cache, meta, rows, args, (*opts, 1.0))
+            n = T if rows < 0 else rows
+            map_combine(o[:n], lam, eps, out_scale, G, out[:n], meta.token_seq)
         return
     o = torch.empty(T, H2, Dv)
     token_attention(o, q, None, k_cache, v_cache, meta, 2 * G, Dv, scale, window, value_heads=G)
