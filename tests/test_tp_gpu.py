@@ -210,7 +210,7 @@ def _replay_http(tmp_path, extra):
 
 @pytest.mark.parametrize("model,tp,extra", [("tiny-llama-tp", 2, []), ("tiny-llama-tp8", 8, []),
                                             pytest.param("llama3-70b", 2, ["--server-args", "--num-layers 2 --num-kv-blocks 2048"],
-                                                         marks=pytest.mark.skip(reason="two ranks of this size sharing one card: a run stalled for "
+                                                         marks=pytest.mark.skip(reason="two ranks of this size sharing one GPU: a run stalled for "
                                                                                 "more than 120 s (usually about 20 s), cause not found"))])
 def test_http_replay_against_tp_server_on_gpu(model, tp, extra, tmp_path):
     """harness → HTTP → api_server --tp N, the ranks joined through launch.bootstrap (probe child,
